@@ -16,6 +16,7 @@
 // dv: the values' head size (the keys' is dh); out is [n, nh * dv].
 // sinks (may be null): a number per head that stands in the softmax's denominator as exp(sink[h]) beside the keys'
 // terms; it has no key, no value, no scale and no bias, and counts once for every query.
+// softcap (0: none): a scaled score s becomes softcap * tanh(s / softcap), before any bias.
 #include "common.h"
 #include "kv_layout.h"
 
@@ -28,7 +29,7 @@ paged_attention_generic_kernel(const T *__restrict__ q, int q_stride, T *__restr
                                const int *__restrict__ q_start, const int *__restrict__ ctx_len,
                                const int *__restrict__ req_of_token, int nh, int nkvh, int dh, int dv, int page,
                                float scale, int window, int chunk, const float *__restrict__ head_slopes,
-                               const float *__restrict__ sinks) {
+                               const float *__restrict__ sinks, float softcap) {
     const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
     const int r = req_of_token[t];
     const int p = ctx_len[r] - (q_start[r + 1] - t);
@@ -62,7 +63,9 @@ paged_attention_generic_kernel(const T *__restrict__ q, int q_stride, T *__restr
 #pragma unroll
                 for (int e = 0; e < 8; ++e) acc += qs[c8 * 8 + e] * to_f32(kk[e]);
             }
-            s = acc * scale + slope * (float)(j - p);
+            acc *= scale;
+            if (softcap > 0.f) acc = softcap * tanhf(acc / softcap);
+            s = acc + slope * (float)(j - p);
         }
         const float m_new = fmaxf(m, wave_max(s));
         const float pj = valid ? expf(s - m_new) : 0.f;
@@ -110,13 +113,13 @@ LCU_API int lcu_paged_attention_generic(const void *q, int q_stride, void *out, 
                                         const void *cache, const int *block_table, int max_pages,
                                         const int *q_start, const int *ctx_len, const int *req_of_token, int n,
                                         int nh, int nkvh, int dh, int dv, int page, float scale, int window,
-                                        int chunk, const float *head_slopes, const float *sinks, hipStream_t stream) {
+                                        int chunk, const float *head_slopes, const float *sinks, float softcap, hipStream_t stream) {
     if (n <= 0) return LCU_OK;
     if (nh <= 0 || nkvh <= 0 || nh % nkvh || dh <= 0 || dh % 8 || dh > MAX_HEAD_DIM || dv <= 0 || dv > MAX_HEAD_DIM || page <= 0 || page % 8 ||
-        max_pages <= 0 || window < 0 || chunk < 0 || (window > 0 && chunk > 0) || nh > 65535)
+        max_pages <= 0 || window < 0 || chunk < 0 || (window > 0 && chunk > 0) || nh > 65535 || softcap < 0.f)
         return LCU_BAD_ARGUMENT;
     dim3 grid(n, nh), block(WAVE);
-#define GO(T, NV) paged_attention_generic_kernel<T, NV><<<grid, block, 0, stream>>>((const T *)q, q_stride, (T *)out, out_stride, (const T *)cache, block_table, max_pages, q_start, ctx_len, req_of_token, nh, nkvh, dh, dv, page, scale, window, chunk, head_slopes, sinks)
+#define GO(T, NV) paged_attention_generic_kernel<T, NV><<<grid, block, 0, stream>>>((const T *)q, q_stride, (T *)out, out_stride, (const T *)cache, block_table, max_pages, q_start, ctx_len, req_of_token, nh, nkvh, dh, dv, page, scale, window, chunk, head_slopes, sinks, softcap)
     if (type == LCU_F32) { if (dv <= 256) GO(float, 4); else GO(float, 10); }
     else if (type == LCU_BF16) { if (dv <= 256) GO(bf16_t, 4); else GO(bf16_t, 10); }
     else return LCU_BAD_ARGUMENT;

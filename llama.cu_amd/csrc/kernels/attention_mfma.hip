@@ -60,11 +60,18 @@ __device__ __forceinline__ f32x4 mfma16(u32x4 a, u32x4 b, f32x4 c) {
 // The same library takes sinks [nh] (may be null) behind the slopes: exp(sink[h]) stands in the denominator of every
 // softmax of head h beside the keys' terms, with no key, value, scale or bias.  It enters where a row's sum is
 // final (sink_share below): once, also where a request's keys were walked in parts.
+//
+// LCU_SCORE_CAP (a third library): every kernel takes a cap on the scores: a scaled score s becomes cap * tanh(s / cap).
+// Inside the kernels a score then stands in units of log2 (the scale is in the cap's constants), so the code behind
+// it multiplies by a scale of 1: SCORE_LOG2.
+#if defined(LCU_SCORE_BIAS) && defined(LCU_SCORE_CAP)
+#error "a bias and a cap together are not built"
+#endif
 #ifdef LCU_SCORE_BIAS
-#define BIAS_KPARAMS , const float *__restrict__ head_slopes, float inv_scale, const float *__restrict__ sinks
-#define BIAS_KARGS(scale) , head_slopes, 1.0f / (scale), sinks
-#define BIAS_PARAMS , const float *head_slopes, const float *sinks
-#define BIAS_ARGS , head_slopes, sinks
+#define SCORE_KPARAMS , const float *__restrict__ head_slopes, float inv_scale, const float *__restrict__ sinks
+#define SCORE_KARGS(scale) , head_slopes, 1.0f / (scale), sinks
+#define SCORE_PARAMS , const float *head_slopes, const float *sinks
+#define SCORE_ARGS , head_slopes, sinks
 #define MERGE_SINKS sinks
 // A row whose keys gave the sum l of 2^(score - m) takes in its sink: returns the factor for the row's
 // unnormalised output, 2^(m - m') / (l 2^(m - m') + 2^(sink log2(e) - m')) with m' = max(m, sink log2(e)).
@@ -73,12 +80,26 @@ __device__ __forceinline__ float sink_share(float m, float l, float sink) {
     const float keep = exp2f(m - m_all);                 // (m = -inf, no key at all: 0)
     return keep / (l * keep + exp2f(sk - m_all));
 }
-#else
+#define SCORE_LOG2(scale) ((scale) * 1.4426950408889634f)
+#elif defined(LCU_SCORE_CAP)
+#define SCORE_KPARAMS , float cap_in, float cap_out
+#define SCORE_KARGS(scale) , 2.0f * 1.4426950408889634f * (scale) / softcap, softcap * 1.4426950408889634f
+#define SCORE_PARAMS , float softcap
+#define SCORE_ARGS , softcap
 #define MERGE_SINKS nullptr
-#define BIAS_KPARAMS
-#define BIAS_KARGS(scale)
-#define BIAS_PARAMS
-#define BIAS_ARGS
+#define SCORE_LOG2(scale) 1.0f
+// cap tanh(s / cap) log2(e) of the raw score x: tanh(y) = 1 - 2 / (1 + e^(2 y)), e^(2 y) = 2^(cap_in x), cap_out = cap log2(e).
+// (An error of some 1e-7 of the cap; both ends are exact: 2^inf gives the cap, 2^-inf its negative.)
+__device__ __forceinline__ float capped(float x, float cap_in, float cap_out) {
+    return fmaf(-2.0f * cap_out, __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(cap_in * x)), cap_out);
+}
+#else
+#define SCORE_LOG2(scale) ((scale) * 1.4426950408889634f)
+#define MERGE_SINKS nullptr
+#define SCORE_KPARAMS
+#define SCORE_KARGS(scale)
+#define SCORE_PARAMS
+#define SCORE_ARGS
 #endif
 
 // What a wave carries through its keys, for QB blocks of 16 rows.
@@ -89,6 +110,9 @@ struct AttnState {
     float l[QB];            // running sum over the lane's own keys only
 #ifdef LCU_SCORE_BIAS
     float bias[QB];         // of the lane's row: slope of its head / scale
+#endif
+#ifdef LCU_SCORE_CAP
+    float cap_in, cap_out;
 #endif
 };
 
@@ -229,6 +253,10 @@ __device__ __forceinline__ void attn_softmax(const f32x4 (&s)[QB][2], int k0, At
 #pragma unroll
         for (int r = 0; r < 8; ++r) v[r] = fmaf(st.bias[b], (float)(k0 + 16 * (r / 4) + 4 * grp + (r % 4) - p_row[b]), v[r]);
 #endif
+#ifdef LCU_SCORE_CAP
+#pragma unroll
+        for (int r = 0; r < 8; ++r) v[r] = capped(v[r], st.cap_in, st.cap_out);
+#endif
         if (MASK) {
 #pragma unroll
             for (int r = 0; r < 8; ++r) {
@@ -331,7 +359,7 @@ attention_decode_kernel(const bf16_t *__restrict__ q, int q_stride, bf16_t *__re
                         const bf16_t *__restrict__ cache, const int *__restrict__ block_table, int max_pages,
                         const int *__restrict__ q_start, const int *__restrict__ ctx_len,
                         const int *__restrict__ req_list, int nh, int nkvh, int page, float scale_log2, int window,
-                        int n_splits, float *__restrict__ part_o, float *__restrict__ part_ml BIAS_KPARAMS) {
+                        int n_splits, float *__restrict__ part_o, float *__restrict__ part_ml SCORE_KPARAMS) {
     extern __shared__ float lds[];                 // [waves][16][DH] outputs, then [waves][16][2] (m, l)
     const int g = nh / nkvh;
     const int chunks = (g + 15) / 16;
@@ -356,6 +384,10 @@ attention_decode_kernel(const bf16_t *__restrict__ q, int q_stride, bf16_t *__re
     attn_init(st);
 #ifdef LCU_SCORE_BIAS
     st.bias[0] = l16 < rows ? head_slopes[head0 + l16] * inv_scale : 0.f;
+#endif
+#ifdef LCU_SCORE_CAP
+    st.cap_in = cap_in;
+    st.cap_out = cap_out;
 #endif
     const int p_row[1] = {p}, lo_row[1] = {lo};
     const int *bt = block_table + (size_t)r * max_pages;
@@ -500,9 +532,9 @@ template <int DH>
 static int launch_decode(const void *q, int q_stride, void *out, int out_stride, const void *cache,
                          const int *block_table, int max_pages, const int *q_start, const int *ctx_len,
                          const int *req_list, int n_req, int nh, int nkvh, int page, float scale, int window,
-                         int n_splits, float *part_o, float *part_ml, hipStream_t stream BIAS_PARAMS) {
+                         int n_splits, float *part_o, float *part_ml, hipStream_t stream SCORE_PARAMS) {
     const int g = nh / nkvh, chunks = (g + 15) / 16;
-    const float scale_log2 = scale * 1.4426950408889634f;
+    const float scale_log2 = SCORE_LOG2(scale);
     const size_t lds_bytes = (size_t)DEC_WAVES * 16 * (DH + 2) * sizeof(float);
     dim3 grid(n_req * nkvh * chunks, n_splits), block(DEC_WAVES * WAVE);
     // Two ways to address the pages (the same arithmetic, the same results).  FLAT: every lane holds
@@ -514,7 +546,7 @@ static int launch_decode(const void *q, int q_stride, void *out, int out_stride,
     const bool flat = n_splits == 1;
     (flat ? attention_decode_kernel<DH, true> : attention_decode_kernel<DH, false>)<<<grid, block, lds_bytes, stream>>>(
         (const bf16_t *)q, q_stride, (bf16_t *)out, out_stride, (const bf16_t *)cache, block_table, max_pages, q_start,
-        ctx_len, req_list, nh, nkvh, page, scale_log2, window, n_splits, part_o, part_ml BIAS_KARGS(scale));
+        ctx_len, req_list, nh, nkvh, page, scale_log2, window, n_splits, part_o, part_ml SCORE_KARGS(scale));
     LCU_LAUNCH_CHECK();
     if (n_splits > 1) {
         attention_merge_kernel<DH><<<dim3(n_req, nh), dim3(DH / 4), 0, stream>>>((bf16_t *)out, out_stride, part_o, part_ml,
@@ -542,15 +574,18 @@ static int decode_arguments(int q_stride, int out_stride, int max_pages, int nh,
 LCU_API int lcu_attention_decode_bf16(const void *q, int q_stride, void *out, int out_stride, const void *cache,
                                       const int *block_table, int max_pages, const int *q_start, const int *ctx_len,
                                       const int *req_list, int n_req, int nh, int nkvh, int dh, int page, float scale,
-                                      int window, int n_splits, float *part_o, float *part_ml, hipStream_t stream BIAS_PARAMS) {
+                                      int window, int n_splits, float *part_o, float *part_ml, hipStream_t stream SCORE_PARAMS) {
     if (n_req <= 0) return LCU_OK;
 #ifdef LCU_SCORE_BIAS
     if (!head_slopes || !(scale > 0.f)) return LCU_BAD_ARGUMENT;
 #endif
+#ifdef LCU_SCORE_CAP
+    if (!(softcap > 0.f)) return LCU_BAD_ARGUMENT;
+#endif
     const int args = decode_arguments(q_stride, out_stride, max_pages, nh, nkvh, dh, page, window, n_splits);
     if (args != LCU_OK) return args;
     if (n_splits > 1 && (!part_o || !part_ml)) return LCU_BAD_ARGUMENT;
-#define GO(D) return launch_decode<D>(q, q_stride, out, out_stride, cache, block_table, max_pages, q_start, ctx_len, req_list, n_req, nh, nkvh, page, scale, window, n_splits, part_o, part_ml, stream BIAS_ARGS)
+#define GO(D) return launch_decode<D>(q, q_stride, out, out_stride, cache, block_table, max_pages, q_start, ctx_len, req_list, n_req, nh, nkvh, page, scale, window, n_splits, part_o, part_ml, stream SCORE_ARGS)
     if (dh == 128) GO(128);
     if (dh == 64) GO(64);
     if (dh == 96) GO(96);
@@ -603,8 +638,8 @@ LCU_API int lcu_attention_decode_bf16_static(const void *q, int q_stride, void *
                                              const int *block_table, int max_pages, const int *q_start, const int *ctx_len,
                                              const int *req_list, int n_req, int nh, int nkvh, int dh, int page, float scale,
                                              int window, int n_splits, hipStream_t stream) {
-#ifdef LCU_SCORE_BIAS
-    return LCU_UNSUPPORTED;        // (this entry point takes no slopes: the library with the bias has no such caller)
+#if defined(LCU_SCORE_BIAS) || defined(LCU_SCORE_CAP)
+    return LCU_UNSUPPORTED;        // (this entry point takes no slopes and no cap: those libraries have no such caller)
 #else
     if (n_req <= 0) return LCU_OK;
     // the arguments first, as the other entry point checks them: a call with bad sizes is told so, whatever
@@ -667,6 +702,9 @@ struct PrefillState {
     float l;                // running sum over the lane's own keys only
 #ifdef LCU_SCORE_BIAS
     float bias;             // of the lane's row: slope of its head / scale (0 for a row that is nobody's)
+#endif
+#ifdef LCU_SCORE_CAP
+    float cap_in, cap_out;
 #endif
 };
 
@@ -900,6 +938,10 @@ __device__ __forceinline__ void attn_turn(const u32x4 *__restrict__ next, u32x4 
         for (int i = 0; i < 16; ++i) x[i] = fmaf(st.bias, (float)(16 * (i / 8) + i % 8 - last0), x[i]);
     }
 #endif
+#ifdef LCU_SCORE_CAP
+#pragma unroll
+    for (int i = 0; i < 16; ++i) x[i] = capped(x[i], st.cap_in, st.cap_out);
+#endif
     if (mask) {
         // a lane's score i is key k0 + 8 hi + c with c = 16 (i / 8) + i % 8: compared as c against the bounds less k0 + 8 hi
         const int last = p_row - k0 - 8 * hi, first = lo_row - k0 - 8 * hi;
@@ -969,7 +1011,7 @@ attention_prefill_kernel(const bf16_t *__restrict__ q, int q_stride, bf16_t *__r
                            const int *__restrict__ q_start, const int *__restrict__ ctx_len,
                            const int *__restrict__ task_req, const int *__restrict__ task_tok0, int max_tasks,
                            const int *__restrict__ n_tasks_dev,
-                           int tasks_per_wg, int nh, int nkvh, int page, uint32_t tile_magic, float scale_log2, int window BIAS_KPARAMS) {
+                           int tasks_per_wg, int nh, int nkvh, int page, uint32_t tile_magic, float scale_log2, int window SCORE_KPARAMS) {
     extern __shared__ u32x4 lds_ring[];            // [PRE_RING][8 * DH]
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / WAVE);
     const int lane = threadIdx.x & (WAVE - 1);
@@ -1026,6 +1068,10 @@ attention_prefill_kernel(const bf16_t *__restrict__ q, int q_stride, bf16_t *__r
     st.l = 0.f;
 #ifdef LCU_SCORE_BIAS
     st.bias = valid ? head_slopes[head0 + n % hc] * inv_scale : 0.f;
+#endif
+#ifdef LCU_SCORE_CAP
+    st.cap_in = cap_in;
+    st.cap_out = cap_out;
 #endif
 #pragma unroll
     for (int t = 0; t < DH / 32; ++t)
@@ -1121,7 +1167,7 @@ template <int DH, bool PAGE16, bool FLAT>
 static int launch_prefill_as(const void *q, int q_stride, void *out, int out_stride, const void *cache, uint32_t cache_bytes,
                              const int *block_table, int max_pages, const int *q_start, const int *ctx_len,
                              const int *task_req, const int *task_tok0, int n_tasks, const int *n_tasks_dev, int tasks_per_wg,
-                             int nh, int nkvh, int page, float scale, int window, hipStream_t stream BIAS_PARAMS) {
+                             int nh, int nkvh, int page, float scale, int window, hipStream_t stream SCORE_PARAMS) {
     const int g = nh / nkvh, chunks = (g + 15) / 16;
     const long long n_wg = (long long)((n_tasks + tasks_per_wg - 1) / tasks_per_wg) * nkvh * chunks;
     if (n_wg > 0x7fffffffll) return LCU_BAD_ARGUMENT;
@@ -1144,7 +1190,7 @@ static int launch_prefill_as(const void *q, int q_stride, void *out, int out_str
     attention_prefill_kernel<DH, PAGE16, FLAT><<<grid, block, lds_bytes, stream>>>(
         (const bf16_t *)q, q_stride, (bf16_t *)out, out_stride, (const bf16_t *)cache, cache_bytes, block_table, max_pages, q_start,
         ctx_len, task_req, task_tok0, n_tasks, n_tasks_dev, tasks_per_wg, nh, nkvh, page,
-        page == 16 ? 0u : (uint32_t)(0x100000000ull / (unsigned)(page / 16)) + 1u, scale * 1.4426950408889634f, window BIAS_KARGS(scale));
+        page == 16 ? 0u : (uint32_t)(0x100000000ull / (unsigned)(page / 16)) + 1u, SCORE_LOG2(scale), window SCORE_KARGS(scale));
     LCU_LAUNCH_CHECK();
     return LCU_OK;
 }
@@ -1154,10 +1200,10 @@ template <int DH>
 static int launch_prefill(const void *q, int q_stride, void *out, int out_stride, const void *cache, long long cache_pages,
                           const int *block_table, int max_pages, const int *q_start, const int *ctx_len,
                           const int *task_req, const int *task_tok0, int n_tasks, const int *n_tasks_dev, int tasks_per_wg,
-                          int nh, int nkvh, int page, float scale, int window, hipStream_t stream BIAS_PARAMS) {
+                          int nh, int nkvh, int page, float scale, int window, hipStream_t stream SCORE_PARAMS) {
     const unsigned long long bytes = (unsigned long long)cache_pages * kv_page_elems(nkvh, DH, page) * sizeof(bf16_t);
     const bool flat = bytes < (1ull << 32);
-#define AS(P, F) return launch_prefill_as<DH, P, F>(q, q_stride, out, out_stride, cache, (uint32_t)(F ? bytes : 0), block_table, max_pages, q_start, ctx_len, task_req, task_tok0, n_tasks, n_tasks_dev, tasks_per_wg, nh, nkvh, page, scale, window, stream BIAS_ARGS)
+#define AS(P, F) return launch_prefill_as<DH, P, F>(q, q_stride, out, out_stride, cache, (uint32_t)(F ? bytes : 0), block_table, max_pages, q_start, ctx_len, task_req, task_tok0, n_tasks, n_tasks_dev, tasks_per_wg, nh, nkvh, page, scale, window, stream SCORE_ARGS)
     if (page == 16) {
         if (flat) AS(true, true);
         AS(true, false);
@@ -1186,16 +1232,19 @@ LCU_API int lcu_attention_prefill_bf16(const void *q, int q_stride, void *out, i
                                        long long cache_pages, const int *block_table, int max_pages, const int *q_start, const int *ctx_len,
                                        const int *task_req, const int *task_tok0, int n_tasks, const int *n_tasks_dev,
                                        int tasks_per_wg, int nh, int nkvh, int dh, int page, float scale, int window,
-                                       hipStream_t stream BIAS_PARAMS) {
+                                       hipStream_t stream SCORE_PARAMS) {
     if (n_tasks <= 0) return LCU_OK;
 #ifdef LCU_SCORE_BIAS
     if (!head_slopes || !(scale > 0.f)) return LCU_BAD_ARGUMENT;
+#endif
+#ifdef LCU_SCORE_CAP
+    if (!(softcap > 0.f)) return LCU_BAD_ARGUMENT;
 #endif
     if ((unsigned long long)kv_page_elems(nkvh, dh, page) * 2ull >= (1ull << 31)) return LCU_UNSUPPORTED;
     if (cache_pages <= 0 || tasks_per_wg < 1 || lcu_attention_prefill_tokens_per_task(nh, nkvh) == 0 || page <= 0 || page % 16 || max_pages <= 0 ||
         q_stride % 8 || out_stride % 4 || nkvh * ((nh / nkvh + 15) / 16) > 65535)
         return LCU_BAD_ARGUMENT;
-#define GO(D) return launch_prefill<D>(q, q_stride, out, out_stride, cache, cache_pages, block_table, max_pages, q_start, ctx_len, task_req, task_tok0, n_tasks, n_tasks_dev, tasks_per_wg, nh, nkvh, page, scale, window, stream BIAS_ARGS)
+#define GO(D) return launch_prefill<D>(q, q_stride, out, out_stride, cache, cache_pages, block_table, max_pages, q_start, ctx_len, task_req, task_tok0, n_tasks, n_tasks_dev, tasks_per_wg, nh, nkvh, page, scale, window, stream SCORE_ARGS)
     if (dh == 128) GO(128);
     if (dh == 64) GO(64);
     if (dh == 96) GO(96);

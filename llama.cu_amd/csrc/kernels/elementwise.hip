@@ -2,6 +2,7 @@
 // sum, SwiGLU, residual add.  Sums, the norm and the activation are computed in
 // 32-bit whatever the storage type.
 #include "common.h"
+#include "gate_act.h"
 
 // ---------------------------------------------------------------- embedding gather
 // out[i, :] = table[ids[i], :] * scale (the product in 32-bit).  An id outside the table writes NaN into the row
@@ -79,12 +80,13 @@ LCU_API int lcu_gather_rows(void *out, const void *x, int type, const int *rows,
 // One block per row.  If `delta` is given: x += delta first (in 32-bit, written back
 // when x is 32-bit: x is then the residual stream); delta may be `planes` planes [n, d],
 // `plane_stride` elements apart (a product's partial sums over slices of K), which are added
-// one after the other in the order of the planes.  Then
+// one after the other in the order of the planes; every element of the branch's output enters
+// times `delta_scale` (1: as it is).  Then
 //   y = x * rsqrt(sum(x^2)/d + eps) * w        (32-bit, one rounding at the store)
 // The order of the sum depends on d and the block size only, not on the batch.
 template <class TX, class TD, class TW, class TO>
 __global__ void rmsnorm_kernel(TX *__restrict__ x, const TD *__restrict__ delta, const TW *__restrict__ w,
-                               TO *__restrict__ out, int d, float eps, int write_back, int planes, size_t plane_stride) {
+                               TO *__restrict__ out, int d, float eps, int write_back, int planes, size_t plane_stride, float delta_scale) {
     __shared__ float scratch[16];
     TX *xr = x + (size_t)blockIdx.x * d;
     const TD *dr = delta ? delta + (size_t)blockIdx.x * d : nullptr;
@@ -92,7 +94,7 @@ __global__ void rmsnorm_kernel(TX *__restrict__ x, const TD *__restrict__ delta,
     for (int c = threadIdx.x; c < d; c += blockDim.x) {
         float v = to_f32(xr[c]);
         if (dr) {
-            for (int p = 0; p < planes; ++p) v += to_f32(dr[p * plane_stride + c]);
+            for (int p = 0; p < planes; ++p) v = fmaf(delta_scale, to_f32(dr[p * plane_stride + c]), v);
             if (write_back) xr[c] = from_f32<TX>(v);
         }
         acc += v * v;
@@ -103,7 +105,7 @@ __global__ void rmsnorm_kernel(TX *__restrict__ x, const TD *__restrict__ delta,
     for (int c = threadIdx.x; c < d; c += blockDim.x) {
         float v = to_f32(xr[c]);
         if (dr && !write_back)
-            for (int p = 0; p < planes; ++p) v += to_f32(dr[p * plane_stride + c]);
+            for (int p = 0; p < planes; ++p) v = fmaf(delta_scale, to_f32(dr[p * plane_stride + c]), v);
         o[c] = from_f32<TO>(rms * v * to_f32(w[c]));
     }
 }
@@ -123,7 +125,7 @@ template <class T> struct alignas(4 * sizeof(T)) Vec4 { T v[4]; };
 template <int THREADS, class TX, class TD, class TW, class TO>
 __global__ void __launch_bounds__(THREADS)
 rmsnorm_fast_kernel(TX *__restrict__ x, const TD *__restrict__ delta, const TW *__restrict__ w, TO *__restrict__ out,
-                    int d, float eps, int write_back, int planes, size_t plane_stride) {
+                    int d, float eps, int write_back, int planes, size_t plane_stride, float delta_scale) {
     constexpr int PLAY = NORM_VTHREADS / THREADS;           // virtual threads per thread
     __shared__ float scratch[NORM_VTHREADS / WAVE];
     TX *xr = x + (size_t)blockIdx.x * d;
@@ -148,7 +150,7 @@ rmsnorm_fast_kernel(TX *__restrict__ x, const TD *__restrict__ delta, const TW *
                         for (int q = 0; q < 4; ++q)
                             if (p0 + q < planes) {
 #pragma unroll
-                                for (int e = 0; e < 4; ++e) v[j][i][e] += to_f32(dv[q].v[e]);
+                                for (int e = 0; e < 4; ++e) v[j][i][e] = fmaf(delta_scale, to_f32(dv[q].v[e]), v[j][i][e]);
                             }
                     }
                     Vec4<TX> back;
@@ -187,10 +189,10 @@ rmsnorm_fast_kernel(TX *__restrict__ x, const TD *__restrict__ delta, const TW *
 
 template <class TX, class TD, class TO>
 static int rmsnorm_w(void *x, const void *delta, const void *w, int w_type, void *out, int n, int d, float eps,
-                     int write_back, hipStream_t stream, int planes = 1, size_t plane_stride = 0) {
+                     int write_back, float delta_scale, hipStream_t stream, int planes = 1, size_t plane_stride = 0) {
     dim3 grid(n), block(d >= 2048 ? 512 : 256);
     if (d % 4 == 0 && d <= NORM_VTHREADS * NORM_ITEMS * 4) {
-#define FAST(T_, TW_) rmsnorm_fast_kernel<T_, TX, TD, TW_, TO><<<grid, dim3(T_), 0, stream>>>((TX *)x, (const TD *)delta, (const TW_ *)w, (TO *)out, d, eps, write_back, planes, plane_stride)
+#define FAST(T_, TW_) rmsnorm_fast_kernel<T_, TX, TD, TW_, TO><<<grid, dim3(T_), 0, stream>>>((TX *)x, (const TD *)delta, (const TW_ *)w, (TO *)out, d, eps, write_back, planes, plane_stride, delta_scale)
         const bool few = n <= 192;        // (measured with four planes: steps of 160 and 192 rows 2 % faster with 1024 threads, of 256 rows 1 % slower)
         if (w_type == LCU_F32) {
             if (few) FAST(1024, float); else FAST(256, float);
@@ -204,9 +206,9 @@ static int rmsnorm_w(void *x, const void *delta, const void *w, int w_type, void
         return LCU_OK;
     }
     if (w_type == LCU_F32)
-        rmsnorm_kernel<TX, TD, float, TO><<<grid, block, 0, stream>>>((TX *)x, (const TD *)delta, (const float *)w, (TO *)out, d, eps, write_back, planes, plane_stride);
+        rmsnorm_kernel<TX, TD, float, TO><<<grid, block, 0, stream>>>((TX *)x, (const TD *)delta, (const float *)w, (TO *)out, d, eps, write_back, planes, plane_stride, delta_scale);
     else if (w_type == LCU_BF16)
-        rmsnorm_kernel<TX, TD, bf16_t, TO><<<grid, block, 0, stream>>>((TX *)x, (const TD *)delta, (const bf16_t *)w, (TO *)out, d, eps, write_back, planes, plane_stride);
+        rmsnorm_kernel<TX, TD, bf16_t, TO><<<grid, block, 0, stream>>>((TX *)x, (const TD *)delta, (const bf16_t *)w, (TO *)out, d, eps, write_back, planes, plane_stride, delta_scale);
     else
         return LCU_BAD_ARGUMENT;
     LCU_LAUNCH_CHECK();
@@ -214,64 +216,94 @@ static int rmsnorm_w(void *x, const void *delta, const void *w, int w_type, void
 }
 
 // x: [n, d] of x_type (read; written when write_back and delta are set), delta: [n, d] of
-// act_type or null, out: [n, d] of act_type.
-LCU_API int lcu_rmsnorm(void *x, int x_type, const void *delta, const void *w, int w_type, void *out,
-                        int act_type, int n, int d, float eps, int write_back, hipStream_t stream) {
+// delta_type or null, out: [n, d] of act_type.  delta enters times delta_scale.
+LCU_API int lcu_rmsnorm(void *x, int x_type, const void *delta, int delta_type, const void *w, int w_type, void *out,
+                        int act_type, int n, int d, float eps, int write_back, float delta_scale, hipStream_t stream) {
     if (n <= 0) return LCU_OK;
     if (d <= 0) return LCU_BAD_ARGUMENT;
-    if (x_type == LCU_F32 && act_type == LCU_F32) return rmsnorm_w<float, float, float>(x, delta, w, w_type, out, n, d, eps, write_back, stream);
-    if (x_type == LCU_F32 && act_type == LCU_BF16) return rmsnorm_w<float, bf16_t, bf16_t>(x, delta, w, w_type, out, n, d, eps, write_back, stream);
-    if (x_type == LCU_BF16 && act_type == LCU_BF16) return rmsnorm_w<bf16_t, bf16_t, bf16_t>(x, delta, w, w_type, out, n, d, eps, write_back, stream);
+#define GO(TX, TD, TO) return rmsnorm_w<TX, TD, TO>(x, delta, w, w_type, out, n, d, eps, write_back, delta_scale, stream)
+    if (x_type == LCU_F32 && act_type == LCU_F32 && delta_type == LCU_F32) GO(float, float, float);
+    if (x_type == LCU_F32 && act_type == LCU_F32 && delta_type == LCU_BF16) GO(float, bf16_t, float);
+    if (x_type == LCU_F32 && act_type == LCU_BF16 && delta_type == LCU_BF16) GO(float, bf16_t, bf16_t);
+    if (x_type == LCU_BF16 && act_type == LCU_BF16 && delta_type == LCU_BF16) GO(bf16_t, bf16_t, bf16_t);
+#undef GO
     return LCU_BAD_ARGUMENT;
 }
 
 // The same with the branch's output as `planes` float32 planes [n, d], one after the other:
-// x (float32) += plane 0 + plane 1 + ... (in this order), then the norm.  d a multiple of 4.
+// x (float32) += delta_scale * (plane 0, plane 1, ... in this order), then the norm.  d a multiple of 4.
 LCU_API int lcu_rmsnorm_planes(float *x, const float *planes_ptr, int planes, const void *w, int w_type, void *out,
-                               int act_type, int n, int d, float eps, int write_back, hipStream_t stream) {
+                               int act_type, int n, int d, float eps, int write_back, float delta_scale, hipStream_t stream) {
     if (n <= 0) return LCU_OK;
     if (d <= 0 || d % 4 || planes <= 0 || !planes_ptr) return LCU_BAD_ARGUMENT;
     const size_t stride = (size_t)n * d;
-    if (act_type == LCU_F32) return rmsnorm_w<float, float, float>(x, planes_ptr, w, w_type, out, n, d, eps, write_back, stream, planes, stride);
-    if (act_type == LCU_BF16) return rmsnorm_w<float, float, bf16_t>(x, planes_ptr, w, w_type, out, n, d, eps, write_back, stream, planes, stride);
+    if (act_type == LCU_F32) return rmsnorm_w<float, float, float>(x, planes_ptr, w, w_type, out, n, d, eps, write_back, delta_scale, stream, planes, stride);
+    if (act_type == LCU_BF16) return rmsnorm_w<float, float, bf16_t>(x, planes_ptr, w, w_type, out, n, d, eps, write_back, delta_scale, stream, planes, stride);
     return LCU_BAD_ARGUMENT;
 }
 
-// ---------------------------------------------------------------- residual add: x (f32) += delta
-template <class TD>
-__global__ void residual_add_kernel(float *__restrict__ x, const TD *__restrict__ delta, size_t total) {
-    size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
-    if (i < total) x[i] += to_f32(delta[i]);
+// ---------------------------------------------------------------- the residual stream as a product's operand
+// x (f32) += delta_scale * delta (planes as above; null: nothing), written back; out[r, c] = x[r, c] in the compute type, rows ldo
+// apart: the stream (or, with no delta, a copy of it) as columns of a wider operand.
+template <class TD, class TO>
+__global__ void stream_rows_kernel(float *__restrict__ x, const TD *__restrict__ delta, int planes, size_t plane_stride, float delta_scale,
+                                   TO *__restrict__ out, int ldo, int d) {
+    float *xr = x + (size_t)blockIdx.x * d;
+    TO *o = out + (size_t)blockIdx.x * ldo;
+    for (int c = threadIdx.x; c < d; c += blockDim.x) {
+        float v = xr[c];
+        if (delta) {
+            const TD *dr = delta + (size_t)blockIdx.x * d + c;
+            for (int p = 0; p < planes; ++p) v = fmaf(delta_scale, to_f32(dr[p * plane_stride]), v);
+            xr[c] = v;
+        }
+        o[c] = from_f32<TO>(v);
+    }
 }
 
-LCU_API int lcu_residual_add(float *x, const void *delta, int delta_type, long long total, hipStream_t stream) {
+LCU_API int lcu_stream_rows(float *x, const void *delta, int delta_type, int planes, float delta_scale, void *out, int out_type, int ldo,
+                            int n, int d, hipStream_t stream) {
+    if (n <= 0) return LCU_OK;
+    if (d <= 0 || ldo < d || planes < 1 || !x || !out) return LCU_BAD_ARGUMENT;
+    const size_t stride = (size_t)n * d;
+    dim3 grid(n), block(256);
+#define GO(TD, TO) stream_rows_kernel<TD, TO><<<grid, block, 0, stream>>>(x, (const TD *)delta, planes, stride, delta_scale, (TO *)out, ldo, d)
+    if (delta_type == LCU_F32 && out_type == LCU_F32) GO(float, float);
+    else if (delta_type == LCU_F32 && out_type == LCU_BF16) GO(float, bf16_t);
+    else if (delta_type == LCU_BF16 && out_type == LCU_BF16) GO(bf16_t, bf16_t);
+    else return LCU_BAD_ARGUMENT;
+#undef GO
+    LCU_LAUNCH_CHECK();
+    return LCU_OK;
+}
+
+// ---------------------------------------------------------------- residual add: x (f32) += scale * delta
+template <class TD>
+__global__ void residual_add_kernel(float *__restrict__ x, const TD *__restrict__ delta, size_t total, float scale) {
+    size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+    if (i < total) x[i] = fmaf(scale, to_f32(delta[i]), x[i]);
+}
+
+LCU_API int lcu_residual_add(float *x, const void *delta, int delta_type, long long total, float scale, hipStream_t stream) {
     if (total <= 0) return LCU_OK;
     dim3 block(256), grid((unsigned)((total + 255) / 256));
-    if (delta_type == LCU_F32) residual_add_kernel<float><<<grid, block, 0, stream>>>(x, (const float *)delta, (size_t)total);
-    else if (delta_type == LCU_BF16) residual_add_kernel<bf16_t><<<grid, block, 0, stream>>>(x, (const bf16_t *)delta, (size_t)total);
+    if (delta_type == LCU_F32) residual_add_kernel<float><<<grid, block, 0, stream>>>(x, (const float *)delta, (size_t)total, scale);
+    else if (delta_type == LCU_BF16) residual_add_kernel<bf16_t><<<grid, block, 0, stream>>>(x, (const bf16_t *)delta, (size_t)total, scale);
     else return LCU_BAD_ARGUMENT;
     LCU_LAUNCH_CHECK();
     return LCU_OK;
 }
 
-// ---------------------------------------------------------------- SwiGLU
-// out[r, c] = act(gate) * up with gate = gu[r, c], up = gu[r, di + c];  ACT 0: gate * (1 / (1 + exp(-gate))) (silu),
-// 1: the tanh form of gelu, 0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))).
-enum { GATE_SILU = 0, GATE_GELU_TANH = 1 };
-template <int ACT>
-__device__ __forceinline__ float gate_act(float z) {
-    if (ACT == GATE_GELU_TANH) return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
-    return z * (1.0f / (1.0f + expf(-z)));
-}
-
+// ---------------------------------------------------------------- SwiGLU and its kin
+// out[r, c] = gate_up(gate, up) with gate = gu[r, c], up = gu[r, di + c] (gate_act.h).
 template <class T, int ACT>
-__global__ void swiglu_kernel(T *__restrict__ out, const T *__restrict__ gu, int di) {
+__global__ void swiglu_kernel(T *__restrict__ out, const T *__restrict__ gu, int di, float alpha, float limit) {
     const int c = blockIdx.x * blockDim.x + threadIdx.x;
     if (c >= di) return;
     const size_t r = blockIdx.y;
     const float gate = to_f32(gu[r * 2 * di + c]);
     const float up = to_f32(gu[r * 2 * di + di + c]);
-    out[r * di + c] = from_f32<T>(gate_act<ACT>(gate) * up);
+    out[r * di + c] = from_f32<T>(gate_up<ACT>(gate, up, alpha, limit));
 }
 
 // The same, eight neighbouring columns per thread (16-byte loads of bfloat16, 32-byte of
@@ -279,7 +311,7 @@ __global__ void swiglu_kernel(T *__restrict__ out, const T *__restrict__ gu, int
 template <class T> struct alignas(8 * sizeof(T)) Vec8 { T v[8]; };
 
 template <class T, int ACT>
-__global__ void swiglu_vec8_kernel(T *__restrict__ out, const T *__restrict__ gu, int di) {
+__global__ void swiglu_vec8_kernel(T *__restrict__ out, const T *__restrict__ gu, int di, float alpha, float limit) {
     const int c = (blockIdx.x * blockDim.x + threadIdx.x) * 8;
     if (c >= di) return;
     const size_t r = blockIdx.y;
@@ -287,43 +319,41 @@ __global__ void swiglu_vec8_kernel(T *__restrict__ out, const T *__restrict__ gu
     const Vec8<T> u = *(const Vec8<T> *)(gu + r * 2 * di + di + c);
     Vec8<T> o;
 #pragma unroll
-    for (int e = 0; e < 8; ++e) {
-        const float gate = to_f32(g.v[e]);
-        o.v[e] = from_f32<T>(gate_act<ACT>(gate) * to_f32(u.v[e]));
-    }
+    for (int e = 0; e < 8; ++e) o.v[e] = from_f32<T>(gate_up<ACT>(to_f32(g.v[e]), to_f32(u.v[e]), alpha, limit));
     *(Vec8<T> *)(out + r * di + c) = o;
 }
 
 template <class T, int ACT>
-static void swiglu_launch(T *out, const T *gate_up, int rows, int di, hipStream_t stream) {
+static void swiglu_launch(T *out, const T *gate_up, int rows, int di, float alpha, float limit, hipStream_t stream) {
     const dim3 block(256);
     if (di % 8 == 0)
-        swiglu_vec8_kernel<T, ACT><<<dim3((di / 8 + 255) / 256, rows), block, 0, stream>>>(out, gate_up, di);
+        swiglu_vec8_kernel<T, ACT><<<dim3((di / 8 + 255) / 256, rows), block, 0, stream>>>(out, gate_up, di, alpha, limit);
     else
-        swiglu_kernel<T, ACT><<<dim3((di + 255) / 256, rows), block, 0, stream>>>(out, gate_up, di);
+        swiglu_kernel<T, ACT><<<dim3((di + 255) / 256, rows), block, 0, stream>>>(out, gate_up, di, alpha, limit);
 }
 
-// act: 0 silu, 1 the tanh form of gelu.
-LCU_API int lcu_swiglu(void *out, const void *gate_up, int type, int n, int di, int act, hipStream_t stream) {
-    if (n <= 0) return LCU_OK;
-    if (di <= 0 || (act != GATE_SILU && act != GATE_GELU_TANH) || (type != LCU_F32 && type != LCU_BF16)) return LCU_BAD_ARGUMENT;
+template <class T>
+static int swiglu_t(T *out, const T *gu, int n, int di, int act, float alpha, float limit, hipStream_t stream) {
     // grid.y is limited to 65535 rows: larger batches go in slices
     for (int r0 = 0; r0 < n; r0 += 65535) {
         const int rows = (n - r0) < 65535 ? (n - r0) : 65535;
-        if (type == LCU_F32) {
-            float *o = (float *)out + (size_t)r0 * di;
-            const float *g = (const float *)gate_up + (size_t)r0 * 2 * di;
-            if (act == GATE_SILU) swiglu_launch<float, GATE_SILU>(o, g, rows, di, stream);
-            else swiglu_launch<float, GATE_GELU_TANH>(o, g, rows, di, stream);
-        } else {
-            bf16_t *o = (bf16_t *)out + (size_t)r0 * di;
-            const bf16_t *g = (const bf16_t *)gate_up + (size_t)r0 * 2 * di;
-            if (act == GATE_SILU) swiglu_launch<bf16_t, GATE_SILU>(o, g, rows, di, stream);
-            else swiglu_launch<bf16_t, GATE_GELU_TANH>(o, g, rows, di, stream);
-        }
+        T *o = out + (size_t)r0 * di;
+        const T *g = gu + (size_t)r0 * 2 * di;
+        if (act == GATE_SILU) swiglu_launch<T, GATE_SILU>(o, g, rows, di, alpha, limit, stream);
+        else if (act == GATE_GELU_TANH) swiglu_launch<T, GATE_GELU_TANH>(o, g, rows, di, alpha, limit, stream);
+        else swiglu_launch<T, GATE_LIMITED>(o, g, rows, di, alpha, limit, stream);
     }
     LCU_LAUNCH_CHECK();
     return LCU_OK;
+}
+
+// act: 0 silu, 1 the tanh form of gelu, 2 the limited form with alpha and limit (gate_act.h).
+LCU_API int lcu_swiglu(void *out, const void *gate_up, int type, int n, int di, int act, float alpha, float limit, hipStream_t stream) {
+    if (n <= 0) return LCU_OK;
+    if (di <= 0 || act < GATE_SILU || act > GATE_LIMITED || (act == GATE_LIMITED && !(limit > 0.f))) return LCU_BAD_ARGUMENT;
+    if (type == LCU_F32) return swiglu_t<float>((float *)out, (const float *)gate_up, n, di, act, alpha, limit, stream);
+    if (type == LCU_BF16) return swiglu_t<bf16_t>((bf16_t *)out, (const bf16_t *)gate_up, n, di, act, alpha, limit, stream);
+    return LCU_BAD_ARGUMENT;
 }
 
 // ---------------------------------------------------------------- a cap on the logits

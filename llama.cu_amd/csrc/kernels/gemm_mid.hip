@@ -33,6 +33,7 @@
 // wave w loads the shares of rows 16 w .. 16 w + 15 before its first loads of W, so they are back
 // first, adds them in a fixed order and leaves the factors in LDS for the epilogue.
 #include "common.h"
+#include "gate_act.h"
 #include "kv_layout.h"
 
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
@@ -136,7 +137,7 @@ template <int NT, int MT, int EPI, bool PACKED, int C>
 __global__ void __launch_bounds__((C + mid_producers(MT)) * WAVE)
 gemm_mid_kernel(const bf16_t *__restrict__ X, int ldx, const bf16_t *__restrict__ W, int ldw, void *__restrict__ Y, int ldy,
                 int M, int N, int K, int steps_per_slice, const float *__restrict__ sumsq_in, int n_in, int norm_width,
-                float eps) {
+                float eps, float act_alpha, float act_limit) {
     extern __shared__ __attribute__((aligned(16))) char xs[];      // the ring of X, then the rows' factors
     constexpr int BUF = 16 * MT * MID_XROW;
     constexpr int XB = mid_xbufs(MT);
@@ -297,7 +298,7 @@ gemm_mid_kernel(const bf16_t *__restrict__ X, int ldx, const bf16_t *__restrict_
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const float gate = acc[0][m][r], up = acc[NT - 1][m][r];
-                o[r] = gate * (1.0f / (1.0f + expf(-gate))) * up;
+                o[r] = gate_up_of(gate, up, act_alpha, act_limit);
             }
             uint2 pk = {pack2_bf16(o[0], o[1]), pack2_bf16(o[2], o[3])};
             *(uint2 *)((bf16_t *)Y + (size_t)tok * ldy + n) = pk;
@@ -328,6 +329,7 @@ struct MidScale {
     const float *sumsq_in;
     int n_in, norm_width;
     float eps;
+    float act_alpha, act_limit;      // SwiGLU: limit > 0 asks for the limited activation (gate_act.h)
 };
 
 // The number of consumer waves: four; two for SwiGLU with up to 32 rows (workgroups of two tiles, two to a compute
@@ -361,7 +363,8 @@ static int mid_launch_c(const void *X, int ldx, const void *W, int ldw, void *Y,
             }                                                                                                               \
         }                                                                                                                   \
         kernel<<<grid, dim3((C + mid_producers(MT_)) * WAVE), mid_lds_bytes(MT_), stream>>>(                                \
-            (const bf16_t *)X, ldx, (const bf16_t *)W, ldw, Y, ldy, M, N, K, per, sc.sumsq_in, sc.n_in, sc.norm_width, sc.eps); \
+            (const bf16_t *)X, ldx, (const bf16_t *)W, ldw, Y, ldy, M, N, K, per, sc.sumsq_in, sc.n_in, sc.norm_width, sc.eps,   \
+            sc.act_alpha, sc.act_limit); \
     } while (0)
 #define GO_MT(MT_)                 \
     do {                           \
@@ -428,18 +431,18 @@ static int mid_bf16(const void *X, int ldx, const void *W, int ldw, void *Y, int
 }
 
 LCU_API int lcu_gemm_mid_bf16(const void *X, int ldx, const void *W, int ldw, void *Y, int ldy, int M, int N, int K,
-                              int epilogue, int slices, int w_packed, hipStream_t stream) {
-    const MidScale none = {nullptr, 0, 0, 0.f};
-    return mid_bf16(X, ldx, W, ldw, Y, ldy, M, N, K, epilogue, slices, w_packed, none, stream);
+                              int epilogue, int slices, int w_packed, float act_alpha, float act_limit, hipStream_t stream) {
+    const MidScale sc = {nullptr, 0, 0, 0.f, act_alpha, act_limit};
+    return mid_bf16(X, ldx, W, ldw, Y, ldy, M, N, K, epilogue, slices, w_packed, sc, stream);
 }
 
 // The same with rows of X that wait for their normalisation: row i of the product is multiplied by
 // rsqrt(sum(sumsq_in[i][0 .. n_in)) / norm_width + eps) before the epilogue.  sumsq_in: [M][n_in] float32.
 LCU_API int lcu_gemm_mid_bf16_scaled(const void *X, int ldx, const void *W, int ldw, void *Y, int ldy, int M, int N, int K,
                                      int epilogue, int slices, int w_packed, const float *sumsq_in, int n_in,
-                                     int norm_width, float eps, hipStream_t stream) {
+                                     int norm_width, float eps, float act_alpha, float act_limit, hipStream_t stream) {
     if (!sumsq_in || n_in <= 0 || norm_width <= 0) return LCU_BAD_ARGUMENT;
-    const MidScale sc = {sumsq_in, n_in, norm_width, eps};
+    const MidScale sc = {sumsq_in, n_in, norm_width, eps, act_alpha, act_limit};
     return mid_bf16(X, ldx, W, ldw, Y, ldy, M, N, K, epilogue, slices, w_packed, sc, stream);
 }
 
@@ -699,7 +702,7 @@ template <int MT, bool PACKED>
 __global__ void __launch_bounds__((MID_CONSUMERS + mid_producers(MT)) * WAVE)
 gemm_mid_add_norm_kernel(const bf16_t *__restrict__ X, int ldx, const bf16_t *__restrict__ W, int ldw, float *__restrict__ residual,
                          int ldr, int M, int N, int K, const void *__restrict__ norm_w, int norm_w_type, bf16_t *__restrict__ h_out,
-                         int ldh, float *__restrict__ sumsq_out) {
+                         int ldh, float *__restrict__ sumsq_out, float res_scale) {
     extern __shared__ __attribute__((aligned(16))) char xs[];      // the ring of X; at the end the waves' sums
     constexpr int BUF = 16 * MT * MID_XROW;
     constexpr int XB = mid_xbufs(MT);
@@ -774,7 +777,8 @@ gemm_mid_add_norm_kernel(const bf16_t *__restrict__ X, int ldx, const bf16_t *__
         if (tok < M) {
             f32x4 *res = (f32x4 *)(residual + (size_t)tok * ldr + n0);
             f32x4 xn = *res;
-            xn[0] += sum[0]; xn[1] += sum[1]; xn[2] += sum[2]; xn[3] += sum[3];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) xn[r] = fmaf(res_scale, sum[r], xn[r]);
             *res = xn;
             float wn[4];
 #pragma unroll
@@ -793,11 +797,11 @@ gemm_mid_add_norm_kernel(const bf16_t *__restrict__ X, int ldx, const bf16_t *__
 #endif
 
 // X: [M, K] bfloat16 rows ldx apart, M <= 64, K a multiple of 128; W: [N, K] bfloat16, N a multiple of 16, rows ldw apart or
-// packed.  residual: [M, N] float32 rows ldr apart (a multiple of 4), updated in place; norm_w: [N] float32 or bfloat16
+// packed.  residual: [M, N] float32 rows ldr apart (a multiple of 4), updated in place by res_scale times the product; norm_w: [N] float32 or bfloat16
 // (norm_w_type LCU_F32 or LCU_BF16); h_out: [M, N] bfloat16 rows ldh apart (a multiple of 4); sumsq_out: [M][N / 16] float32.
 LCU_API int lcu_gemm_mid_bf16_add_norm(const void *X, int ldx, const void *W, int ldw, float *residual, int ldr, int M, int N, int K,
                                        const void *norm_w, int norm_w_type, void *h_out, int ldh, float *sumsq_out, int w_packed,
-                                       hipStream_t stream) {
+                                       float res_scale, hipStream_t stream) {
     if (M <= 0 || N <= 0) return LCU_OK;
     if (M > 64 || K <= 0 || K % 128 || N % 16 || ldx % 8 || ldx < K || ldr < N || ldr % 4 || ldh < N || ldh % 4 || !residual || !norm_w ||
         !h_out || !sumsq_out || (norm_w_type != LCU_F32 && norm_w_type != LCU_BF16))
@@ -811,7 +815,7 @@ LCU_API int lcu_gemm_mid_bf16_add_norm(const void *X, int ldx, const void *W, in
         constexpr int lds = mid_xbufs(MT_) * 16 * MT_ * MID_XROW;                                                            \
         static_assert(lds >= MID_CONSUMERS * MT_ * WAVE * 16 && lds <= 64 * 1024, "the waves' sums lie over the ring");      \
         gemm_mid_add_norm_kernel<MT_, P_><<<grid, dim3((MID_CONSUMERS + mid_producers(MT_)) * WAVE), lds, stream>>>(         \
-            (const bf16_t *)X, ldx, (const bf16_t *)W, ldw, residual, ldr, M, N, K, norm_w, norm_w_type, (bf16_t *)h_out, ldh, sumsq_out); \
+            (const bf16_t *)X, ldx, (const bf16_t *)W, ldw, residual, ldr, M, N, K, norm_w, norm_w_type, (bf16_t *)h_out, ldh, sumsq_out, res_scale); \
     } while (0)
 #define GO_MT(MT_)                   \
     do {                             \

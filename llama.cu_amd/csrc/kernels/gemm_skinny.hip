@@ -23,8 +23,13 @@
 //
 // Epilogues: store bfloat16; store float32 (logits); add into float32 (the residual
 // stream); SwiGLU, where the workgroup's two tiles are the gate rows n and the up rows
-// n + N/2 of one matrix and silu(gate) * up is stored.
+// n + N/2 of one matrix and silu(gate) * up (or the limited form, gate_act.h) is stored.
+//
+// Grouped: W is several matrices of group_rows rows one above the other, and each multiplies rows of X of its own
+// (group g reads X + g * x_group_stride): one product per head, or several projections of differently mixed rows, in
+// one launch.  Their outputs may be multiplied by the sigmoid of a gate [M, N] on the way out.
 #include "common.h"
+#include "gate_act.h"
 #include "kv_layout.h"
 
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
@@ -66,6 +71,15 @@ struct SkinnyExtra {
     bf16_t *q_out;             // [M, heads * head_dim] rows ldq apart
     int ldq;
     int heads, kv_heads, head_dim, page;
+    // EPI_ADD_NORM: what the product is multiplied by before it is added to the residual stream
+    float res_scale;
+    // EPI_SWIGLU: limit > 0 asks for the limited activation (gate_act.h)
+    float act_alpha, act_limit;
+    // grouped products (group_rows 0: one matrix, one X)
+    int group_rows;
+    size_t x_group_stride;
+    const void *gate;          // [M, N] rows ldg apart, or null
+    int gate_type, ldg;
 };
 
 __device__ __forceinline__ f32x4 mfma16(u32x4 a, u32x4 b, f32x4 c) {
@@ -154,6 +168,7 @@ gemm_skinny_kernel(const bf16_t *__restrict__ X, int ldx, const bf16_t *__restri
         wrow[t] = PACKED ? W + ((size_t)(row / 16) * (K / 128)) * 2048 + (size_t)lane * 8   // (the tile of the row)
                            : W + (size_t)row * ldw;
     }
+    if (ex.group_rows > 0) X += (size_t)(n0 / ex.group_rows) * ex.x_group_stride;      // (a workgroup's rows lie in one group)
     const bf16_t *xrow[MT];
     bool xvalid[MT];
 #pragma unroll
@@ -311,7 +326,7 @@ gemm_skinny_kernel(const bf16_t *__restrict__ X, int ldx, const bf16_t *__restri
                     const int n = n0 + 16 * t + 4 * grp + r;
                     if (tok >= M || n >= N) continue;
                     float *res = (float *)Y + (size_t)tok * ldy + n;
-                    const float xn = *res + acc[t][m][r];
+                    const float xn = fmaf(ex.res_scale, acc[t][m][r], *res);
                     *res = xn;
                     ss += xn * xn;
                     const float wn = ex.norm_w_type == LCU_F32 ? ((const float *)ex.norm_w)[n] : to_f32(((const bf16_t *)ex.norm_w)[n]);
@@ -335,8 +350,7 @@ gemm_skinny_kernel(const bf16_t *__restrict__ X, int ldx, const bf16_t *__restri
                     const int n = n0 + 16 * t + 4 * grp + r;
                     if (n >= n_out) continue;
                     const float gate = acc[t][m][r], up = acc[t + NT / 2][m][r];
-                    const float sig = 1.0f / (1.0f + expf(-gate));
-                    ((bf16_t *)Y)[(size_t)tok * ldy + n] = from_f32<bf16_t>(gate * sig * up);
+                    ((bf16_t *)Y)[(size_t)tok * ldy + n] = from_f32<bf16_t>(gate_up_of(gate, up, ex.act_alpha, ex.act_limit));
                 }
         } else {
 #pragma unroll
@@ -346,6 +360,11 @@ gemm_skinny_kernel(const bf16_t *__restrict__ X, int ldx, const bf16_t *__restri
                     const int n = n0 + 16 * t + 4 * grp + r;
                     if (n >= N) continue;
                     const size_t at = (size_t)tok * ldy + n;
+                    if (EPI == EPI_BF16 && ex.gate != nullptr) {
+                        const size_t ga = (size_t)tok * ex.ldg + n;
+                        const float z = ex.gate_type == LCU_F32 ? ((const float *)ex.gate)[ga] : to_f32(((const bf16_t *)ex.gate)[ga]);
+                        acc[t][m][r] *= 1.0f / (1.0f + expf(-z));
+                    }
                     if (EPI == EPI_BF16) ((bf16_t *)Y)[at] = from_f32<bf16_t>(acc[t][m][r]);
                     else if (EPI == EPI_F32) ((float *)Y)[at] = acc[t][m][r];
                     else ((float *)Y)[at] += acc[t][m][r];
@@ -441,24 +460,42 @@ static int skinny_bf16(const void *X, int ldx, const void *W, int ldw, void *Y, 
 }
 
 LCU_API int lcu_gemm_skinny_bf16(const void *X, int ldx, const void *W, int ldw, void *Y, int ldy, int M, int N, int K,
-                                 int epilogue, int tiles, int waves, int w_packed, hipStream_t stream) {
+                                 int epilogue, int tiles, int waves, int w_packed, float act_alpha, float act_limit, hipStream_t stream) {
     if (epilogue == EPI_ADD_NORM) return LCU_BAD_ARGUMENT;
-    const SkinnyExtra none = {};
-    return skinny_bf16(X, ldx, W, ldw, Y, ldy, M, N, K, epilogue, tiles, waves, w_packed, none, stream);
+    SkinnyExtra ex = {};
+    ex.act_alpha = act_alpha; ex.act_limit = act_limit;
+    return skinny_bf16(X, ldx, W, ldw, Y, ldy, M, N, K, epilogue, tiles, waves, w_packed, ex, stream);
+}
+
+// Grouped: rows g * group_rows .. of W multiply the rows X + g * x_group_stride (M rows ldx apart); Y [M, N] takes all groups
+// side by side, bfloat16 or float32 (epilogue).  gate (bfloat16 output only; may be null): [M, N] rows ldg apart of
+// gate_type, the product is multiplied by its sigmoid before it is rounded.  group_rows a multiple of 16 * tiles.
+LCU_API int lcu_gemm_skinny_bf16_grouped(const void *X, int ldx, long long x_group_stride, const void *W, int ldw, int group_rows, void *Y,
+                                         int ldy, int M, int N, int K, int epilogue, int tiles, int waves, int w_packed,
+                                         const void *gate, int gate_type, int ldg, hipStream_t stream) {
+    if ((epilogue != EPI_BF16 && epilogue != EPI_F32) || group_rows <= 0 || tiles <= 0 || group_rows % (16 * tiles) || N % group_rows ||
+        x_group_stride < 0 || x_group_stride % 8)
+        return LCU_BAD_ARGUMENT;
+    if (gate && (epilogue != EPI_BF16 || ldg < N || (gate_type != LCU_F32 && gate_type != LCU_BF16))) return LCU_BAD_ARGUMENT;
+    SkinnyExtra ex = {};
+    ex.group_rows = group_rows; ex.x_group_stride = (size_t)x_group_stride;
+    ex.gate = gate; ex.gate_type = gate_type; ex.ldg = ldg;
+    return skinny_bf16(X, ldx, W, ldw, Y, ldy, M, N, K, epilogue, tiles, waves, w_packed, ex, stream);
 }
 
 // The product that ends a branch, the residual sum and the next norm's weight in one kernel:
-// res[M, N] (float32, rows ldres apart) += X W^T; h_out[M, N] = bfloat16(res * norm_w), not yet
+// res[M, N] (float32, rows ldres apart) += res_scale * (X W^T); h_out[M, N] = bfloat16(res * norm_w), not yet
 // normalised; sumsq_out[M][ceil(N / (16 tiles))] = each workgroup's share of the rows' sums of
 // squares.  At most 32 rows, tiles 1 or 2.
 LCU_API int lcu_gemm_skinny_bf16_add_norm(const void *X, int ldx, const void *W, int ldw, float *res, int ldres, int M, int N,
                                           int K, const void *norm_w, int norm_w_type, void *h_out, int ldh, float *sumsq_out,
-                                          int sumsq_cols, int tiles, int waves, int w_packed, hipStream_t stream) {
+                                          int sumsq_cols, int tiles, int waves, int w_packed, float res_scale, hipStream_t stream) {
     if (M > 32 || (tiles != 1 && tiles != 2) || !res || !norm_w || !h_out || !sumsq_out || ldh < N || ldres < N ||
         (norm_w_type != LCU_F32 && norm_w_type != LCU_BF16) || sumsq_cols != (N + 16 * tiles - 1) / (16 * tiles))
         return LCU_BAD_ARGUMENT;
     SkinnyExtra ex = {};
     ex.norm_w = norm_w; ex.norm_w_type = norm_w_type; ex.h_out = (bf16_t *)h_out; ex.ldh = ldh; ex.sumsq_out = sumsq_out;
+    ex.res_scale = res_scale;
     return skinny_bf16(X, ldx, W, ldw, res, ldres, M, N, K, EPI_ADD_NORM, tiles, waves, w_packed, ex, stream);
 }
 
@@ -466,10 +503,11 @@ LCU_API int lcu_gemm_skinny_bf16_add_norm(const void *X, int ldx, const void *W,
 // rsqrt(sum(sumsq_in[i][0 .. n_in)) / norm_width + eps) before the epilogue (not EPI_ADD_NORM).
 LCU_API int lcu_gemm_skinny_bf16_scaled(const void *X, int ldx, const void *W, int ldw, void *Y, int ldy, int M, int N, int K,
                                         int epilogue, int tiles, int waves, int w_packed, const float *sumsq_in, int n_in,
-                                        int norm_width, float eps, hipStream_t stream) {
+                                        int norm_width, float eps, float act_alpha, float act_limit, hipStream_t stream) {
     if (epilogue == EPI_ADD_NORM || !sumsq_in || n_in <= 0 || norm_width <= 0) return LCU_BAD_ARGUMENT;
     SkinnyExtra ex = {};
     ex.sumsq_in = sumsq_in; ex.n_in = n_in; ex.norm_width = norm_width; ex.eps = eps;
+    ex.act_alpha = act_alpha; ex.act_limit = act_limit;
     return skinny_bf16(X, ldx, W, ldw, Y, ldy, M, N, K, epilogue, tiles, waves, w_packed, ex, stream);
 }
 

@@ -7,13 +7,21 @@
 //              [max_pos, rot_dim / 2]; pairing 0: (i, i + rot_dim/2), 1: (2i, 2i + 1)); the other dims pass
 //   q -> q_out [n, nh * dhp]; k, v -> the token's place in its page
 //
+// Maps (maps > 1): every query head and every key head is `maps` vectors of dh dims side by side in the rows, each normed and
+// rotated by itself, over the head's one set of values (attention that is several attentions over the same values).  The
+// kernels behind this one see plain attention heads, one per (head, map), in one of two layouts:
+//   joint   a key head is its maps' keys side by side (maps * dh dims); the query of map m has its dims at m * dh and zeros
+//           elsewhere, so its score is that of map m alone; query heads in the order (head, map);
+//   split   a key head for every (key head, map), each with a copy of the values; query heads in the order (key head, map,
+//           head of the group).
+//
 // The head sizes of the rows (dh, dv) may be any; what is stored has dhp >= dh and dvp >= dv dims per head, the
 // dims beyond the true ones zeros (dhp a multiple of 8, as the pages' layout wants; zeros change no score and no
 // output).  All arithmetic is 32-bit, one rounding at each store.  One wave per (token, head).
 #include "common.h"
 #include "kv_layout.h"
 
-constexpr int QP_MAX_DIM = 256;
+constexpr int QP_MAX_DIM = 640;
 
 template <class TI, class T>
 __global__ void __launch_bounds__(WAVE)
@@ -22,8 +30,10 @@ qkv_prepare_kernel(const TI *__restrict__ rows, int row_stride, int q_off, int k
                    float eps, const int *__restrict__ positions, const float *__restrict__ cos_t,
                    const float *__restrict__ sin_t, int max_pos, int rot_dim, int pairing, T *__restrict__ q_out,
                    const int *__restrict__ slots, T *__restrict__ cache, int nh, int nkvh, int dh, int dhp, int dv,
-                   int dvp, int page, int store_kv) {
+                   int dvp, int page, int store_kv, int maps, int joint) {
+    // nh and nkvh count (head, map) pairs; stored_kvh: key/value heads in the cache
     const int t = blockIdx.x, head = blockIdx.y, lane = threadIdx.x;
+    const int stored_kvh = joint ? nkvh / maps : nkvh;
     const TI *row = rows + (size_t)t * row_stride;
     __shared__ float xs[QP_MAX_DIM];
     int slot = -1;
@@ -32,15 +42,15 @@ qkv_prepare_kernel(const TI *__restrict__ rows, int row_stride, int q_off, int k
     if (head >= nh) {
         slot = store_kv ? slots[t] : -1;
         if (slot < 0) return;
-        pg = cache + (size_t)(slot / page) * kv_page_elems(nkvh, dhp, dvp, page);
+        pg = cache + (size_t)(slot / page) * kv_page_elems(stored_kvh, dhp, dvp, page);
         tok = slot % page;
     }
     if (head >= nh + nkvh) {                                  // a value head: product + bias, as it is
-        const int kvh = head - nh - nkvh, col0 = v_off + kvh * dv;
+        const int kvh = head - nh - nkvh, col0 = v_off + (joint ? kvh : kvh / maps) * dv;
         for (int c = lane; c < dvp; c += WAVE) {
             float v = 0.f;
             if (c < dv) v = to_f32(row[col0 + c]) + (bias ? bias[col0 + c] : 0.f);
-            pg[kv_value_offset(nkvh, kvh, tok, c, dhp, dvp, page)] = from_f32<T>(v);
+            pg[kv_value_offset(stored_kvh, kvh, tok, c, dhp, dvp, page)] = from_f32<T>(v);
         }
         return;
     }
@@ -70,32 +80,43 @@ qkv_prepare_kernel(const TI *__restrict__ rows, int row_stride, int q_off, int k
         }
         __syncthreads();
     }
+    // where the vector's first dim goes among the stored head's dims; a joint head's other dims are zeros in a query and the
+    // other maps' in a key, whose last map also writes the zeros behind them
+    const int map = maps > 1 ? (is_key ? head - nh : head) % maps : 0, at = joint ? map * dh : 0;
     if (!is_key) {
-        T *o = q_out + (size_t)t * nh * dhp + (size_t)head * dhp;
-        for (int c = lane; c < dhp; c += WAVE) o[c] = from_f32<T>(c < dh ? xs[c] : 0.f);
+        int place = head;
+        if (maps > 1 && !joint) {
+            const int group = nh / nkvh, qh = head / maps;            // query heads of a key head
+            place = (qh / group * maps + map) * group + qh % group;
+        }
+        T *o = q_out + (size_t)t * nh * dhp + (size_t)place * dhp;
+        for (int c = lane; c < dhp; c += WAVE) o[c] = from_f32<T>(c >= at && c < at + dh ? xs[c - at] : 0.f);
     } else {
-        const int kvh = head - nh;
-        for (int c = lane; c < dhp; c += WAVE) pg[kv_key_offset(kvh, tok, c, dhp, page)] = from_f32<T>(c < dh ? xs[c] : 0.f);
+        const int kvh = joint ? (head - nh) / maps : head - nh;
+        const int end = !joint || map == maps - 1 ? dhp : at + dh;
+        for (int c = at + lane; c < end; c += WAVE) pg[kv_key_offset(kvh, tok, c, dhp, page)] = from_f32<T>(c < at + dh ? xs[c - at] : 0.f);
     }
 }
 
 // rows: [n, row_stride] of in_type, a token's q heads at column q_off (nh * dh), k heads at k_off (nkvh * dh), v heads
 // at v_off (nkvh * dv); bias: null or float32 over the row's columns; q_norm, k_norm: null or float32 [dh].
 // q_out: [n, nh * dhp] of type; cache: this layer's pages of type, kv_page_elems(nkvh, dhp, dvp, page) each;
-// slots[t] = page * page_size + place, or -1 to store nothing for token t.  store_kv 0: queries only.
+// slots[t] = page * page_size + place, or -1 to store nothing for token t.  store_kv 0: queries only.  maps > 1: nh and nkvh count
+// (head, map) pairs; the cache's pages hold nkvh / maps (joint) or nkvh (split) key/value heads, dhp >= maps * dh (joint) or dh.
 LCU_API int lcu_qkv_prepare(const void *rows, int in_type, int n, int row_stride, int q_off, int k_off, int v_off,
                             const float *bias, const float *q_norm, const float *k_norm, float eps, const int *positions,
                             const float *cos_t, const float *sin_t, int max_pos, int rot_dim, int pairing, void *q_out,
                             int type, const int *slots, void *cache, int nh, int nkvh, int dh, int dhp, int dv, int dvp,
-                            int page, int store_kv, hipStream_t stream) {
+                            int page, int store_kv, int maps, int joint, hipStream_t stream) {
     if (n <= 0) return LCU_OK;
     if (nh <= 0 || nkvh < 0 || dh <= 0 || dh > QP_MAX_DIM || dhp < dh || dhp % 8 || dhp > QP_MAX_DIM || dv <= 0 || dvp < dv ||
         dvp > QP_MAX_DIM || page <= 0 || page % 8 || rot_dim < 0 || rot_dim % 2 || rot_dim > dh || (pairing != 0 && pairing != 1) ||
-        !rows || !q_out || (cos_t && (!sin_t || !positions || rot_dim == 0)) || nh + 2 * nkvh > 65535)
+        !rows || !q_out || (cos_t && (!sin_t || !positions || rot_dim == 0)) || nh + 2 * nkvh > 65535 || maps < 1 || nh % maps || nkvh % maps || (joint && (maps < 2 || dhp < maps * dh)) ||
+        (maps > 1 && !store_kv))
         return LCU_BAD_ARGUMENT;
     if (store_kv && (!cache || !slots || nkvh <= 0)) return LCU_BAD_ARGUMENT;
-    dim3 grid(n, store_kv ? nh + 2 * nkvh : nh), block(WAVE);
-#define GO(TI, T) qkv_prepare_kernel<TI, T><<<grid, block, 0, stream>>>((const TI *)rows, row_stride, q_off, k_off, v_off, bias, q_norm, k_norm, eps, positions, cos_t, sin_t, max_pos, rot_dim, pairing, (T *)q_out, slots, (T *)cache, nh, nkvh, dh, dhp, dv, dvp, page, store_kv)
+    dim3 grid(n, store_kv ? nh + nkvh + (joint ? nkvh / maps : nkvh) : nh), block(WAVE);
+#define GO(TI, T) qkv_prepare_kernel<TI, T><<<grid, block, 0, stream>>>((const TI *)rows, row_stride, q_off, k_off, v_off, bias, q_norm, k_norm, eps, positions, cos_t, sin_t, max_pos, rot_dim, pairing, (T *)q_out, slots, (T *)cache, nh, nkvh, dh, dhp, dv, dvp, page, store_kv, maps, joint)
     if (in_type == LCU_F32 && type == LCU_F32) GO(float, float);
     else if (in_type == LCU_F32 && type == LCU_BF16) GO(float, bf16_t);
     else if (in_type == LCU_BF16 && type == LCU_BF16) GO(bf16_t, bf16_t);

@@ -16,27 +16,11 @@
 //
 // o is written [head][tile of 16 columns][token][16].  The output: each head's o divided by its root mean square (eps, no weight), times silu(gate) (second kernel).
 #include "common.h"
+#include "lane_moves.h"
 
 constexpr int RT_THREADS = 256;
 constexpr int RT_LANES = 16;                      // lanes that share a column
 constexpr int RT_COLS = RT_THREADS / RT_LANES;    // columns a workgroup
-
-// Moves between the lanes of a group of sixteen inside the vector unit (no trip through LDS): the neighbour, the lane two
-// away, the mirror image within eight and within sixteen.  After the first two every lane of a quad holds the quad's sum,
-// so the mirror image within eight brings the other quad's, and the one within sixteen the other eight's.
-__device__ __forceinline__ float lane_xor1(float v) {
-    return __builtin_bit_cast(float, __builtin_amdgcn_mov_dpp(__builtin_bit_cast(int, v), 0xB1, 0xF, 0xF, true));     // quad_perm [1, 0, 3, 2]
-}
-__device__ __forceinline__ float lane_xor2(float v) {
-    return __builtin_bit_cast(float, __builtin_amdgcn_mov_dpp(__builtin_bit_cast(int, v), 0x4E, 0xF, 0xF, true));     // quad_perm [2, 3, 0, 1]
-}
-__device__ __forceinline__ float lane_mirror8(float v) {
-    return __builtin_bit_cast(float, __builtin_amdgcn_mov_dpp(__builtin_bit_cast(int, v), 0x141, 0xF, 0xF, true));    // row_half_mirror
-}
-
-__device__ __forceinline__ float lane_mirror16(float v) {
-    return __builtin_bit_cast(float, __builtin_amdgcn_mov_dpp(__builtin_bit_cast(int, v), 0x140, 0xF, 0xF, true));    // row_mirror
-}
 
 // q and k of every (token, head), rotated, k scaled, and v, 32-bit: qkv [nh][n][2 d + dv], a head's tokens one after the
 // other, so that the scan's workgroups, which own a head, each stream a run of memory of their own (with rows of all

@@ -163,8 +163,8 @@ def gather_rows(x: torch.Tensor, rows: torch.Tensor, out: Optional[torch.Tensor]
 
 
 def rmsnorm(x: torch.Tensor, weight: torch.Tensor, eps: float, out: torch.Tensor,
-            delta: Optional[torch.Tensor] = None, write_back: bool = True) -> torch.Tensor:
-    """``y = x' * rsqrt(mean(x'^2) + eps) * weight`` with ``x' = x + delta`` (``x`` if there is
+            delta: Optional[torch.Tensor] = None, write_back: bool = True, delta_scale: float = 1.0) -> torch.Tensor:
+    """``y = x' * rsqrt(mean(x'^2) + eps) * weight`` with ``x' = x + delta_scale * delta`` (``x`` if there is
     no ``delta``), all in 32-bit.  With ``write_back`` the sum ``x'`` replaces ``x`` (the
     residual stream takes in the branch's output).  ``delta`` may also be float32 planes
     ``[planes, n, d]`` (a product's partial sums, ``gemm_mid(..., slices=)``) beside a float32
@@ -183,39 +183,69 @@ def rmsnorm(x: torch.Tensor, weight: torch.Tensor, eps: float, out: torch.Tensor
             raise KernelError("norm delta: planes must be float32 [planes, n, d] beside a float32 input, d a multiple of 4")
         lib = build.load("elementwise")
         _check(lib.lcu_rmsnorm_planes(_ptr(x), _ptr(delta), delta.shape[0], _ptr(weight), _type(weight, "norm weight"),
-                                      _ptr(out), at, n, d, ctypes.c_float(eps), int(bool(write_back)), _stream()),
+                                      _ptr(out), at, n, d, ctypes.c_float(eps), int(bool(write_back)), ctypes.c_float(delta_scale), _stream()),
                "rmsnorm (planes)")
         return out
     if delta is not None:
         _contig(delta, "norm delta")
-        if delta.shape != (n, d) or delta.dtype != out.dtype:
-            raise KernelError("norm delta: must have the output's shape and type")
-    if (xt, at) not in ((F32, F32), (F32, BF16), (BF16, BF16)):
-        raise KernelError(f"norm: input {x.dtype} with output {out.dtype} is not supported")
+        if delta.shape != (n, d):
+            raise KernelError("norm delta: must have the output's shape")
+    dt = at if delta is None else _type(delta, "norm delta")
+    if (xt, dt, at) not in ((F32, F32, F32), (F32, BF16, F32), (F32, BF16, BF16), (BF16, BF16, BF16)):
+        raise KernelError(f"norm: input {x.dtype} with output {out.dtype}" + ("" if delta is None else f" and delta {delta.dtype}") + " is not supported")
     lib = build.load("elementwise")
-    _check(lib.lcu_rmsnorm(_ptr(x), xt, _ptr(delta), _ptr(weight), _type(weight, "norm weight"), _ptr(out), at,
-                           n, d, ctypes.c_float(eps), int(bool(write_back)), _stream()), "rmsnorm")
+    _check(lib.lcu_rmsnorm(_ptr(x), xt, _ptr(delta), dt, _ptr(weight), _type(weight, "norm weight"), _ptr(out), at,
+                           n, d, ctypes.c_float(eps), int(bool(write_back)), ctypes.c_float(delta_scale), _stream()), "rmsnorm")
     return out
 
 
-def residual_add(x: torch.Tensor, delta: torch.Tensor) -> torch.Tensor:
-    """``x += delta`` in 32-bit (``x`` is float32)."""
+def residual_add(x: torch.Tensor, delta: torch.Tensor, scale: float = 1.0) -> torch.Tensor:
+    """``x += scale * delta`` in 32-bit (``x`` is float32)."""
     _gpu(x, delta)
     _contig(x, "residual"); _contig(delta, "delta")
     if x.dtype != torch.float32 or x.shape != delta.shape:
         raise KernelError("residual_add: x must be float32 and delta of the same shape")
     lib = build.load("elementwise")
-    _check(lib.lcu_residual_add(_ptr(x), _ptr(delta), _type(delta, "delta"), ctypes.c_longlong(x.numel()), _stream()),
+    _check(lib.lcu_residual_add(_ptr(x), _ptr(delta), _type(delta, "delta"), ctypes.c_longlong(x.numel()), ctypes.c_float(scale), _stream()),
            "residual_add")
     return x
 
 
-GATE_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1}
+def stream_rows(x: torch.Tensor, out: torch.Tensor, delta: Optional[torch.Tensor] = None, delta_scale: float = 1.0) -> torch.Tensor:
+    """``x += delta_scale * delta`` in 32-bit (``x`` float32 ``[n, d]``, in place; ``delta`` None: nothing; rows, or float32 planes
+    ``[planes, n, d]``), then ``out[:, :] = x`` in ``out``'s type: ``out [n, d]`` may be columns of a wider row."""
+    _gpu(x, out, delta)
+    _rows(x, "stream"); _contig(x, "stream"); _rows(out, "stream rows")
+    n, d = x.shape
+    if x.dtype != torch.float32 or out.shape != (n, d):
+        raise KernelError(f"stream_rows: the stream must be float32 and the output {(n, d)}")
+    planes = 1
+    dt = F32 if out.dtype == torch.float32 else BF16
+    if delta is not None:
+        _contig(delta, "stream delta")
+        if delta.dim() == 3:
+            planes = delta.shape[0]
+            if delta.dtype != torch.float32:
+                raise KernelError("stream_rows: planes of partial sums are float32")
+        if delta.shape[-2:] != (n, d):
+            raise KernelError("stream_rows: the delta must have the stream's shape")
+        dt = _type(delta, "stream delta")
+    lib = build.load("elementwise")
+    _check(lib.lcu_stream_rows(_ptr(x), _ptr(delta), dt, planes, ctypes.c_float(delta_scale), _ptr(out), _type(out, "stream rows"),
+                               out.stride(0), n, d, _stream()), "stream_rows")
+    return out
 
 
-def swiglu(gate_up: torch.Tensor, out: Optional[torch.Tensor] = None, activation: str = "silu") -> torch.Tensor:
+GATE_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1, "limited": 2}
+
+
+def swiglu(gate_up: torch.Tensor, out: Optional[torch.Tensor] = None, activation: str = "silu", alpha: float = 1.0,
+           limit: float = 0.0) -> torch.Tensor:
     """``out = act(gate) * up`` for ``gate_up = [gate | up]`` of shape ``[n, 2*di]``; ``activation``: ``silu`` (``gate *
-    sigmoid(gate)``) or ``gelu_tanh`` (``0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3)))``)."""
+    sigmoid(gate)``) or ``gelu_tanh`` (``0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3)))``); or ``limited``: ``out = g
+    sigmoid(alpha g) (u + 1)`` with ``g = min(gate, limit)`` and ``u`` = ``up`` held within ``-limit .. limit``."""
+    if activation == "limited" and not limit > 0:
+        raise KernelError("swiglu: the limited activation needs a positive limit")
     if activation not in GATE_ACTIVATIONS:
         raise KernelError(f"swiglu: no activation {activation!r}; known: {sorted(GATE_ACTIVATIONS)}")
     _gpu(gate_up, out)
@@ -229,7 +259,8 @@ def swiglu(gate_up: torch.Tensor, out: Optional[torch.Tensor] = None, activation
     if out.shape != (n, di) or out.dtype != gate_up.dtype or not out.is_contiguous():
         raise KernelError("swiglu out: wrong shape, type or layout")
     lib = build.load("elementwise")
-    _check(lib.lcu_swiglu(_ptr(out), _ptr(gate_up), _type(gate_up, "gate_up"), n, di, GATE_ACTIVATIONS[activation], _stream()), "swiglu")
+    _check(lib.lcu_swiglu(_ptr(out), _ptr(gate_up), _type(gate_up, "gate_up"), n, di, GATE_ACTIVATIONS[activation],
+                          ctypes.c_float(alpha), ctypes.c_float(limit), _stream()), "swiglu")
     return out
 
 
@@ -333,12 +364,13 @@ def paged_attention_generic(q: torch.Tensor, out: torch.Tensor, cache: torch.Ten
                             q_start: torch.Tensor, ctx_len: torch.Tensor, req_of_token: torch.Tensor,
                             n_heads: int, n_kv_heads: int, head_dim: int, page_size: int, scale: float,
                             window: int = 0, head_slopes: Optional[torch.Tensor] = None, value_dim: int = 0,
-                            chunk: int = 0, sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+                            chunk: int = 0, sinks: Optional[torch.Tensor] = None, softcap: float = 0.0) -> torch.Tensor:
     """Causal attention of the step's queries over the paged cache (every shape).  ``head_slopes``
     (float32 [n_heads]) adds ``slope[h] * (key position - query position)`` to the scaled scores.
     ``value_dim``: the values' head size if it is not the keys' (``out`` is ``[n, n_heads * value_dim]``).
     ``chunk``: the query at position ``p`` sees the keys from ``p - p % chunk`` on only (instead of a window).
-    ``sinks`` (float32 [n_heads]): ``exp(sink[h])`` stands in every softmax's denominator beside the keys' terms."""
+    ``sinks`` (float32 [n_heads]): ``exp(sink[h])`` stands in every softmax's denominator beside the keys' terms.
+    ``softcap`` > 0: a scaled score ``s`` becomes ``softcap * tanh(s / softcap)``, before any bias."""
     n = _attention_args(q, out, cache, block_table, q_start, ctx_len, req_of_token, n_heads, n_kv_heads, head_dim,
                         page_size, value_dim)
     value_dim = value_dim or head_dim
@@ -354,7 +386,7 @@ def paged_attention_generic(q: torch.Tensor, out: torch.Tensor, cache: torch.Ten
                                            _ptr(block_table), block_table.shape[1], _ptr(q_start), _ptr(ctx_len),
                                            _ptr(req_of_token), n, n_heads, n_kv_heads, head_dim, value_dim, page_size,
                                            ctypes.c_float(scale), int(window), int(chunk), _ptr(head_slopes), _ptr(sinks),
-                                           _stream()), "paged_attention_generic")
+                                           ctypes.c_float(softcap), _stream()), "paged_attention_generic")
     return out
 
 
@@ -406,20 +438,28 @@ def mfma_attention_supported(q: torch.Tensor, n_heads: int, n_kv_heads: int, hea
     return mfma_attention_refusal(q.dtype, n_heads, n_kv_heads, head_dim, page_size) is None and q.stride(0) % 8 == 0
 
 
+def _attention_library(head_slopes=None, softcap: float = 0.0):
+    """The matrix-core attention library whose kernels these scores need: with a bias (and sinks), with a cap, or plain."""
+    if head_slopes is not None:
+        return "attention_mfma_bias"
+    return "attention_mfma_cap" if softcap else "attention_mfma"
+
+
 def attention_decode(q, out, cache, block_table, q_start, ctx_len, n_req, n_heads, n_kv_heads, head_dim, page_size,
                      scale, window, n_splits, req_list: Optional[torch.Tensor] = None,
-                     head_slopes: Optional[torch.Tensor] = None, sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+                     head_slopes: Optional[torch.Tensor] = None, sinks: Optional[torch.Tensor] = None, softcap: float = 0.0) -> torch.Tensor:
     """Matrix-core attention for requests that feed one token each: all ``n_req`` requests of
     the batch, or the ``n_req`` whose indices ``req_list`` holds.  ``head_slopes``: the bias on the distance inside
-    the scores (the kernels of the second library, ``attention_mfma_bias``)."""
+    the scores (the kernels of the second library, ``attention_mfma_bias``); ``softcap``: a cap on them (the third,
+    ``attention_mfma_cap``)."""
     if req_list is not None:
         _i32(req_list, "req_list", n_req)
     part_o = part_ml = None
     if n_splits > 1:
         part_o = torch.empty(n_req * n_heads * n_splits * head_dim, dtype=torch.float32, device=q.device)
         part_ml = torch.empty(n_req * n_heads * n_splits * 2, dtype=torch.float32, device=q.device)
-    lib = build.load("attention_mfma" if head_slopes is None else "attention_mfma_bias")
-    more = () if head_slopes is None else (_ptr(head_slopes), _ptr(sinks))
+    lib = build.load(_attention_library(head_slopes, softcap))
+    more = (_ptr(head_slopes), _ptr(sinks)) if head_slopes is not None else (ctypes.c_float(softcap),) if softcap else ()
     _check(lib.lcu_attention_decode_bf16(_ptr(q), q.stride(0), _ptr(out), out.stride(0), _ptr(cache), _ptr(block_table),
                                          block_table.shape[1], _ptr(q_start), _ptr(ctx_len), _ptr(req_list), n_req, n_heads,
                                          n_kv_heads,
@@ -466,7 +506,7 @@ def prefill_tasks(q_lens, ctx_lens, tokens_per_task: int, device, skip_single: b
 
 def attention_prefill(q, out, cache, block_table, q_start, ctx_len, task_req, task_tok0, n_tasks, tasks_per_wg, n_heads,
                       n_kv_heads, head_dim, page_size, scale, window, n_tasks_dev: Optional[torch.Tensor] = None,
-                      head_slopes: Optional[torch.Tensor] = None, sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+                      head_slopes: Optional[torch.Tensor] = None, sinks: Optional[torch.Tensor] = None, softcap: float = 0.0) -> torch.Tensor:
     """Matrix-core attention for any mix of portions and single tokens.  ``n_tasks_dev`` (int32 on the device, one
     entry): the lists hold that many tasks, at most ``n_tasks``, for which the grid is made."""
     if task_req.numel() < n_tasks or task_tok0.numel() < n_tasks:
@@ -475,8 +515,8 @@ def attention_prefill(q, out, cache, block_table, q_start, ctx_len, task_req, ta
     if n_tasks_dev is not None:
         _gpu(n_tasks_dev)
         _i32(n_tasks_dev, "n_tasks_dev")
-    lib = build.load("attention_mfma" if head_slopes is None else "attention_mfma_bias")
-    more = () if head_slopes is None else (_ptr(head_slopes), _ptr(sinks))
+    lib = build.load(_attention_library(head_slopes, softcap))
+    more = (_ptr(head_slopes), _ptr(sinks)) if head_slopes is not None else (ctypes.c_float(softcap),) if softcap else ()
     _check(lib.lcu_attention_prefill_bf16(_ptr(q), q.stride(0), _ptr(out), out.stride(0), _ptr(cache),
                                           ctypes.c_longlong(cache.shape[0]), _ptr(block_table),
                                           block_table.shape[1], _ptr(q_start), _ptr(ctx_len), _ptr(task_req),
@@ -500,7 +540,7 @@ class AttentionPlan:
         return (self.max_tasks, self.per_wg, self.n_single, self.single_splits)
 
 
-def plan_attention(step, n_heads: int, n_kv_heads: int, window: int = 0, biased: bool = False) -> Optional[AttentionPlan]:
+def plan_attention(step, n_heads: int, n_kv_heads: int, window: int = 0, biased: bool = False, capped: bool = False) -> Optional[AttentionPlan]:
     """The AttentionPlan of ``step`` for layers with these heads and this window (one per step and kind of layer,
     kept in ``step.scratch``); None for a step of single tokens only, which needs none.  Called before the step's
     arrays go to the device (``Part.prepare``) it lays its lists into the step's own memory (``step.extra``): their
@@ -509,7 +549,7 @@ def plan_attention(step, n_heads: int, n_kv_heads: int, window: int = 0, biased:
     if step.decode_only:
         return None
     # (the library whose kernels will run is asked: a model with a bias inside its scores needs the other one for nothing)
-    lib = build.load("attention_mfma_bias" if biased else "attention_mfma")
+    lib = build.load("attention_mfma_bias" if biased else "attention_mfma_cap" if capped else "attention_mfma")
     tpt = lib.lcu_attention_prefill_tokens_per_task(n_heads, n_kv_heads)
     if tpt <= 0:
         return None
@@ -590,12 +630,13 @@ def _zero_slopes(n_heads: int, device) -> torch.Tensor:
 def paged_attention(q: torch.Tensor, out: torch.Tensor, cache: torch.Tensor, step, group: int, n_heads: int,
                     n_kv_heads: int, head_dim: int, page_size: int, scale: float, window: int = 0,
                     force_generic: bool = False, head_slopes: Optional[torch.Tensor] = None, value_dim: int = 0,
-                    chunk: int = 0, sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+                    chunk: int = 0, sinks: Optional[torch.Tensor] = None, softcap: float = 0.0) -> torch.Tensor:
     """Attention for the batch ``step`` (an engine.batch.StepContext) over cache group
     ``group``: picks the kernel for the batch's shape and type.  ``chunk``: keys of the query's own chunk of so many
     positions only (the matrix-core kernels take it as a negative window).  With a bias inside the scores
     (``head_slopes``) or with ``sinks`` (``exp(sink[h])`` in the denominator of head ``h``'s softmax) the matrix-core
-    kernels are those of the second library, which need a positive scale."""
+    kernels are those of the second library, which need a positive scale.  ``softcap``: a scaled score ``s`` becomes
+    ``softcap * tanh(s / softcap)`` (the third library; together with a bias or sinks the generic kernel)."""
     bt = step.block_table(group)
     if sinks is not None:
         _gpu(sinks)
@@ -608,10 +649,12 @@ def paged_attention(q: torch.Tensor, out: torch.Tensor, cache: torch.Tensor, ste
     if chunk and window:
         raise KernelError("attention: a window and chunks together are not supported")
     second = head_slopes is not None or sinks is not None          # the library with the bias and the sinks
-    if force_generic or (second and not scale > 0) or (value_dim and value_dim != head_dim) \
+    if softcap < 0:
+        raise KernelError(f"attention: the cap on the scores {softcap} must be positive (or 0 for none)")
+    if force_generic or (second and (softcap or not scale > 0)) or (value_dim and value_dim != head_dim) \
             or not mfma_attention_supported(q, n_heads, n_kv_heads, head_dim, page_size):
         return paged_attention_generic(q, out, cache, bt, step.q_start, step.ctx_len, step.req_of_token, n_heads,
-                                       n_kv_heads, head_dim, page_size, scale, window, head_slopes, value_dim, chunk, sinks)
+                                       n_kv_heads, head_dim, page_size, scale, window, head_slopes, value_dim, chunk, sinks, softcap)
     n = _attention_args(q, out, cache, bt, step.q_start, step.ctx_len, step.req_of_token, n_heads, n_kv_heads, head_dim,
                         page_size)
     if chunk:
@@ -623,17 +666,18 @@ def paged_attention(q: torch.Tensor, out: torch.Tensor, cache: torch.Tensor, ste
         # the workgroups start in the order of the requests' list: the requests with the most keys first, where the
         # batch says which they are (64 requests of 150 to 2,200 keys: the step 11.2 -> 11.0 ms)
         return attention_decode(q, out, cache, bt, step.q_start, step.ctx_len, step.n_req, n_heads, n_kv_heads, head_dim,
-                                page_size, scale, window, splits, req_list=step.decode_order, head_slopes=head_slopes, sinks=sinks)
+                                page_size, scale, window, splits, req_list=step.decode_order, head_slopes=head_slopes, sinks=sinks,
+                                softcap=softcap)
     # a mixed batch: the requests that decode one token go to the decode kernel, the portions
     # to the prefill kernel (each would be slow at the other's work)
-    plan = plan_attention(step, n_heads, n_kv_heads, window, biased=second)
+    plan = plan_attention(step, n_heads, n_kv_heads, window, biased=second, capped=bool(softcap))
     if plan.n_single:
         attention_decode(q, out, cache, bt, step.q_start, step.ctx_len, plan.n_single, n_heads, n_kv_heads, head_dim, page_size,
-                         scale, window, plan.single_splits, req_list=plan.singles, head_slopes=head_slopes, sinks=sinks)
+                         scale, window, plan.single_splits, req_list=plan.singles, head_slopes=head_slopes, sinks=sinks, softcap=softcap)
     if plan.max_tasks:
         attention_prefill(q, out, cache, bt, step.q_start, step.ctx_len, plan.task_req, plan.task_tok0, plan.max_tasks,
                           plan.per_wg, n_heads, n_kv_heads, head_dim, page_size, scale, window, n_tasks_dev=plan.n_tasks_dev,
-                          head_slopes=head_slopes, sinks=sinks)
+                          head_slopes=head_slopes, sinks=sinks, softcap=softcap)
     return out
 
 
@@ -715,9 +759,10 @@ def gemm_skinny(x: torch.Tensor, w: torch.Tensor, out: Optional[torch.Tensor] = 
                 out_dtype: Optional[torch.dtype] = None, accumulate: bool = False, swiglu: bool = False,
                 tiles: Optional[int] = None, waves: Optional[int] = None,
                 row_sumsq: Optional[torch.Tensor] = None, norm_width: int = 0, eps: float = 0.0,
-                packed: bool = False) -> torch.Tensor:
+                packed: bool = False, act_alpha: float = 1.0, act_limit: float = 0.0) -> torch.Tensor:
     """``out (+)= x @ w.T`` for at most 32 rows of bfloat16 ``x`` by streaming ``w`` once.
-    ``swiglu``: ``w`` holds gate rows, then up rows; ``out = silu(x @ gate.T) * (x @ up.T)``.
+    ``swiglu``: ``w`` holds gate rows, then up rows; ``out = silu(x @ gate.T) * (x @ up.T)``, or, with ``act_limit`` > 0,
+    the limited activation of ``swiglu`` with ``act_alpha``.
     ``row_sumsq [m, parts]``: the rows of ``x`` wait for their normalisation (see
     ``gemm_skinny_add_norm``); row ``i`` of the product is multiplied by
     ``rsqrt(sum(row_sumsq[i]) / norm_width + eps)`` before the epilogue.
@@ -755,11 +800,52 @@ def gemm_skinny(x: torch.Tensor, w: torch.Tensor, out: Optional[torch.Tensor] = 
             raise KernelError("gemm_skinny: row_sumsq must be a contiguous float32 [rows, parts] tensor, with the norm's width")
         _check(lib.lcu_gemm_skinny_bf16_scaled(_ptr(x), x.stride(0), _ptr(w), w.stride(0), _ptr(out), out.stride(0), m, n, k,
                                                _EPILOGUES[epi], tiles, waves, int(packed), _ptr(row_sumsq), row_sumsq.shape[1],
-                                               int(norm_width), ctypes.c_float(eps), _stream()), "gemm_skinny (scaled rows)")
+                                               int(norm_width), ctypes.c_float(eps), ctypes.c_float(act_alpha), ctypes.c_float(act_limit),
+                                               _stream()), "gemm_skinny (scaled rows)")
         return out
     _check(lib.lcu_gemm_skinny_bf16(_ptr(x), x.stride(0), _ptr(w), w.stride(0), _ptr(out), out.stride(0), m, n, k,
-                                    _EPILOGUES[epi], tiles, waves, int(packed), _stream()),
+                                    _EPILOGUES[epi], tiles, waves, int(packed), ctypes.c_float(act_alpha), ctypes.c_float(act_limit), _stream()),
            "gemm_skinny")
+    return out
+
+
+def skinny_grouped_supported(x: torch.Tensor, w: torch.Tensor, groups: int) -> bool:
+    """Whether ``gemm_skinny_grouped`` takes ``x [groups, m, k]`` with ``w [groups * rows, k]``."""
+    return (x.dim() == 3 and x.shape[0] == groups and w.shape[0] % groups == 0 and (w.shape[0] // groups) % 16 == 0
+            and x.stride(2) == 1 and x.stride(0) % 8 == 0 and x.stride(1) >= x.shape[2]      # (strides of one group's rows)
+            and skinny_supported(x[0], w, torch.bfloat16))
+
+
+def gemm_skinny_grouped(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, packed: bool = False, gate: Optional[torch.Tensor] = None,
+                        tiles: Optional[int] = None, waves: Optional[int] = None) -> torch.Tensor:
+    """Several products in one launch: rows ``g * rows .. (g + 1) * rows - 1`` of ``w [groups * rows, k]`` multiply ``x[g]`` (``x
+    [groups, m, k]``, at most 32 rows), and ``out [m, groups * rows]`` (bfloat16 or float32) takes the groups side by side.
+    ``gate [m, groups * rows]`` (float32 or bfloat16, bfloat16 output only): the product is multiplied by ``sigmoid(gate)``
+    before it is rounded.  ``packed``: ``w`` is the result of ``pack_weight``."""
+    _gpu(x, w, out, gate)
+    groups, m, k = x.shape
+    n = w.shape[0]
+    if packed and not (packable(w) and w.is_contiguous()):
+        raise KernelError("gemm_skinny_grouped: a packed weight is a contiguous result of pack_weight")
+    _rows(w, "grouped w"); _rows(out, "grouped out")
+    if w.shape[1] != k or not skinny_grouped_supported(x, w, groups):
+        raise KernelError(f"gemm_skinny_grouped: x {tuple(x.shape)} {x.dtype} with w {tuple(w.shape)} {w.dtype} is not supported")
+    if out.shape != (m, n) or out.dtype not in (torch.bfloat16, torch.float32):
+        raise KernelError(f"gemm_skinny_grouped out: {out.dtype} {tuple(out.shape)}, expected bfloat16 or float32 {(m, n)}")
+    if gate is not None:
+        _rows(gate, "grouped gate")
+        if gate.shape != (m, n) or out.dtype != torch.bfloat16:
+            raise KernelError("gemm_skinny_grouped: the gate has the output's shape and goes with bfloat16 output")
+    rows = n // groups
+    tiles = tiles or _skinny_tiles(n, m, packed)
+    while rows % (16 * tiles):
+        tiles //= 2
+    waves = waves or (8 if n <= TUNING.skinny_eight_waves_to and k > 512 else 4)      # (a wave needs a macro-step of 128 to work on)
+    lib = build.load("gemm_skinny")
+    _check(lib.lcu_gemm_skinny_bf16_grouped(_ptr(x), x.stride(1), ctypes.c_longlong(x.stride(0)), _ptr(w), w.stride(0), rows, _ptr(out),
+                                            out.stride(0), m, n, k, _EPILOGUES["f32" if out.dtype == torch.float32 else "bf16"], tiles,
+                                            waves, int(packed), _ptr(gate), F32 if gate is None else _type(gate, "grouped gate"),
+                                            0 if gate is None else gate.stride(0), _stream()), "gemm_skinny_grouped")
     return out
 
 
@@ -785,10 +871,11 @@ def mid_planes(k: int, slices: int) -> int:
 
 def gemm_mid(x: torch.Tensor, w: torch.Tensor, out: Optional[torch.Tensor] = None, swiglu: bool = False,
              slices: Optional[int] = None, packed: bool = False, row_sumsq: Optional[torch.Tensor] = None,
-             norm_width: int = 0, eps: float = 0.0) -> torch.Tensor:
+             norm_width: int = 0, eps: float = 0.0, act_alpha: float = 1.0, act_limit: float = 0.0) -> torch.Tensor:
     """``x @ w.T`` for up to 256 rows of bfloat16 ``x`` (chosen from 12 to 33 rows on, by the product), streaming ``w`` once while
     the waves of a workgroup share ``x`` through LDS.  ``slices=None``: ``out [m, n]`` bfloat16
-    (``swiglu``: ``w`` holds gate rows, then up rows, ``out [m, n/2] = silu(gate) * up``).
+    (``swiglu``: ``w`` holds gate rows, then up rows, ``out [m, n/2] = silu(gate) * up``, or the limited activation with
+    ``act_limit`` > 0).
     ``slices=s``: K is cut into (at most) ``s`` slices and ``out [planes, m, n]`` float32 holds
     each slice's sum; whoever reads it adds the planes (``rmsnorm(..., delta=planes)`` does).
     ``packed``: ``w`` is the result of ``pack_weight``.  ``row_sumsq [m, parts]``: the rows of ``x``
@@ -825,10 +912,10 @@ def gemm_mid(x: torch.Tensor, w: torch.Tensor, out: Optional[torch.Tensor] = Non
                               f"for at most {MID_MAX_SCALED_ROWS} rows")
         _check(lib.lcu_gemm_mid_bf16_scaled(_ptr(x), x.stride(0), _ptr(w), w.stride(0), _ptr(out), out.stride(-2), m, n, k, epi,
                                             slices or 1, int(packed), _ptr(row_sumsq), row_sumsq.shape[1], int(norm_width),
-                                            ctypes.c_float(eps), _stream()), "gemm_mid (scaled rows)")
+                                            ctypes.c_float(eps), ctypes.c_float(act_alpha), ctypes.c_float(act_limit), _stream()), "gemm_mid (scaled rows)")
         return out
     _check(lib.lcu_gemm_mid_bf16(_ptr(x), x.stride(0), _ptr(w), w.stride(0), _ptr(out), out.stride(-2), m, n, k, epi,
-                                 slices or 1, int(packed), _stream()), "gemm_mid")
+                                 slices or 1, int(packed), ctypes.c_float(act_alpha), ctypes.c_float(act_limit), _stream()), "gemm_mid")
     return out
 
 
@@ -836,9 +923,9 @@ ADD_NORM_MAX_ROWS = 32
 
 
 def gemm_skinny_add_norm(x: torch.Tensor, w: torch.Tensor, residual: torch.Tensor, norm_weight: torch.Tensor,
-                         tiles: Optional[int] = None, waves: Optional[int] = None, packed: bool = False):
+                         tiles: Optional[int] = None, waves: Optional[int] = None, packed: bool = False, scale: float = 1.0):
     """The product that ends a branch, the residual sum and the next norm's weight in one
-    kernel: ``residual += x @ w.T`` (float32, in place); returns ``(h, sumsq)`` with
+    kernel: ``residual += scale * (x @ w.T)`` (float32, in place); returns ``(h, sumsq)`` with
     ``h = bfloat16(residual * norm_weight)``, not yet normalised, and ``sumsq [rows, parts]``,
     the workgroups' shares of each row's sum of squares, for ``gemm_skinny(..., row_sumsq=)``.
     At most 32 rows."""
@@ -862,7 +949,7 @@ def gemm_skinny_add_norm(x: torch.Tensor, w: torch.Tensor, residual: torch.Tenso
     lib = build.load("gemm_skinny")
     _check(lib.lcu_gemm_skinny_bf16_add_norm(_ptr(x), x.stride(0), _ptr(w), w.stride(0), _ptr(residual), residual.stride(0),
                                              m, n, k, _ptr(norm_weight), _type(norm_weight, "norm weight"), _ptr(h),
-                                             h.stride(0), _ptr(sumsq), parts, tiles, waves, int(packed), _stream()),
+                                             h.stride(0), _ptr(sumsq), parts, tiles, waves, int(packed), ctypes.c_float(scale), _stream()),
            "gemm_skinny_add_norm")
     return h, sumsq
 
@@ -870,8 +957,9 @@ def gemm_skinny_add_norm(x: torch.Tensor, w: torch.Tensor, residual: torch.Tenso
 MID_ADD_NORM_MAX_ROWS = 64
 
 
-def gemm_mid_add_norm(x: torch.Tensor, w: torch.Tensor, residual: torch.Tensor, norm_weight: torch.Tensor, packed: bool = False):
-    """``gemm_skinny_add_norm`` for up to 64 rows, by the kernel that shares the rows through LDS: ``residual += x @ w.T``
+def gemm_mid_add_norm(x: torch.Tensor, w: torch.Tensor, residual: torch.Tensor, norm_weight: torch.Tensor, packed: bool = False,
+                      scale: float = 1.0):
+    """``gemm_skinny_add_norm`` for up to 64 rows, by the kernel that shares the rows through LDS: ``residual += scale * (x @ w.T)``
     (float32, in place); returns ``(h, sumsq)`` with ``h = bfloat16(residual * norm_weight)``, not yet normalised, and
     ``sumsq [rows, out / 16]``, the workgroups' shares of each row's sum of squares.  A workgroup takes 16 output
     features over all of K and reads every row: for products with a short K (the output projection)."""
@@ -893,7 +981,7 @@ def gemm_mid_add_norm(x: torch.Tensor, w: torch.Tensor, residual: torch.Tensor, 
     lib = build.load("gemm_mid")
     _check(lib.lcu_gemm_mid_bf16_add_norm(_ptr(x), x.stride(0), _ptr(w), w.stride(0), _ptr(residual), residual.stride(0), m, n, k,
                                           _ptr(norm_weight), _type(norm_weight, "norm weight"), _ptr(h), h.stride(0), _ptr(sumsq),
-                                          int(packed), _stream()), "gemm_mid_add_norm")
+                                          int(packed), ctypes.c_float(scale), _stream()), "gemm_mid_add_norm")
     return h, sumsq
 
 
@@ -1345,29 +1433,43 @@ def scaled_sum(acc: Optional[torch.Tensor], x: torch.Tensor, scale: float) -> to
 # ------------------------------------------------------------------ bias, head norm, rotation, cache write
 
 
+QKV_PREPARE_MAX_DIM = 640        # what a head may take in the rows and in the cache
+
+
 def qkv_prepare(rows: torch.Tensor, offsets, n_heads: int, n_kv_heads: int, head_dim: int, value_dim: int, stored_dim: int,
                 stored_value_dim: int, dtype: torch.dtype, positions: Optional[torch.Tensor] = None,
                 bias: Optional[torch.Tensor] = None, q_norm: Optional[torch.Tensor] = None, k_norm: Optional[torch.Tensor] = None,
                 eps: float = 0.0, cos: Optional[torch.Tensor] = None, sin: Optional[torch.Tensor] = None, rot_dim: int = 0,
                 pairing: int = 0, cache: Optional[torch.Tensor] = None, slots: Optional[torch.Tensor] = None,
-                page_size: int = 16) -> torch.Tensor:
+                page_size: int = 16, maps: int = 1, joint: bool = False) -> torch.Tensor:
     """What stands between a q, k, v product and its attention, each piece optional: ``rows [n, *]`` holds the product
     with q at column ``offsets[0]`` (``n_heads * head_dim``), k at ``offsets[1]``, v at ``offsets[2]`` (``n_kv_heads *
     value_dim``); ``bias`` (float32 over the rows' columns) is added; q and k are divided by the root mean square over
     each head and multiplied by ``q_norm`` / ``k_norm`` (float32 ``[head_dim]``); the first ``rot_dim`` dims of every q and
     k head are rotated (tables ``cos``, ``sin``; ``pairing`` 0: halves, 1: neighbours).  Returns q as ``[n, n_heads *
     stored_dim]`` of ``dtype`` and writes k and v into ``cache`` at ``slots`` with ``stored_dim`` / ``stored_value_dim`` dims
-    a head, the dims beyond the true ones zeros.  ``cache=None``: queries only."""
+    a head, the dims beyond the true ones zeros.  ``cache=None``: queries only.
+    ``maps`` > 1: every query and key head is ``maps`` vectors of ``head_dim`` side by side, each normed and rotated by itself,
+    over the head's one set of values; ``n_heads`` and ``n_kv_heads`` count (head, map) pairs, and the kernels behind see
+    one plain head per pair.  ``joint``: a stored key is its maps' keys side by side (``n_kv_heads / maps`` stored heads of
+    ``maps * head_dim`` or more dims) and the query of map ``m`` has zeros outside its map's dims, queries in the order
+    (head, map).  Else every (key head, map) is a stored head of its own with a copy of the values, queries in the order
+    (key head, map, head of the group)."""
+    if maps < 1 or n_heads % maps or n_kv_heads % maps or (maps > 1 and cache is None) or (joint and maps < 2):
+        raise KernelError(f"qkv_prepare: {maps} maps do not fit {n_heads} query and {n_kv_heads} key heads (and need a cache to write to)")
+    joint_dim = maps * head_dim if joint else head_dim
+    stored_heads = n_kv_heads // maps if joint else n_kv_heads
+    value_heads = n_kv_heads // maps                          # that the rows hold
     _gpu(rows, positions, bias, q_norm, k_norm, cos, sin, cache, slots)
     _rows(rows, "qkv rows")
     n, width = rows.shape
     store = cache is not None
     q_off, k_off, v_off = (int(o) for o in offsets)
     if q_off < 0 or q_off + n_heads * head_dim > width or (store and (k_off < 0 or k_off + n_kv_heads * head_dim > width
-                                                                      or v_off < 0 or v_off + n_kv_heads * value_dim > width)):
+                                                                      or v_off < 0 or v_off + value_heads * value_dim > width)):
         raise KernelError(f"qkv_prepare: the columns of q, k or v lie outside the rows' {width} columns")
-    if stored_dim % 8 or stored_dim < head_dim or stored_value_dim < value_dim or max(stored_dim, stored_value_dim) > 256:
-        raise KernelError(f"qkv_prepare: stored head sizes {stored_dim} / {stored_value_dim} do not fit {head_dim} / {value_dim} (keys a multiple of 8, at most 256)")
+    if stored_dim % 8 or stored_dim < joint_dim or stored_value_dim < value_dim or max(stored_dim, stored_value_dim) > QKV_PREPARE_MAX_DIM:
+        raise KernelError(f"qkv_prepare: stored head sizes {stored_dim} / {stored_value_dim} do not fit {joint_dim} / {value_dim} (keys a multiple of 8, at most {QKV_PREPARE_MAX_DIM})")
     _f32_vec(bias, "qkv bias", width); _f32_vec(q_norm, "query norm weight", head_dim); _f32_vec(k_norm, "key norm weight", head_dim)
     max_pos = 0
     if cos is not None:
@@ -1379,14 +1481,14 @@ def qkv_prepare(rows: torch.Tensor, offsets, n_heads: int, n_kv_heads: int, head
     if store:
         _i32(slots, "cache slots", n)
         _contig(cache, "cache")
-        if cache.dtype != dtype or cache.dim() != 3 or cache.shape[1] * cache.shape[2] != n_kv_heads * (stored_dim + stored_value_dim) * page_size:
-            raise KernelError(f"cache: {cache.dtype} {tuple(cache.shape)} does not hold pages of {n_kv_heads} x ({stored_dim} + {stored_value_dim}) x {page_size} {dtype}")
+        if cache.dtype != dtype or cache.dim() != 3 or cache.shape[1] * cache.shape[2] != stored_heads * (stored_dim + stored_value_dim) * page_size:
+            raise KernelError(f"cache: {cache.dtype} {tuple(cache.shape)} does not hold pages of {stored_heads} x ({stored_dim} + {stored_value_dim}) x {page_size} {dtype}")
     q = torch.empty((n, n_heads * stored_dim), dtype=dtype, device=rows.device)
     lib = build.load("qkv_prepare")
     _check(lib.lcu_qkv_prepare(_ptr(rows), _type(rows, "qkv rows"), n, rows.stride(0), q_off, k_off, v_off, _ptr(bias), _ptr(q_norm),
                                _ptr(k_norm), ctypes.c_float(eps), _ptr(positions), _ptr(cos), _ptr(sin), max_pos, int(rot_dim), int(pairing),
                                _ptr(q), _type(q, "q"), _ptr(slots), _ptr(cache), n_heads, n_kv_heads if store else 0, head_dim,
-                               stored_dim, value_dim, stored_value_dim, page_size, int(store), _stream()), "qkv_prepare")
+                               stored_dim, value_dim, stored_value_dim, page_size, int(store), int(maps), int(bool(joint)), _stream()), "qkv_prepare")
     return q
 
 
@@ -1403,21 +1505,38 @@ def head_gate(out: torch.Tensor, gate_rows: torch.Tensor, g_off: int, n_heads: i
     return out
 
 
-def latent_prepare(rows: torch.Tensor, q_out: torch.Tensor, n_heads: int, q_head_stride: int, q_rot_off: int, kv_off: int,
-                   rank: int, rot: int, stored_dim: int, stored_value_dim: int, positions: torch.Tensor, cos: torch.Tensor,
-                   sin: torch.Tensor, c_norm: Optional[torch.Tensor] = None, eps: float = 0.0,
-                   cache: Optional[torch.Tensor] = None, slots: Optional[torch.Tensor] = None, page_size: int = 16) -> torch.Tensor:
+def latent_prepare(rows: torch.Tensor, q_out: Optional[torch.Tensor], n_heads: int, q_head_stride: int, q_rot_off: int, kv_off: int,
+                   rank: int, rot: int, stored_dim: int, stored_value_dim: int, positions: Optional[torch.Tensor],
+                   cos: Optional[torch.Tensor], sin: Optional[torch.Tensor], c_norm: Optional[torch.Tensor] = None, eps: float = 0.0,
+                   cache: Optional[torch.Tensor] = None, slots: Optional[torch.Tensor] = None, page_size: int = 16,
+                   cq_off: int = 0, cq_norm: Optional[torch.Tensor] = None, cq_out: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
     """Latent attention between its input product and the attention over the cache.  ``rows [n, *]``: query head ``h``'s
     turned part at column ``h * q_head_stride + q_rot_off`` (``rot`` columns), the latent product at ``kv_off`` (``rank +
     rot`` columns).  ``q_out [n, n_heads * stored_dim]`` holds every head's folded plain part in its first ``rank``
     columns already; the rotated turned part is written behind it, zeros behind that.  With ``cache``: the latent's first
     ``rank`` columns, divided by their root mean square and multiplied by ``c_norm`` (float32), and the rotated last ``rot``
     go to the token's place in its page as the one key head ``[c, r]`` (``stored_dim`` dims) with the value ``c``
-    (``stored_value_dim`` dims).  The rotation pairs dim ``i`` with ``i + rot / 2``."""
-    _gpu(rows, q_out, positions, cos, sin, c_norm, cache, slots)
-    _rows(rows, "latent rows"); _rows(q_out, "folded queries"); _contig(q_out, "folded queries")
+    (``stored_value_dim`` dims).  The rotation pairs dim ``i`` with ``i + rot / 2``.  ``rot`` 0: no turned parts (``q_out``,
+    ``positions`` and the tables are not used).  ``cq_out [n, q_rank]``: the queries' own latent at column ``cq_off``, divided by
+    its root mean square and multiplied by ``cq_norm`` (float32)."""
+    _gpu(rows, q_out, positions, cos, sin, c_norm, cache, slots, cq_norm, cq_out)
+    _rows(rows, "latent rows")
     n, width = rows.shape
     store = cache is not None
+    q_rank = 0
+    if cq_out is not None:
+        _rows(cq_out, "query latent"); _contig(cq_out, "query latent")
+        q_rank = cq_out.shape[1]
+        _f32_vec(cq_norm, "query latent norm weight", q_rank)
+        if cq_norm is None or cq_out.shape[0] != n or cq_off < 0 or cq_off + q_rank > width:
+            raise KernelError(f"latent_prepare: the queries' latent lies outside the rows' {width} columns, or has no norm weight")
+    out_type = q_out if q_out is not None else cq_out if cq_out is not None else cache
+    if out_type is None or any(x is not None and x.dtype != out_type.dtype for x in (q_out, cq_out, cache)):
+        raise KernelError("latent_prepare: the queries, the queries' latent and the cache have one type")
+    if rot == 0:
+        return _latent_prepare_unturned(rows, n, width, n_heads, kv_off, rank, stored_dim, stored_value_dim, c_norm, eps, cache, slots,
+                                        page_size, cq_off, q_rank, cq_norm, cq_out, out_type)
+    _rows(q_out, "folded queries"); _contig(q_out, "folded queries")
     if q_out.shape != (n, n_heads * stored_dim) or stored_dim % 8 or rank + rot > stored_dim or stored_value_dim < rank \
             or max(stored_dim, stored_value_dim) > 640 or rot % 2 or rot < 2:
         raise KernelError(f"latent_prepare: queries {tuple(q_out.shape)} do not fit {n_heads} heads of {stored_dim} holding {rank} + {rot}")
@@ -1440,8 +1559,139 @@ def latent_prepare(rows: torch.Tensor, q_out: torch.Tensor, n_heads: int, q_head
                                   int(kv_off), _ptr(c_norm), ctypes.c_float(eps), _ptr(positions), _ptr(cos), _ptr(sin),
                                   cos.shape[0], _ptr(q_out), _type(q_out, "folded queries"), _ptr(slots), _ptr(cache), n_heads,
                                   int(rank), int(rot), int(stored_dim), int(stored_value_dim), int(page_size), int(store),
-                                  _stream()), "latent_prepare")
+                                  int(cq_off), q_rank, _ptr(cq_norm), _ptr(cq_out), _stream()), "latent_prepare")
     return q_out
+
+
+def _latent_prepare_unturned(rows, n, width, n_heads, kv_off, rank, stored_dim, stored_value_dim, c_norm, eps, cache, slots, page_size,
+                             cq_off, q_rank, cq_norm, cq_out, out_type):
+    """``latent_prepare`` without turned parts: the latent's norm and cache write, the queries' latent's norm."""
+    if stored_dim % 8 or rank > stored_dim or stored_value_dim < rank or max(stored_dim, stored_value_dim) > 640 or rank < 1:
+        raise KernelError(f"latent_prepare: stored sizes {stored_dim} / {stored_value_dim} do not hold a latent of {rank} (at most 640)")
+    if cache is not None:
+        _f32_vec(c_norm, "latent norm weight", rank)
+        if c_norm is None or kv_off < 0 or kv_off + rank > width:
+            raise KernelError(f"latent_prepare: the latent lies outside the rows' {width} columns, or has no norm weight")
+        _i32(slots, "cache slots", n)
+        _contig(cache, "cache")
+        if cache.dim() != 3 or cache.shape[1] * cache.shape[2] != (stored_dim + stored_value_dim) * page_size:
+            raise KernelError(f"cache: {cache.dtype} {tuple(cache.shape)} does not hold pages of ({stored_dim} + {stored_value_dim}) x {page_size}")
+    lib = build.load("latent")
+    _check(lib.lcu_latent_prepare(_ptr(rows), _type(rows, "latent rows"), n, rows.stride(0), 0, 0, int(kv_off), _ptr(c_norm),
+                                  ctypes.c_float(eps), _ptr(None), _ptr(None), _ptr(None), 0, _ptr(None), _type(out_type, "latent output"),
+                                  _ptr(slots), _ptr(cache), n_heads, int(rank), 0, int(stored_dim), int(stored_value_dim), int(page_size),
+                                  int(cache is not None), int(cq_off), q_rank, _ptr(cq_norm), _ptr(cq_out), _stream()), "latent_prepare")
+    return cq_out
+
+
+# ------------------------------------------------------------------ between attention and its output product
+
+
+def element_gate(x: torch.Tensor, gate: torch.Tensor, heads: int, value_dim: int, head_stride: int = 0) -> torch.Tensor:
+    """``x[t, h, :value_dim] * sigmoid(gate[t, h * value_dim + ...])`` as ``[n, heads * value_dim]`` of ``x``'s type; head ``h``
+    of ``x`` starts at column ``h * head_stride`` (0: the heads side by side)."""
+    _gpu(x, gate)
+    _rows(x, "gated rows"); _rows(gate, "gate rows")
+    n, stride = x.shape[0], int(head_stride or value_dim)
+    if stride < value_dim or x.shape[1] < (heads - 1) * stride + value_dim or gate.shape != (n, heads * value_dim):
+        raise KernelError(f"element_gate: {heads} heads of {value_dim} do not fit rows {tuple(x.shape)} and a gate {tuple(gate.shape)}")
+    out = torch.empty((n, heads * value_dim), dtype=x.dtype, device=x.device)
+    lib = build.load("head_mix")
+    _check(lib.lcu_element_gate(_ptr(x), _type(x, "gated rows"), stride, x.stride(0), _ptr(gate), _type(gate, "gate rows"), gate.stride(0),
+                                _ptr(out), n, heads, value_dim, _stream()), "element_gate")
+    return out
+
+
+def two_maps(x: torch.Tensor, heads: int, value_dim: int, lam: float, eps: float, factor: float, gate: Optional[torch.Tensor] = None,
+             head_stride: int = 0, map_group: int = 1) -> torch.Tensor:
+    """Two attentions per head over the same values, joined: ``o = a1 - lam * a2``, ``o / sqrt(mean(o^2) + eps) * factor``, times
+    ``sigmoid(gate)`` (``[n, heads * value_dim]``) if given; ``[n, heads * value_dim]`` of ``x``'s type.  ``x [n, 2 * heads *
+    head_stride]``: ``map_group`` 1: a head's two maps side by side; g: the first maps of g heads, then their second ones."""
+    _gpu(x, gate)
+    _rows(x, "maps")
+    n, stride = x.shape[0], int(head_stride or value_dim)
+    if stride < value_dim or x.shape[1] != 2 * heads * stride or heads % map_group or value_dim > 640:
+        raise KernelError(f"two_maps: {heads} heads of {value_dim} (at most 640) in groups of {map_group} do not fit rows {tuple(x.shape)}")
+    if gate is not None:
+        _rows(gate, "gate rows")
+        if gate.shape != (n, heads * value_dim):
+            raise KernelError(f"two_maps: the gate must be {(n, heads * value_dim)}")
+    out = torch.empty((n, heads * value_dim), dtype=x.dtype, device=x.device)
+    lib = build.load("head_mix")
+    _check(lib.lcu_two_maps(_ptr(x), _type(x, "maps"), stride, x.stride(0), int(map_group), ctypes.c_float(lam), ctypes.c_float(eps),
+                            ctypes.c_float(factor), _ptr(gate), _type(x if gate is None else gate, "gate rows"),
+                            0 if gate is None else gate.stride(0), _ptr(out), n, heads, value_dim, _stream()), "two_maps")
+    return out
+
+
+# ------------------------------------------------------------------ a time mixer with a decay per key channel
+
+
+def token_shift(h: torch.Tensor, mu: torch.Tensor, state: torch.Tensor, offset: int, step, out_dtype: torch.dtype) -> torch.Tensor:
+    """``out[s, t] = h[t] + (h[t - 1] - h[t]) * mu[s]`` for ``h`` float32 ``[n, d]`` and ``mu`` float32 ``[sets, d]``: ``[sets, n, d]`` in
+    ``out_dtype``.  The row in front of a request's first token of the step is the one that ``state [slots, *]`` (float32)
+    holds from column ``offset`` on (zeros at position 0), and the step's last row is left there."""
+    _gpu(h, mu, state)
+    _rows(h, "token_shift h"); _contig(h, "token_shift h"); _rows(mu, "token_shift mu"); _contig(mu, "token_shift mu")
+    n, d = h.shape
+    if h.dtype != torch.float32 or mu.dtype != torch.float32 or mu.shape[1] != d:
+        raise KernelError("token_shift: h and mu must be float32 of one width")
+    if state.dtype != torch.float32 or state.dim() != 2 or state.stride(1) != 1 or offset < 0 or offset + d > state.shape[1]:
+        raise KernelError(f"token_shift: the state {tuple(state.shape)} does not hold {d} floats from column {offset} on")
+    if n != step.n or max(step.state_slots, default=0) >= state.shape[0]:
+        raise KernelError("token_shift: the rows are not the step's, or a request's slot lies outside the state")
+    out = torch.empty((mu.shape[0], n, d), dtype=out_dtype, device=h.device)
+    lib = build.load("wkv")
+    _check(lib.lcu_token_shift(_ptr(h), _ptr(mu), mu.shape[0], _ptr(state[:, offset:]), ctypes.c_longlong(state.stride(0)),
+                               _ptr(step.req_of_token), _ptr(step.q_start), _ptr(step.ctx_len), _ptr(step.state_slot), _ptr(out),
+                               _type(out, "token_shift out"), n, d, _stream()), "token_shift")
+    return out
+
+
+def wkv(rows: torch.Tensor, offsets: Dict[str, int], low: torch.Tensor, w2_t: torch.Tensor, w0: torch.Tensor, u: torch.Tensor,
+        norm: torch.Tensor, state: torch.Tensor, step, heads: int, dim: int, eps: float, out_dtype: torch.dtype) -> torch.Tensor:
+    """The recurrence of a time mixer between its projections and its output product, request by request from each
+    request's state (the first ``heads * dim * dim`` floats of ``state [slots, *]``, float32; taken as zero at a request's position 0
+    and left as the step's last token makes it).  ``rows [n, *]`` holds r, k, v, g (``heads * dim`` columns each) at ``offsets``;
+    ``low [n, rank]`` float32 the decay's low-rank projection, ``w2_t [rank, heads * dim]``, ``w0``, ``u``, ``norm`` ``[heads * dim]``
+    float32.  Per head ``w = exp(-exp(w2 tanh(low) + w0))``, ``o = (S + diag(u) k v^T)^T r``, ``S <- diag(w) S + k v^T``; returns ``o``
+    divided by its root mean square per head, times ``norm``, times ``silu(g)``, ``[n, heads * dim]`` in ``out_dtype``."""
+    _gpu(rows, low, w2_t, w0, u, norm, state)
+    _rows(rows, "wkv rows"); _rows(low, "wkv low")
+    n, width = rows.shape
+    hd, rank = heads * dim, low.shape[1]
+    for name in ("r", "k", "v", "g"):
+        if name not in offsets or offsets[name] < 0 or offsets[name] + hd > width:
+            raise KernelError(f"wkv: the columns of {name!r} lie outside the rows' {width} columns")
+    if low.dtype != torch.float32 or low.shape[0] != n:
+        raise KernelError("wkv: the low-rank rows must be float32, one for every row")
+    if w2_t.dtype != torch.float32 or w2_t.shape != (rank, hd) or not w2_t.is_contiguous():
+        raise KernelError(f"wkv: w2_t must be contiguous float32 {(rank, hd)}")
+    _f32_vec(w0, "wkv w0", hd); _f32_vec(u, "wkv u", hd); _f32_vec(norm, "wkv norm weight", hd)
+    if dim > 256 or rank > 512:
+        raise KernelError(f"wkv: heads of {dim} or a decay of rank {rank} are not supported (at most 256 and 512)")
+    if state.dtype != torch.float32 or state.dim() != 2 or state.stride(1) != 1 or state.shape[1] < heads * dim * dim:
+        raise KernelError(f"wkv: state must be float32 [slots, at least {heads * dim * dim}]")
+    if n != step.n or max(step.state_slots, default=0) >= state.shape[0]:
+        raise KernelError("wkv: the rows are not the step's, or a request's slot lies outside the state")
+    out = torch.empty((n, hd), dtype=out_dtype, device=rows.device)
+    lib = build.load("wkv")
+    head = (_ptr(rows), _type(rows, "wkv rows"), rows.stride(0), offsets["r"], offsets["k"], offsets["v"], offsets["g"], _ptr(low),
+            low.stride(0), _ptr(w2_t), _ptr(w0), _ptr(u), _ptr(norm))
+    slot = (_ptr(state), ctypes.c_longlong(state.stride(0)), _ptr(out), _type(out, "wkv out"), _ptr(step.q_start), _ptr(step.ctx_len),
+            _ptr(step.state_slot))
+    if step.decode_only:
+        _check(lib.lcu_wkv_single(*head, *slot, step.n_req, heads, dim, dim, rank, ctypes.c_float(eps), _stream()), "wkv (single tokens)")
+        return out
+    for f in (lib.lcu_wkv_prep_floats, lib.lcu_wkv_out_floats, lib.lcu_wkv_run_floats):
+        f.restype = ctypes.c_longlong
+    n_long = sum(1 for q in step.q_lens if q >= lib.lcu_wkv_long())
+    f32 = lambda size: torch.empty(size, dtype=torch.float32, device=rows.device)
+    prep, o = f32(lib.lcu_wkv_prep_floats(n, heads, dim, dim)), f32(lib.lcu_wkv_out_floats(n, heads, dim))
+    runs = f32(lib.lcu_wkv_run_floats(n_long, heads, dim, dim)) if n_long else None
+    _check(lib.lcu_wkv(*head, _ptr(prep), _ptr(o), _ptr(runs), n_long, *slot, n, step.n_req, heads, dim, dim, rank, ctypes.c_float(eps),
+                       _stream()), "wkv")
+    return out
 
 
 # ------------------------------------------------------------------ retention

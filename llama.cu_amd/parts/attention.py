@@ -347,7 +347,7 @@ class Attention(Part):
             return linear(out, self.w_o, out_dtype=out_dtype)
         if into is not None:
             residual, norm = into
-            fused = linear_into_norm(out, self.w_o, residual, norm.weight)
+            fused = linear_into_norm(out, self.w_o, residual, norm.weight, scale=norm.delta_scale)
             if fused is not None:
                 return ScaledRows(fused[0], fused[1], norm.size, norm.eps)
         if planes_ok and self.dtype == torch.bfloat16 and mid_takes(n_rows, self.w_o):

@@ -14,6 +14,8 @@ the registry of its category:
   ``ffn``       ``forward(h) -> delta``
   ``position``  ``tables(...)``/``apply(...)``         see parts.position
   ``block``     ``forward(x, pending, step, cache) -> pending``   the arrangement of the four above
+  ``stream``    ``forward(x, pending, start) -> x``     a change of the residual stream between two layers; ``start`` is what
+                ``begin(x)`` made of the embedding's output
 
 Every part also has ``tensors() -> {relative name: TensorSpec}``,
 ``load(tensors, build)`` and the flag ``graph_safe`` (see Part).  No part knows which model it is in: sizes and constants
@@ -51,9 +53,11 @@ class PartSpec:
 class RunEntry:
     """One step of the run order: which layer runs, and whose cache it uses.  ``cache_of``
     None: a cache of its own.  ``cache_of = j``: it reads the cache that entry ``j`` of the
-    run order wrote (and writes none)."""
+    run order wrote (and writes none).  ``before = k``: the residual stream passes the model's stream
+    part ``k`` (``ModelSpec.streams``) right before the layer runs."""
     layer: int
     cache_of: Optional[int] = None
+    before: Optional[int] = None
 
 
 @dataclass
@@ -68,6 +72,7 @@ class ModelSpec:
     final_norm: PartSpec
     head: PartSpec
     eos_token_ids: Tuple[int, ...] = ()
+    streams: List[PartSpec] = field(default_factory=list)    # changes of the stream that entries of the run order name
 
 
 # ------------------------------------------------------------------ cache needs
@@ -240,11 +245,14 @@ class Part:
     # norm:  ``deferrable``: the norm is a factor per row times a weight per column (``weight``, ``size``,
     #        ``eps``), so the factor may be applied after the next matrix product (ScaledRows);
     #        ``takes_planes``: ``forward(x, delta)`` also takes float32 planes ``[planes, rows, width]``
-    #        of partial sums as ``delta``.
+    #        of partial sums as ``delta``;
+    #        ``delta_scale``: what ``delta`` is multiplied by before it is added to the stream, also by a
+    #        product that ends in this norm.
     # mixer, feed-forward:  ``ends_in_norm``: ``forward(..., into=(residual, norm))`` may add its output to
     #        the residual stream itself and return ScaledRows made with ``norm``;
     #        ``ends_in_planes``: ``forward(..., planes_ok=True)`` may return float32 planes;
-    #        ``takes_scaled_rows(n_rows)``: whether ``forward`` takes ScaledRows of that many rows.
+    #        ``takes_scaled_rows(n_rows)``: whether ``forward`` takes ScaledRows of that many rows;
+    #        ``reads_float32``: a mixer whose rows go on in 32-bit: the block's norm writes float32 rows for it.
     # block: ``ends_in_next_norm``: ``forward(..., next_norm=)`` may end in the norm that follows the block;
     #        ``ends_in_planes`` / ``takes_planes`` / ``takes_scaled_rows`` as above, for its last branch
     #        and its first norm.
@@ -252,6 +260,8 @@ class Part:
     #        norm in the same kernel and returns NormedRows; ``takes_normed_rows``: ``pending`` may be NormedRows
     #        made with its ``first_norm``.
     deferrable = False
+    delta_scale = 1.0
+    reads_float32 = False
     takes_planes = False
     ends_in_norm = False
     ends_in_planes = False
@@ -314,7 +324,8 @@ class Part:
 
 
 _REGISTRIES: Dict[str, Dict[str, Callable[..., Part]]] = {
-    "norm": {}, "mixer": {}, "ffn": {}, "position": {}, "block": {}, "embedding": {}, "head": {}}
+    "norm": {}, "mixer": {}, "ffn": {}, "position": {}, "block": {}, "embedding": {}, "head": {},
+    "stream": {}}
 
 
 def register_part(category: str, kind: str, factory: Callable[..., Part], replace: bool = False) -> None:

@@ -3,7 +3,8 @@
 ``parallel``: ``x += mixer(norm1(x)) + ffn(norm2(x))``, both branches reading the same ``x``, each
 optionally through a short causal convolution over time (ParallelBlock below).
 
-``prenorm``: ``x += mixer(norm1(x)); x += ffn(norm2(x))``
+``prenorm``: ``x += mixer(norm1(x)); x += ffn(norm2(x))`` (the feed-forward, with its norm, may be missing; a factor on
+both outputs is the ``delta_scale`` of the norms that add them)
 (llama.cu/src/model/mod.rs:100-157, ``TransformerBlk::new(norm, attention, norm, mlp)``;
 the residual is added where the output and down projections end,
 llama.cu/src/op/linear.rs:35-62).  Here the residual stream ``x`` is float32 and each
@@ -22,18 +23,20 @@ from .norm import LayerNorm, NoNorm
 
 
 class PreNormBlock(Part):
-    def __init__(self, norm1: PartSpec, mixer: PartSpec, norm2: PartSpec, ffn: PartSpec):
+    def __init__(self, norm1: PartSpec, mixer: PartSpec, norm2: Optional[PartSpec] = None, ffn: Optional[PartSpec] = None):
+        if (norm2 is None) != (ffn is None):
+            raise ValueError("prenorm block: the second norm and the feed-forward come together or not at all")
         self.specs = {"norm1": norm1, "mixer": mixer, "norm2": norm2, "ffn": ffn}
         self.norm1 = make_part("norm", norm1)
         self.mixer = make_part("mixer", mixer)
-        self.norm2 = make_part("norm", norm2)
-        self.ffn = make_part("ffn", ffn)
-        self.graph_safe = all(p.graph_safe for p in (self.norm1, self.mixer, self.norm2, self.ffn))
+        self.norm2 = make_part("norm", norm2) if norm2 is not None else None
+        self.ffn = make_part("ffn", ffn) if ffn is not None else None
+        self.graph_safe = all(p.graph_safe for _, p in self._children())
         # parts that say so may pass rows between them whose normalisation is still to be applied
-        self._fuse = self.mixer.ends_in_norm and self.norm2.deferrable
+        self._fuse = self.ffn is not None and self.mixer.ends_in_norm and self.norm2.deferrable
 
     def _children(self):
-        return [(self.specs[k].name, getattr(self, k)) for k in ("norm1", "mixer", "norm2", "ffn")]
+        return [(self.specs[k].name, getattr(self, k)) for k in ("norm1", "mixer", "norm2", "ffn") if getattr(self, k) is not None]
 
     def tensors(self) -> Dict[str, TensorSpec]:
         out = {}
@@ -87,12 +90,17 @@ class PreNormBlock(Part):
         ScaledRows; then the feed-forward may end in it.  ``planes_ok``: whoever takes the new
         ``pending`` adds float32 planes of partial sums as well as plain rows.  Returns the new
         ``pending``."""
-        h = pending if isinstance(pending, ScaledRows) else self.norm1.forward(x, pending)
+        if isinstance(pending, ScaledRows):
+            h = pending
+        else:
+            h = self.norm1.forward(x, pending, out_dtype=torch.float32) if self.mixer.reads_float32 else self.norm1.forward(x, pending)
         n_rows = x.shape[0]
-        ffn_into = (x, next_norm) if next_norm is not None and self.ffn.ends_in_norm else None
-        ffn_kw = {"into": ffn_into} if ffn_into else {}
-        if planes_ok and self.ffn.ends_in_planes:
-            ffn_kw["planes_ok"] = True
+        last = self.ffn if self.ffn is not None else self.mixer
+        last_kw = {"into": (x, next_norm)} if next_norm is not None and last.ends_in_norm else {}
+        if planes_ok and last.ends_in_planes:
+            last_kw["planes_ok"] = True
+        if self.ffn is None:
+            return self.mixer.forward(h, step, cache, **last_kw)
         mixer_kw = {}
         if self.norm2.takes_planes and self.mixer.ends_in_planes:
             mixer_kw["planes_ok"] = True
@@ -101,11 +109,11 @@ class PreNormBlock(Part):
             # product; then the feed-forward applies the norm's factor in its first one
             a = self.mixer.forward(h, step, cache, into=(x, self.norm2), **mixer_kw)
             if isinstance(a, ScaledRows):
-                return self.ffn.forward(a, **ffn_kw)
+                return self.ffn.forward(a, **last_kw)
         else:
             a = self.mixer.forward(h, step, cache, **mixer_kw)
         h2 = self.norm2.forward(x, a)
-        return self.ffn.forward(h2, **ffn_kw)
+        return self.ffn.forward(h2, **last_kw)
 
 
 register_part("block", "prenorm", PreNormBlock)

@@ -1,4 +1,5 @@
-"""The dense gated feed-forward: ``down(act(gate) * up)``, ``act`` silu (``gate * sigmoid(gate)``) unless a layout says otherwise.
+"""The dense gated feed-forward: ``down(act(gate) * up)``, ``act`` silu (``gate * sigmoid(gate)``) unless a layout says otherwise
+(the tanh form of gelu, or a limited form of both).
 
 gate and up projections as one matrix product (gate rows first, the layout of the
 reference's fused tensor, llama.cu/src/model/mod.rs:140-147), the activation of
@@ -24,15 +25,23 @@ class SwiGLU(Part):
     # the tensors' names under the part's own; ``names`` replaces any
     NAMES = {"gate": "gate_proj.weight", "up": "up_proj.weight", "down": "down_proj.weight"}
 
-    def __init__(self, hidden_size: int, intermediate_size: int, names=None, activation: str = "silu"):
-        """``activation``: what the gate passes through, ``silu`` or ``gelu_tanh`` (the tanh form of gelu).  The products
-        with the activation in their epilogue are written for silu; another activation runs product, activation
-        kernel, product."""
+    def __init__(self, hidden_size: int, intermediate_size: int, names=None, activation: str = "silu",
+                 alpha: float = 1.0, limit: float = 0.0):
+        """``activation``: what the gate passes through, ``silu`` or ``gelu_tanh`` (the tanh form of gelu), or ``limited``: with
+        ``g = min(gate, limit)`` and ``u`` = ``up`` held within ``-limit .. limit`` the product's rows are ``g sigmoid(alpha g) (u +
+        1)``.  The products with the activation in their epilogue are written for silu and the limited form; gelu runs
+        product, activation kernel, product."""
         self.hidden_size, self.intermediate_size = int(hidden_size), int(intermediate_size)
         if activation not in ops.GATE_ACTIVATIONS:
             raise ValueError(f"feed-forward: no activation {activation!r}; known: {sorted(ops.GATE_ACTIVATIONS)}")
         self.activation = str(activation)
-        self.silu = self.activation == "silu"
+        self.fused_activation = self.activation != "gelu_tanh"       # the products have it in their epilogue
+        self.act = {}
+        if self.activation == "limited":
+            if not limit > 0:
+                raise ValueError(f"feed-forward: the limit {limit} must be positive")
+            self.act = {"act_alpha": float(alpha), "act_limit": float(limit)}
+        self.alpha, self.limit = float(alpha), float(limit)
         self.names = dict(self.NAMES, **(names or {}))
         self.w_gate_up = self.w_down = None
 
@@ -70,7 +79,7 @@ class SwiGLU(Part):
     def takes_scaled_rows(self, n_rows: int) -> bool:
         """Whether ``forward`` could be given ScaledRows of ``n_rows`` rows in the place of
         plain rows: the factor then goes into the first product's epilogue."""
-        if self.dtype != torch.bfloat16 or not self.silu:
+        if self.dtype != torch.bfloat16 or not self.fused_activation:
             return False
         if n_rows <= min(ops.ADD_NORM_MAX_ROWS, skinny_row_limit(self.w_gate_up)) and skinny_takes(n_rows, self.w_gate_up):
             return True
@@ -93,26 +102,26 @@ class SwiGLU(Part):
         return self._forward(h, into, planes_ok)
 
     def _forward(self, h, into=None, planes_ok=False, out_dtype=None):
-        if not self.silu:
+        if not self.fused_activation:
             if isinstance(h, ScaledRows):
-                raise ops.KernelError("feed-forward: rows that wait for their normalisation go with silu only")
+                raise ops.KernelError("feed-forward: rows that wait for their normalisation go with an activation in the product's epilogue only")
             act = ops.swiglu(linear(h, self.w_gate_up, out_dtype=self.dtype), activation=self.activation)
         elif isinstance(h, ScaledRows) and mid_swiglu_takes(h.rows.shape[0], self.w_gate_up) and ops.mid_supported(h.rows, self.w_gate_up.plain):
-            act = linear_swiglu_mid(h, self.w_gate_up)
+            act = linear_swiglu_mid(h, self.w_gate_up, **self.act)
         elif isinstance(h, ScaledRows):
             if not ops.skinny_supported(h.rows, self.w_gate_up.plain, self.dtype):
                 raise ops.KernelError("feed-forward: rows that wait for their normalisation need the kernel for few rows")
-            act = linear_swiglu(h.rows, self.w_gate_up, row_sumsq=h.sumsq, norm_width=h.width, eps=h.eps)
+            act = linear_swiglu(h.rows, self.w_gate_up, row_sumsq=h.sumsq, norm_width=h.width, eps=h.eps, **self.act)
         elif self.dtype == torch.bfloat16 and mid_swiglu_takes(h.shape[0], self.w_gate_up) and ops.mid_supported(h, self.w_gate_up.plain):
             # 15 to 192 rows (mid_swiglu_max_rows): the rows shared through LDS, the activation in the product's epilogue
-            act = linear_swiglu_mid(h, self.w_gate_up)
+            act = linear_swiglu_mid(h, self.w_gate_up, **self.act)
         elif (self.dtype == torch.bfloat16 and h.shape[0] <= skinny_row_limit(self.w_gate_up)
               and ops.skinny_supported(h, self.w_gate_up.plain, self.dtype)):
             # few rows: one pass over the weights, the activation in the product's epilogue
-            act = linear_swiglu(h, self.w_gate_up)
+            act = linear_swiglu(h, self.w_gate_up, **self.act)
         else:
             gu = linear(h, self.w_gate_up, out_dtype=self.dtype)
-            act = ops.swiglu(gu)
+            act = ops.swiglu(gu, activation=self.activation, alpha=self.alpha, limit=self.limit)
         if act.shape[1] != self.intermediate_size:
             act = act[:, :self.intermediate_size]      # without what the rows of zeros gave
         if out_dtype is not None:
@@ -124,7 +133,7 @@ class SwiGLU(Part):
         if into is not None and act.dtype == torch.bfloat16 and skinny_takes(act.shape[0], self.w_down, preferred=True):
             # only where the kernel for few rows is the faster one for this product anyway
             residual, norm = into
-            fused = linear_into_norm(act, self.w_down, residual, norm.weight)
+            fused = linear_into_norm(act, self.w_down, residual, norm.weight, scale=norm.delta_scale)
             if fused is not None:
                 return ScaledRows(fused[0], fused[1], norm.size, norm.eps)
         return linear(act, self.w_down, out_dtype=self.dtype)

@@ -83,11 +83,12 @@ def linear(x: torch.Tensor, weight: Union[torch.Tensor, Weight], out_dtype: Opti
     return ops.gemm_nt(x, weight, out=out, out_dtype=out_dtype, accumulate=accumulate)
 
 
-def linear_swiglu(h, weight: Union[torch.Tensor, Weight], row_sumsq=None, norm_width: int = 0, eps: float = 0.0):
+def linear_swiglu(h, weight: Union[torch.Tensor, Weight], row_sumsq=None, norm_width: int = 0, eps: float = 0.0, **act):
     """``silu(h @ gate.T) * (h @ up.T)`` with the weight-streaming kernel (``weight`` holds the gate
-    rows, then the up rows); ``row_sumsq``: the rows wait for their normalisation."""
+    rows, then the up rows); ``row_sumsq``: the rows wait for their normalisation; ``act``: ``act_alpha`` and ``act_limit`` of
+    the limited activation."""
     weight, packed = _split(weight)
-    kw = dict(row_sumsq=row_sumsq, norm_width=norm_width, eps=eps) if row_sumsq is not None else {}
+    kw = dict(act, row_sumsq=row_sumsq, norm_width=norm_width, eps=eps) if row_sumsq is not None else act
     if packed is not None:
         return ops.gemm_skinny(h, packed, swiglu=True, packed=True, **kw)
     return ops.gemm_skinny(h, weight, swiglu=True, **kw)
@@ -203,11 +204,11 @@ def mid_swiglu_takes(n_rows: int, weight: Union[torch.Tensor, Weight]) -> bool:
             and w.shape[1] % 128 == 0 and w.shape[0] >= ops.TUNING.mid_swiglu_features)
 
 
-def linear_swiglu_mid(h, weight: Union[torch.Tensor, Weight]) -> torch.Tensor:
+def linear_swiglu_mid(h, weight: Union[torch.Tensor, Weight], **act) -> torch.Tensor:
     """``h``: bfloat16 rows or ScaledRows (the factor then goes into the epilogue)."""
     if isinstance(h, ScaledRows):
-        return ops.gemm_mid(h.rows, _split(weight)[1], swiglu=True, packed=True, row_sumsq=h.sumsq, norm_width=h.width, eps=h.eps)
-    return ops.gemm_mid(h, _split(weight)[1], swiglu=True, packed=True)
+        return ops.gemm_mid(h.rows, _split(weight)[1], swiglu=True, packed=True, row_sumsq=h.sumsq, norm_width=h.width, eps=h.eps, **act)
+    return ops.gemm_mid(h, _split(weight)[1], swiglu=True, packed=True, **act)
 
 
 def skinny_row_limit(weight: Union[torch.Tensor, Weight]) -> int:
@@ -235,8 +236,9 @@ def mid_add_norm_takes(n_rows: int, weight: Union[torch.Tensor, Weight]) -> bool
             and w.shape[0] // 16 <= t.compute_units)
 
 
-def linear_into_norm(a: torch.Tensor, weight: Union[torch.Tensor, Weight], residual: torch.Tensor, norm_weight: torch.Tensor):
-    """``residual += a @ weight.T`` and the rows for the product after the next norm, in one
+def linear_into_norm(a: torch.Tensor, weight: Union[torch.Tensor, Weight], residual: torch.Tensor, norm_weight: torch.Tensor,
+                     scale: float = 1.0):
+    """``residual += scale * (a @ weight.T)`` and the rows for the product after the next norm, in one
     kernel: returns ``(rows, sumsq)`` for a ``ScaledRows``, or None if the kernel for it does
     not take these operands (then nothing has been done)."""
     whole = weight
@@ -246,12 +248,12 @@ def linear_into_norm(a: torch.Tensor, weight: Union[torch.Tensor, Weight], resid
         return None
     if mid_add_norm_takes(a.shape[0], whole) and ops.mid_supported(a, weight) and residual.stride(0) % 4 == 0 \
             and residual.data_ptr() % 16 == 0:
-        return ops.gemm_mid_add_norm(a, packed, residual, norm_weight, packed=True)
+        return ops.gemm_mid_add_norm(a, packed, residual, norm_weight, packed=True, scale=scale)
     if not (a.shape[0] <= ops.ADD_NORM_MAX_ROWS and ops.skinny_supported(a, weight, torch.float32)):
         return None
     if packed is not None:
-        return ops.gemm_skinny_add_norm(a, packed, residual, norm_weight, packed=True)
-    return ops.gemm_skinny_add_norm(a, weight, residual, norm_weight)
+        return ops.gemm_skinny_add_norm(a, packed, residual, norm_weight, packed=True, scale=scale)
+    return ops.gemm_skinny_add_norm(a, weight, residual, norm_weight, scale=scale)
 
 
 def mid_qkv_takes(n_rows: int, weight: Union[torch.Tensor, Weight]) -> bool:
@@ -292,3 +294,62 @@ def linear_qkv_rope(h, weight: Union[torch.Tensor, Weight], positions, slots, co
                                         page_size, packed=True, **kw)
     return ops.gemm_skinny_qkv_rope(rows, weight, positions, slots, cos, sin, cache_pages, heads, kv_heads, head_dim,
                                     page_size, **kw)
+
+
+def project(h, weight: Union[torch.Tensor, Weight], dtype: torch.dtype) -> torch.Tensor:
+    """A branch's first product: ``h`` plain rows, or ScaledRows whose factor goes into the product's epilogue."""
+    if isinstance(h, ScaledRows):
+        return linear_scaled(h, weight, out_dtype=dtype)
+    return linear(h, weight, out_dtype=dtype)
+
+
+def finish(a: torch.Tensor, weight: Union[torch.Tensor, Weight], dtype: torch.dtype, into=None, planes_ok: bool = False,
+           out_dtype: Optional[torch.dtype] = None):
+    """A branch's last product, ended as whoever called the branch allows: ``into = (residual, norm)``: the residual sum and that
+    norm's weight in its epilogue where a kernel for few rows takes it (ScaledRows); ``planes_ok``: float32 planes of
+    partial sums where K is cut; else plain rows of ``out_dtype`` (``dtype``)."""
+    if out_dtype is not None and out_dtype != dtype:
+        return linear(a, weight, out_dtype=out_dtype)
+    if into is not None:
+        residual, norm = into
+        fused = linear_into_norm(a, weight, residual, norm.weight, scale=norm.delta_scale)
+        if fused is not None:
+            return ScaledRows(fused[0], fused[1], norm.size, norm.eps)
+    if planes_ok and dtype == torch.bfloat16 and mid_takes(a.shape[0], weight):
+        return linear_planes(a, weight)
+    return linear(a, weight, out_dtype=dtype)
+
+
+class GroupWeight:
+    """Several matrices ``[groups, rows, k]`` (``[out, in]`` each), every one of which multiplies rows of its own: a matrix per
+    head, or projections of differently mixed rows.  Kept as the weight-streaming kernel takes them (one above the other,
+    packed where that is possible) and, for the library's batched product of many bfloat16 rows, once more with ``k`` in front:
+    that product's right operand must be contiguous."""
+
+    def __init__(self, tensor: torch.Tensor, build=None):
+        self.groups, self.rows, self.k = tensor.shape
+        self.each = tensor.contiguous()
+        self.stacked = Weight(self.each.view(self.groups * self.rows, self.k), build)
+        self.kn = tensor.transpose(1, 2).contiguous() if tensor.dtype == torch.bfloat16 else None
+
+
+def linear_groups(x: torch.Tensor, weight: GroupWeight, out: torch.Tensor, gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``out[:, g * rows: (g + 1) * rows] = x[g] @ weight.each[g].T`` for ``x [groups, m, k]`` (a view of wider rows will do) and
+    ``out [m, groups * rows]``; with ``gate [m, groups * rows]`` the result is multiplied by ``sigmoid(gate)`` (and is then a tensor
+    of its own where no kernel has the gate in its epilogue).  Few bfloat16 rows: one weight-streaming launch for all
+    groups; many: the library's batched product; float32: the engine's own product, group by group."""
+    g, m, _ = x.shape
+    if x.dtype == torch.bfloat16 and weight.each.dtype == torch.bfloat16:
+        packed = weight.stacked.packed
+        if m <= ops.skinny_max_rows(packed is not None) and ops.skinny_grouped_supported(x, weight.stacked.plain, g):
+            return ops.gemm_skinny_grouped(x, weight.stacked.plain if packed is None else packed, out, packed=packed is not None, gate=gate)
+        if out.dtype == torch.bfloat16:
+            torch.bmm(x, weight.kn, out=out.view(m, g, weight.rows).permute(1, 0, 2))
+            return out if gate is None else ops.element_gate(out, gate, g, weight.rows)
+    for i in range(g):
+        part = out[:, i * weight.rows:(i + 1) * weight.rows]
+        if ops.skinny_f32_supported(x[i], weight.each[i], out.dtype):
+            ops.gemm_skinny_f32(x[i], weight.each[i], out=part)
+        else:
+            ops.gemm_nt(x[i], weight.each[i], out=part)
+    return out if gate is None else ops.element_gate(out, gate, g, weight.rows)

@@ -88,11 +88,14 @@ class DecoderModel:
         self.layers: List[Part] = [make_part("block", s) for s in spec.layers]
         self.final_norm = make_part("norm", spec.final_norm)
         self.head = make_part("head", spec.head)
-        self.graph_safe = all(p.graph_safe for p in [self.embedding, self.final_norm, self.head] + self.layers)
+        self.streams: List[Part] = [make_part("stream", s) for s in spec.streams]
+        self.graph_safe = all(p.graph_safe for p in [self.embedding, self.final_norm, self.head] + self.layers + self.streams)
         n = len(self.layers)
         for i, e in enumerate(spec.run_order):
             if not 0 <= e.layer < n:
                 raise ValueError(f"run order entry {i} names layer {e.layer}, but there are {n} layers")
+            if e.before is not None and not 0 <= e.before < len(self.streams):
+                raise ValueError(f"run order entry {i} names stream part {e.before}, but there are {len(self.streams)}")
             if e.cache_of is not None:
                 if not 0 <= e.cache_of < i:
                     raise ValueError(f"run order entry {i} reads the cache of entry {e.cache_of}, which does not run before it")
@@ -103,6 +106,8 @@ class DecoderModel:
     def _named_parts(self):
         yield self.spec.embedding.name, self.embedding
         for s, p in zip(self.spec.layers, self.layers):
+            yield s.name, p
+        for s, p in zip(self.spec.streams, self.streams):
             yield s.name, p
         yield self.spec.final_norm.name, self.final_norm
         yield self.spec.head.name, self.head
@@ -157,13 +162,17 @@ class DecoderModel:
             x = self.embedding.forward(step.tokens)
             pending = None
             order = self.spec.run_order
+            starts = [s.begin(x) for s in self.streams]      # what they keep of the embedding's output
             for i, e in enumerate(order):
+                if e.before is not None:
+                    x, pending = self.streams[e.before].forward(x, pending, starts[e.before]), None
                 # a block may end in the norm that follows it, if what comes then takes such rows: the
                 # next block with its first norm, or, when every token's logits are wanted, the output
                 # matrix with the final norm
+                nothing_between = i + 1 < len(order) and order[i + 1].before is None
                 if i + 1 < len(order):
-                    follower = self.layers[order[i + 1].layer]
-                    norm = follower.first_norm
+                    follower = self.layers[order[i + 1].layer] if nothing_between else None
+                    norm = follower.first_norm if nothing_between else None
                 else:
                     follower = self.head if step.logits_all and self.final_norm.deferrable else None
                     norm = self.final_norm
@@ -171,7 +180,7 @@ class DecoderModel:
                 kw = {}
                 if follower is not None and norm is not None and layer.ends_in_next_norm and follower.takes_scaled_rows(x.shape[0]):
                     kw["next_norm"] = norm
-                elif i + 1 < len(order) and norm is not None and layer.hands_over_normed and follower.takes_normed_rows \
+                elif nothing_between and norm is not None and layer.hands_over_normed and follower.takes_normed_rows \
                         and norm.deferrable:
                     # the block adds its last output to the stream and runs the next block's first norm in one kernel
                     kw["next_norm"] = norm
@@ -179,8 +188,10 @@ class DecoderModel:
                 # if that norm takes them: the next block's first, or the final norm when no rows are
                 # gathered before it
                 if layer.ends_in_planes:
-                    takes = self.layers[order[i + 1].layer].takes_planes if i + 1 < len(order) \
-                        else (step.logits_all and self.final_norm.takes_planes)
+                    if i + 1 < len(order):
+                        takes = follower.takes_planes if nothing_between else self.streams[order[i + 1].before].takes_planes
+                    else:
+                        takes = step.logits_all and self.final_norm.takes_planes
                     if takes:
                         kw["planes_ok"] = True
                 pending = layer.forward(x, pending, step, caches[i], **kw)

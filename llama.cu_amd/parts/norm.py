@@ -17,9 +17,14 @@ from .base import BuildContext, Part, TensorSpec, register_part
 class RMSNorm(Part):
     graph_safe = True
 
-    def __init__(self, size: int, eps: float, tensor: str = "weight", one_plus: bool = False):
+    def __init__(self, size: int, eps: float, tensor: str = "weight", one_plus: bool = False, delta_scale: float = 1.0,
+                 factor: float = 1.0):
         """``tensor``: the weight's name under the part's.  ``one_plus``: the file holds the weight around zero and the
-        factor is ``1 + w``; the sum is made once, at load, in 32-bit, and ``weight`` is the factor."""
+        factor is ``1 + w``; the sum is made once, at load, in 32-bit, and ``weight`` is the factor.  ``delta_scale``: what a
+        branch's output is multiplied by before it is added to the stream in front of this norm (by the norm's kernel, or by
+        the product that ends in it).  ``factor``: the norm's output is multiplied by it (it goes into the 32-bit weight at load:
+        a factor on the logits, say, costs nothing in the norm before them)."""
+        self.delta_scale, self.factor = float(delta_scale), float(factor)
         self.size = int(size)
         self.eps = float(eps)
         self.tensor, self.one_plus = str(tensor), bool(one_plus)
@@ -32,16 +37,18 @@ class RMSNorm(Part):
     def load(self, tensors, build: BuildContext) -> None:
         w = tensors[self.tensor]
         self.weight = (1.0 + w.float()).contiguous() if self.one_plus else w.contiguous()
+        if self.factor != 1.0:
+            self.weight = (self.weight.float() * self.factor).contiguous()
         # the factor in 32-bit, for kernels that take it so (a norm behind a sublayer, ``ops.norm_post``)
         self.weight32 = self.weight if self.weight.dtype == torch.float32 else self.weight.float().contiguous()
         self.dtype = build.dtype
 
-    def forward(self, x: torch.Tensor, delta: Optional[torch.Tensor] = None) -> torch.Tensor:
+    def forward(self, x: torch.Tensor, delta: Optional[torch.Tensor] = None, out_dtype=None) -> torch.Tensor:
         """``x`` (float32 residual stream) takes in ``delta`` if there is one (rows in the compute
         type, or float32 planes ``[planes, n, d]`` of partial sums); returns the normalised rows
-        in the compute type."""
-        out = torch.empty(x.shape, dtype=self.dtype, device=x.device)
-        return ops.rmsnorm(x, self.weight, self.eps, out, delta=delta, write_back=True)
+        in the compute type (or ``out_dtype``)."""
+        out = torch.empty(x.shape, dtype=out_dtype or self.dtype, device=x.device)
+        return ops.rmsnorm(x, self.weight, self.eps, out, delta=delta, write_back=True, delta_scale=self.delta_scale)
 
 
     # This norm is a factor per row times a weight per column, so its factor may be applied
