@@ -445,9 +445,29 @@ def mufotar_config(z, positions):
                                     "logit_softcap": 30.0, "max_positions": positions})
 
 
+def gefudra_config(z, positions):
+    """As many layer runs as the Llama model beside it has layers, each with its dense feed-forward: latent attention (a latent of
+    128, one head of the matrix-core attention kernels' largest size; queries through a latent of 3/8 of the width; a window
+    of 1,024), then the recurrent mixer (heads of 64), latent attention and differential attention (two maps of half a
+    Llama head over values of a whole one) as a loop that runs twice where there are eight runs, then latent attention."""
+    from llama_cu_amd.config import GefudraConfig
+    inter = (z["top"] * 2 * z["ff"] // 3 + 127) // 128 * 128
+    d, h, g, w = z["dim"], z["heads"], z["kv_heads"], z["width"]
+    latent = {"type": "latent_attention", "mixer": {"heads": h, "dim": d, "vdim": d, "kv_rank": 128, "q_rank": 3 * w // 8, "scale": d ** -0.5,
+                                                    "mask": {"size": 1024}}}
+    mixer = {"type": "wkv", "mixer": {"heads": w // 64, "dim": 64, "rank": 64}}
+    differential = {"type": "attention", "mixer": {"heads": h, "kv_heads": g, "dim": d // 2, "vdim": d, "scale": (d // 2) ** -0.5, "diff": 0.5,
+                                                   "softcap": 30.0, "rot": {"dims": d // 2, "base": 50000.0}}}
+    times, left = divmod(z["layers"] - 1, 3)
+    layers = [latent, mixer, latent, differential] + [latent] * left
+    return GefudraConfig.from_dict({"architecture": "Gefudra", "vocab": z["vocab"], "width": w, "norm": {"eps": 1e-6}, "residual_mult": 0.5,
+                                    "logit_scale": 0.5, "layers": [dict(l, mlp={"kind": "dense", "ff": inter, "limit": 7.0}) for l in layers],
+                                    "loop": {"start": 1, "stop": 4, "times": times}, "max_positions": positions})
+
+
 DESIGN_CONFIGS = {"divasun": lambda z, p: divasun_config(z, p), "llama": lambda z, p: llama_like(z, p),
                   "lozezen": lambda z, p: lozezen_config(z, p), "ralepel": lambda z, p: ralepel_config(z, p),
-                  "mufotar": lambda z, p: mufotar_config(z, p)}
+                  "mufotar": lambda z, p: mufotar_config(z, p), "gefudra": lambda z, p: gefudra_config(z, p)}
 
 
 def llama_like(z, positions):
@@ -574,10 +594,10 @@ def main() -> int:
                          "decode while a prompt of 16 tokens arrives every second step (host time and the GPU's busy "
                          "fraction per kind of step)")
     ap.add_argument("--designs", default="divasun,llama", metavar="NAMES",
-                    help="with --workload designs: which designs are measured side by side, of divasun, lozezen, ralepel, mufotar and llama "
+                    help="with --workload designs: which designs are measured side by side, of divasun, lozezen, ralepel, mufotar, gefudra and llama "
                          "(default: divasun,llama)")
     ap.add_argument("--designs-one", metavar="DESIGN:SIZE:WHAT", default=None,
-                    help="with --workload designs, for a profiler: only DESIGN (divasun, lozezen, ralepel, mufotar or llama) at SIZE (w2048, w4096), and "
+                    help="with --workload designs, for a profiler: only DESIGN (divasun, lozezen, ralepel, mufotar, gefudra or llama) at SIZE (w2048, w4096), and "
                          "only WHAT: 'prefill' (three steps of 2,048 tokens) or a number of requests that decode ten steps over "
                          "prompts of 512 tokens; steps are launched one kernel at a time, not replayed from graphs")
     ap.add_argument("--no-points", action="store_true", help="skip decoding at batch 1 and 64, the prefill and the check")

@@ -245,20 +245,34 @@ LCU_API int lcu_rmsnorm_planes(float *x, const float *planes_ptr, int planes, co
 // ---------------------------------------------------------------- the residual stream as a product's operand
 // x (f32) += delta_scale * delta (planes as above; null: nothing), written back; out[r, c] = x[r, c] in the compute type, rows ldo
 // apart: the stream (or, with no delta, a copy of it) as columns of a wider operand.
-template <class TD, class TO>
-__global__ void stream_rows_kernel(float *__restrict__ x, const TD *__restrict__ delta, int planes, size_t plane_stride, float delta_scale,
-                                   TO *__restrict__ out, int ldo, int d) {
-    float *xr = x + (size_t)blockIdx.x * d;
-    TO *o = out + (size_t)blockIdx.x * ldo;
-    for (int c = threadIdx.x; c < d; c += blockDim.x) {
-        float v = xr[c];
-        if (delta) {
-            const TD *dr = delta + (size_t)blockIdx.x * d + c;
-            for (int p = 0; p < planes; ++p) v = fmaf(delta_scale, to_f32(dr[p * plane_stride]), v);
-            xr[c] = v;
+// V neighbouring columns a thread, all loads of a thread's planes (four at a time) before it waits for one.
+template <class T, int V> struct alignas(V * sizeof(T)) VecN { T v[V]; };
+
+template <class TD, class TO, int V>
+__global__ void __launch_bounds__(256)
+stream_rows_kernel(float *__restrict__ x, const TD *__restrict__ delta, int planes, size_t plane_stride, float delta_scale,
+                   TO *__restrict__ out, int ldo, int d) {
+    const int c = (blockIdx.y * 256 + threadIdx.x) * V;
+    if (c >= d) return;
+    const size_t at = (size_t)blockIdx.x * d + c;
+    VecN<float, V> v = *(const VecN<float, V> *)(x + at);
+    if (delta) {
+        for (int p0 = 0; p0 < planes; p0 += 4) {
+            VecN<TD, V> q[4];
+#pragma unroll
+            for (int p = 0; p < 4; ++p) q[p] = *(const VecN<TD, V> *)(delta + (p0 + p < planes ? p0 + p : p0) * plane_stride + at);
+#pragma unroll
+            for (int p = 0; p < 4; ++p)
+                if (p0 + p < planes)
+#pragma unroll
+                    for (int e = 0; e < V; ++e) v.v[e] = fmaf(delta_scale, to_f32(q[p].v[e]), v.v[e]);
         }
-        o[c] = from_f32<TO>(v);
+        *(VecN<float, V> *)(x + at) = v;
     }
+    VecN<TO, V> o;
+#pragma unroll
+    for (int e = 0; e < V; ++e) o.v[e] = from_f32<TO>(v.v[e]);
+    *(VecN<TO, V> *)(out + (size_t)blockIdx.x * ldo + c) = o;
 }
 
 LCU_API int lcu_stream_rows(float *x, const void *delta, int delta_type, int planes, float delta_scale, void *out, int out_type, int ldo,
@@ -266,8 +280,13 @@ LCU_API int lcu_stream_rows(float *x, const void *delta, int delta_type, int pla
     if (n <= 0) return LCU_OK;
     if (d <= 0 || ldo < d || planes < 1 || !x || !out) return LCU_BAD_ARGUMENT;
     const size_t stride = (size_t)n * d;
-    dim3 grid(n), block(256);
-#define GO(TD, TO) stream_rows_kernel<TD, TO><<<grid, block, 0, stream>>>(x, (const TD *)delta, planes, stride, delta_scale, (TO *)out, ldo, d)
+    const int v = d % 4 == 0 && ldo % 4 == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)delta % 16 == 0 && (uintptr_t)out % 16 == 0 ? 4 : 1;
+    dim3 grid(n, (d + 256 * v - 1) / (256 * v)), block(256);
+#define GO(TD, TO)                                                                                                                              \
+    do {                                                                                                                                        \
+        if (v == 4) stream_rows_kernel<TD, TO, 4><<<grid, block, 0, stream>>>(x, (const TD *)delta, planes, stride, delta_scale, (TO *)out, ldo, d); \
+        else stream_rows_kernel<TD, TO, 1><<<grid, block, 0, stream>>>(x, (const TD *)delta, planes, stride, delta_scale, (TO *)out, ldo, d);   \
+    } while (0)
     if (delta_type == LCU_F32 && out_type == LCU_F32) GO(float, float);
     else if (delta_type == LCU_F32 && out_type == LCU_BF16) GO(float, bf16_t);
     else if (delta_type == LCU_BF16 && out_type == LCU_BF16) GO(bf16_t, bf16_t);

@@ -24,3 +24,12 @@ __device__ __forceinline__ float sum_over_16(float v) {
     v += lane_mirror16(v);
     return v;
 }
+
+// The sum over a wave, in all lanes: within sixteen as above, then across the rows of sixteen by exchanging them in the vector unit.
+__device__ __forceinline__ float wave_sum_in_place(float v) {
+    const unsigned u = __float_as_uint(sum_over_16(v));
+    const auto a = __builtin_amdgcn_permlane16_swap(u, u, false, false);     // (rows 0 0 2 2, rows 1 1 3 3)
+    const unsigned w = __float_as_uint(__uint_as_float(a[0]) + __uint_as_float(a[1]));
+    const auto b = __builtin_amdgcn_permlane32_swap(w, w, false, false);     // (lower half twice, upper half twice)
+    return __uint_as_float(b[0]) + __uint_as_float(b[1]);
+}

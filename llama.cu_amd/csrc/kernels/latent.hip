@@ -21,6 +21,7 @@
 // All arithmetic is 32-bit, one rounding at each store.
 #include "common.h"
 #include "kv_layout.h"
+#include "lane_moves.h"
 
 constexpr int LP_MAX_DIM = 640;
 
@@ -36,20 +37,32 @@ latent_prepare_kernel(const TI *__restrict__ rows, int row_stride, int q_head_st
     const int head = blockIdx.y;
     const TI *row = rows + (size_t)t * row_stride;
     if (head == turned_heads + store_kv) {
+        constexpr int ITEMS = 16;                             // the row stays in registers, its loads in flight together, up to 1024 columns
         const TI *x = row + cq_off;
-        float sq = 0.f;
-        for (int c = lane; c < q_rank; c += WAVE) {
-            const float v = to_f32(x[c]);
-            sq += v * v;
+        T *o = cq_out + (size_t)t * q_rank;
+        float v[ITEMS], w[ITEMS], sq = 0.f;
+#pragma unroll
+        for (int i = 0; i < ITEMS; ++i) {
+            const int c = min(lane + WAVE * i, q_rank - 1);   // (no branch around a load)
+            v[i] = to_f32(x[c]);
+            w[i] = cq_norm[c];
         }
-        const float f = rsqrtf(wave_sum(sq) / (float)q_rank + eps);
-        for (int c = lane; c < q_rank; c += WAVE) cq_out[(size_t)t * q_rank + c] = from_f32<T>(to_f32(x[c]) * f * cq_norm[c]);
+#pragma unroll
+        for (int i = 0; i < ITEMS; ++i) sq += lane + WAVE * i < q_rank ? v[i] * v[i] : 0.f;
+        for (int c = lane + WAVE * ITEMS; c < q_rank; c += WAVE) {
+            const float y = to_f32(x[c]);
+            sq += y * y;
+        }
+        const float f = rsqrtf(wave_sum_in_place(sq) / (float)q_rank + eps);
+#pragma unroll
+        for (int i = 0; i < ITEMS; ++i)
+            if (lane + WAVE * i < q_rank) o[lane + WAVE * i] = from_f32<T>(v[i] * f * w[i]);
+        for (int c = lane + WAVE * ITEMS; c < q_rank; c += WAVE) o[c] = from_f32<T>(to_f32(x[c]) * f * cq_norm[c]);
         return;
     }
     const int pos = rot > 0 ? positions[t] : 0, half = rot / 2;
     const bool in_table = pos >= 0 && pos < max_pos;
     const float nan = __uint_as_float(0x7fc00000u);          // a position outside the table gives NaN, not a wrong value
-    __shared__ float xs[LP_MAX_DIM];
     if (head < turned_heads) {
         const TI *qr = row + (size_t)head * q_head_stride + q_rot_off;
         T *o = q_out + ((size_t)t * nh + head) * dhp;
@@ -67,17 +80,27 @@ latent_prepare_kernel(const TI *__restrict__ rows, int row_stride, int q_head_st
     T *pg = cache + (size_t)(slot / page) * kv_page_elems(1, dhp, dvp, page);
     const int tok = slot % page;
     const TI *kv = row + kv_off;
-    float sq = 0.f;
-    for (int c = lane; c < rank; c += WAVE) {
-        const float v = to_f32(kv[c]);
-        xs[c] = v;
-        sq += v * v;
-    }
-    const float f = rsqrtf(wave_sum(sq) / (float)rank + eps);
-    for (int c = lane; c < rank; c += WAVE) {
-        const T v = from_f32<T>(xs[c] * f * c_norm[c]);
-        pg[kv_key_offset(0, tok, c, dhp, page)] = v;
-        pg[kv_value_offset(1, 0, tok, c, dhp, dvp, page)] = v;
+    constexpr int ITEMS = LP_MAX_DIM / WAVE;
+    float x[ITEMS], w[ITEMS], sq = 0.f;
+#pragma unroll
+    for (int i = 0; i < ITEMS; ++i)
+        if (WAVE * i < rank) {                               // (the same in all lanes)
+            const int c = min(lane + WAVE * i, rank - 1);
+            x[i] = to_f32(kv[c]);
+            w[i] = c_norm[c];
+        }
+#pragma unroll
+    for (int i = 0; i < ITEMS; ++i)
+        if (WAVE * i < rank) sq += lane + WAVE * i < rank ? x[i] * x[i] : 0.f;
+    const float f = rsqrtf(wave_sum_in_place(sq) / (float)rank + eps);
+#pragma unroll
+    for (int i = 0; i < ITEMS; ++i) {
+        const int c = lane + WAVE * i;
+        if (c < rank) {
+            const T v = from_f32<T>(x[i] * f * w[i]);
+            pg[kv_key_offset(0, tok, c, dhp, page)] = v;
+            pg[kv_value_offset(1, 0, tok, c, dhp, dvp, page)] = v;
+        }
     }
     for (int i = lane; i < half; i += WAVE) {
         float ra = nan, rb = nan;

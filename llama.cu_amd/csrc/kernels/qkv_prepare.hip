@@ -17,14 +17,27 @@
 //
 // The head sizes of the rows (dh, dv) may be any; what is stored has dhp >= dh and dvp >= dv dims per head, the
 // dims beyond the true ones zeros (dhp a multiple of 8, as the pages' layout wants; zeros change no score and no
-// output).  All arithmetic is 32-bit, one rounding at each store.  One wave per (token, head).
+// output).  All arithmetic is 32-bit, one rounding at each store.  One wave per (token, head), four to a workgroup.
 #include "common.h"
 #include "kv_layout.h"
 
 constexpr int QP_MAX_DIM = 640;
 
+constexpr int QP_WAVES = 4;
+
+// Between a wave's writes to LDS that is its own and its lanes' reads of one another's: a wave's LDS accesses are carried out
+// in order, so only the compiler has to keep them so.
+__device__ __forceinline__ void own_lds_fence() {
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+}
+
+// two neighbouring elements in one store (p + c on a boundary of two elements)
+__device__ __forceinline__ void store_two(float *p, float a, float b) { *(float2 *)p = make_float2(a, b); }
+__device__ __forceinline__ void store_two(bf16_t *p, float a, float b) { *(uint32_t *)p = pack2_bf16(a, b); }
+
 template <class TI, class T>
-__global__ void __launch_bounds__(WAVE)
+__global__ void __launch_bounds__(QP_WAVES *WAVE)
 qkv_prepare_kernel(const TI *__restrict__ rows, int row_stride, int q_off, int k_off, int v_off,
                    const float *__restrict__ bias, const float *__restrict__ q_norm, const float *__restrict__ k_norm,
                    float eps, const int *__restrict__ positions, const float *__restrict__ cos_t,
@@ -32,10 +45,12 @@ qkv_prepare_kernel(const TI *__restrict__ rows, int row_stride, int q_off, int k
                    const int *__restrict__ slots, T *__restrict__ cache, int nh, int nkvh, int dh, int dhp, int dv,
                    int dvp, int page, int store_kv, int maps, int joint) {
     // nh and nkvh count (head, map) pairs; stored_kvh: key/value heads in the cache
-    const int t = blockIdx.x, head = blockIdx.y, lane = threadIdx.x;
+    const int wave = threadIdx.x / WAVE, t = blockIdx.x, head = blockIdx.y * QP_WAVES + wave, lane = threadIdx.x & (WAVE - 1);
     const int stored_kvh = joint ? nkvh / maps : nkvh;
+    if (head >= (store_kv ? nh + nkvh + stored_kvh : nh)) return;         // (no barrier below: a wave's LDS is its own)
     const TI *row = rows + (size_t)t * row_stride;
-    __shared__ float xs[QP_MAX_DIM];
+    extern __shared__ float xs_all[];                                     // a wave's dh numbers, rounded up to whole words of its own
+    float *xs = xs_all + wave * ((dh + 3) / 4 * 4);
     int slot = -1;
     T *pg = nullptr;
     int tok = 0;
@@ -67,7 +82,7 @@ qkv_prepare_kernel(const TI *__restrict__ rows, int row_stride, int q_off, int k
         const float f = rsqrtf(wave_sum(sq) / (float)dh + eps);
         for (int c = lane; c < dh; c += WAVE) xs[c] = xs[c] * f * nw[c];
     }
-    __syncthreads();
+    own_lds_fence();
     if (cos_t) {
         const int pos = positions[t], half = rot_dim / 2;
         const bool in_table = pos >= 0 && pos < max_pos;
@@ -78,7 +93,7 @@ qkv_prepare_kernel(const TI *__restrict__ rows, int row_stride, int q_off, int k
             xs[ia] = ra;
             xs[ib] = rb;
         }
-        __syncthreads();
+        own_lds_fence();
     }
     // where the vector's first dim goes among the stored head's dims; a joint head's other dims are zeros in a query and the
     // other maps' in a key, whose last map also writes the zeros behind them
@@ -90,12 +105,104 @@ qkv_prepare_kernel(const TI *__restrict__ rows, int row_stride, int q_off, int k
             place = (qh / group * maps + map) * group + qh % group;
         }
         T *o = q_out + (size_t)t * nh * dhp + (size_t)place * dhp;
-        for (int c = lane; c < dhp; c += WAVE) o[c] = from_f32<T>(c >= at && c < at + dh ? xs[c - at] : 0.f);
+        auto dim = [&](int c) { return c >= at && c < at + dh ? xs[c - at] : 0.f; };
+        for (int c = 2 * lane; c < dhp; c += 2 * WAVE) store_two(o + c, dim(c), dim(c + 1));
     } else {
         const int kvh = joint ? (head - nh) / maps : head - nh;
         const int end = !joint || map == maps - 1 ? dhp : at + dh;
-        for (int c = at + lane; c < end; c += WAVE) pg[kv_key_offset(kvh, tok, c, dhp, page)] = from_f32<T>(c < at + dh ? xs[c - at] : 0.f);
+        auto dim = [&](int c) { return c < at + dh ? xs[c - at] : 0.f; };
+        if (at % 2 == 0 && end % 2 == 0) {
+            for (int c = at + 2 * lane; c < end; c += 2 * WAVE) store_two(pg + kv_key_offset(kvh, tok, c, dhp, page), dim(c), dim(c + 1));
+        } else {
+            for (int c = at + lane; c < end; c += WAVE) pg[kv_key_offset(kvh, tok, c, dhp, page)] = from_f32<T>(dim(c));
+        }
     }
+}
+
+// The common case in one pass with wide accesses: no bias, no norm, pairs (i, i + rot_dim/2) or no rotation, every size and column
+// a multiple of 8 (rot_dim of 16).  A thread takes eight neighbouring dims of what is stored for one head of one token (and, of a
+// turned part, the eight that they are paired with), or eight dims of a value.  The same roundings as above.
+template <class T> struct alignas(8 * sizeof(T)) QpRow8 { T v[8]; };
+
+template <class TI, class T>
+__global__ void __launch_bounds__(256)
+qkv_prepare_wide_kernel(const TI *__restrict__ rows, int row_stride, int q_off, int k_off, int v_off, const int *__restrict__ positions,
+                        const float *__restrict__ cos_t, const float *__restrict__ sin_t, int max_pos, int rot_dim, T *__restrict__ q_out,
+                        const int *__restrict__ slots, T *__restrict__ cache, int nh, int nkvh, int dh, int dhp, int dv, int dvp, int page,
+                        int store_kv, int maps, int joint) {
+    const int t = blockIdx.x, half8 = rot_dim / 16, stored_kvh = joint ? nkvh / maps : nkvh;
+    // the work items of a stored query head: its turned pairs, its other dims, its zeros; of a (key head, map): the same without
+    // zeros (a joint head has them once, at its last map)
+    const int turned = half8 + (dh - rot_dim) / 8, q_items = turned + (dhp - dh) / 8, k_zeros = joint ? (dhp - maps * dh) / 8 : (dhp - dh) / 8;
+    const int k_items = turned + k_zeros, n_q = nh * q_items, n_k = store_kv ? nkvh * k_items : 0, n_v = store_kv ? stored_kvh * (dvp / 8) : 0;
+    const int w = blockIdx.y * 256 + threadIdx.x;
+    if (w >= n_q + n_k + n_v) return;
+    const TI *row = rows + (size_t)t * row_stride;
+    T *pg = nullptr;
+    int tok = 0;
+    if (w >= n_q) {
+        const int slot = slots[t];
+        if (slot < 0) return;
+        pg = cache + (size_t)(slot / page) * kv_page_elems(stored_kvh, dhp, dvp, page);
+        tok = slot % page;
+    }
+    if (w >= n_q + n_k) {
+        const int kvh = (w - n_q - n_k) / (dvp / 8), c0 = (w - n_q - n_k) % (dvp / 8) * 8;
+        QpRow8<TI> a = {};
+        if (c0 < dv) a = *(const QpRow8<TI> *)(row + v_off + (joint ? kvh : kvh / maps) * dv + c0);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) pg[kv_value_offset(stored_kvh, kvh, tok, c0 + e, dhp, dvp, page)] = from_f32<T>(to_f32(a.v[e]));
+        return;
+    }
+    const bool is_key = w >= n_q;
+    const int head = is_key ? (w - n_q) / k_items : w / q_items, item = is_key ? (w - n_q) % k_items : w % q_items;
+    const int map = maps > 1 ? head % maps : 0, at = joint ? map * dh : 0;
+    int place = joint && is_key ? head / maps : head;
+    if (!is_key && maps > 1 && !joint) {
+        const int group = nh / nkvh, qh = head / maps;
+        place = (qh / group * maps + map) * group + qh % group;
+    }
+    // where eight dims of the stored head lie
+    auto at_dim = [&](int c) -> QpRow8<T> * {
+        return (QpRow8<T> *)(is_key ? pg + kv_key_offset(place, tok, c, dhp, page) : q_out + (size_t)t * nh * dhp + (size_t)place * dhp + c);
+    };
+    if (item >= turned) {
+        // zeros: of a query every dim that is not its map's, of a key the dims behind the true ones
+        const int z = (item - turned) * 8;
+        if (is_key && joint && map != maps - 1) return;
+        const int c = is_key ? (joint ? maps * dh : dh) + z : (z < at ? z : z + dh);
+        QpRow8<T> o;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) o.v[e] = from_f32<T>(0.f);
+        *at_dim(c) = o;
+        return;
+    }
+    const TI *x = row + (is_key ? k_off : q_off) + head * dh;
+    if (item >= half8) {
+        const int c = rot_dim + (item - half8) * 8;
+        const QpRow8<TI> a = *(const QpRow8<TI> *)(x + c);
+        QpRow8<T> o;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) o.v[e] = from_f32<T>(to_f32(a.v[e]));
+        *at_dim(at + c) = o;
+        return;
+    }
+    const int i0 = item * 8, half = rot_dim / 2, pos = positions[t];
+    const bool in_table = pos >= 0 && pos < max_pos;
+    const size_t tab = (size_t)(in_table ? pos : 0) * half + i0;
+    const QpRow8<TI> a = *(const QpRow8<TI> *)(x + i0), b = *(const QpRow8<TI> *)(x + half + i0);
+    const QpRow8<float> cs = *(const QpRow8<float> *)(cos_t + tab), sn = *(const QpRow8<float> *)(sin_t + tab);
+    QpRow8<T> oa, ob;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+        float ra, rb;
+        rotate_pair(to_f32(a.v[e]), to_f32(b.v[e]), cs.v[e], sn.v[e], ra, rb);
+        if (!in_table) ra = rb = __uint_as_float(0x7fc00000u);        // a position outside the table gives NaN, not a wrong value
+        oa.v[e] = from_f32<T>(ra);
+        ob.v[e] = from_f32<T>(rb);
+    }
+    *at_dim(at + i0) = oa;
+    *at_dim(at + half + i0) = ob;
 }
 
 // rows: [n, row_stride] of in_type, a token's q heads at column q_off (nh * dh), k heads at k_off (nkvh * dh), v heads
@@ -111,12 +218,31 @@ LCU_API int lcu_qkv_prepare(const void *rows, int in_type, int n, int row_stride
     if (n <= 0) return LCU_OK;
     if (nh <= 0 || nkvh < 0 || dh <= 0 || dh > QP_MAX_DIM || dhp < dh || dhp % 8 || dhp > QP_MAX_DIM || dv <= 0 || dvp < dv ||
         dvp > QP_MAX_DIM || page <= 0 || page % 8 || rot_dim < 0 || rot_dim % 2 || rot_dim > dh || (pairing != 0 && pairing != 1) ||
-        !rows || !q_out || (cos_t && (!sin_t || !positions || rot_dim == 0)) || nh + 2 * nkvh > 65535 || maps < 1 || nh % maps || nkvh % maps || (joint && (maps < 2 || dhp < maps * dh)) ||
-        (maps > 1 && !store_kv))
+        !rows || !q_out || (cos_t && (!sin_t || !positions || rot_dim == 0)) || nh + 2 * nkvh > 65535 ||
+        maps < 1 || nh % maps || nkvh % maps || (joint && (maps < 2 || dhp < maps * dh)) || (maps > 1 && !store_kv))
         return LCU_BAD_ARGUMENT;
     if (store_kv && (!cache || !slots || nkvh <= 0)) return LCU_BAD_ARGUMENT;
-    dim3 grid(n, store_kv ? nh + nkvh + (joint ? nkvh / maps : nkvh) : nh), block(WAVE);
-#define GO(TI, T) qkv_prepare_kernel<TI, T><<<grid, block, 0, stream>>>((const TI *)rows, row_stride, q_off, k_off, v_off, bias, q_norm, k_norm, eps, positions, cos_t, sin_t, max_pos, rot_dim, pairing, (T *)q_out, slots, (T *)cache, nh, nkvh, dh, dhp, dv, dvp, page, store_kv, maps, joint)
+    const int stored_kvh = joint ? nkvh / maps : nkvh;
+    if (!bias && !q_norm && !k_norm && (!cos_t || (pairing == 0 && rot_dim % 16 == 0)) && dh % 8 == 0 && dv % 8 == 0 && dvp % 8 == 0 &&
+        row_stride % 8 == 0 && q_off % 8 == 0 && k_off % 8 == 0 && v_off % 8 == 0 && (uintptr_t)rows % 32 == 0 && (uintptr_t)q_out % 32 == 0 &&
+        (uintptr_t)cache % 32 == 0 && (uintptr_t)cos_t % 32 == 0 && (uintptr_t)sin_t % 32 == 0) {
+        const int rot = cos_t ? rot_dim : 0, turned = rot / 16 + (dh - rot) / 8;
+        const int items = nh * (turned + (dhp - dh) / 8) +
+                          (store_kv ? nkvh * (turned + (joint ? dhp - maps * dh : dhp - dh) / 8) + stored_kvh * (dvp / 8) : 0);
+        dim3 wgrid(n, (items + 255) / 256), wblock(256);
+#define WIDE(TI, T) qkv_prepare_wide_kernel<TI, T><<<wgrid, wblock, 0, stream>>>((const TI *)rows, row_stride, q_off, k_off, v_off, positions, cos_t, sin_t, max_pos, rot, (T *)q_out, slots, (T *)cache, nh, nkvh, dh, dhp, dv, dvp, page, store_kv ? 1 : 0, maps, joint)
+        if (in_type == LCU_F32 && type == LCU_F32) WIDE(float, float);
+        else if (in_type == LCU_F32 && type == LCU_BF16) WIDE(float, bf16_t);
+        else if (in_type == LCU_BF16 && type == LCU_BF16) WIDE(bf16_t, bf16_t);
+        else return LCU_BAD_ARGUMENT;
+#undef WIDE
+        LCU_LAUNCH_CHECK();
+        return LCU_OK;
+    }
+    const int heads = store_kv ? nh + nkvh + stored_kvh : nh;
+    dim3 grid(n, (heads + QP_WAVES - 1) / QP_WAVES), block(QP_WAVES * WAVE);
+    const size_t lds = (size_t)QP_WAVES * ((dh + 3) / 4 * 4) * sizeof(float);
+#define GO(TI, T) qkv_prepare_kernel<TI, T><<<grid, block, lds, stream>>>((const TI *)rows, row_stride, q_off, k_off, v_off, bias, q_norm, k_norm, eps, positions, cos_t, sin_t, max_pos, rot_dim, pairing, (T *)q_out, slots, (T *)cache, nh, nkvh, dh, dhp, dv, dvp, page, store_kv, maps, joint)
     if (in_type == LCU_F32 && type == LCU_F32) GO(float, float);
     else if (in_type == LCU_F32 && type == LCU_BF16) GO(float, bf16_t);
     else if (in_type == LCU_BF16 && type == LCU_BF16) GO(bf16_t, bf16_t);

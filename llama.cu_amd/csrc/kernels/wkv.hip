@@ -10,8 +10,8 @@
 //
 // A step of single tokens: one kernel per layer, a workgroup per (request, head), which streams the head's state through
 // its registers and makes everything between the projections and the output product.
-// Any other step: prep (parallel over tokens and heads; rows r, k, w, b, v of a head one after the other, so that the
-// scan's workgroups each stream a run of memory), scan, out.  The scan: column j of S depends on column j alone; a
+// Any other step: prep (parallel over tokens and heads: w and b, 32-bit, a head's tokens one after the other), scan, out.  The
+// scan (r, k and v as the projections left them go through LDS beside w, a stage of tokens at a time, the next stage on its way): column j of S depends on column j alone; a
 // workgroup keeps 64 columns of one head in registers, a lane four columns of a sixteenth of the key channels; the sum over
 // key channels crosses sixteen lanes after a stage of tokens.  A request that feeds at least WK_LONG tokens is cut into
 // WK_RUNS runs that are walked at once, twice: first from zeros, which gives what a run adds to any state it starts from
@@ -30,31 +30,56 @@ constexpr int WK_COLS = WK_THREADS / WK_LANES * WK_CPL;    // columns of a workg
 constexpr int WK_TOK = 8;                                  // tokens of a stage
 constexpr int WK_RUNS = 16;
 constexpr int WK_LONG = 512;
-constexpr int WK_PREP_TOK = 8;                             // tokens of a prep workgroup
+constexpr int WK_PREP_TOK = 16;                            // tokens of a prep workgroup
 
 // ---------------------------------------------------------------- the mix with the token before
 // h: [n, d] 32-bit; mu: [sets, d]; out: [sets, n, d].  The previous token's h of a request's first token of the step lies at
 // prev + slot * slot_stride (d floats); that token's workgroup also leaves the step's last h there (each thread reads an
 // element before it writes it, so nothing races).
-template <class T>
-__global__ void token_shift_kernel(const float *__restrict__ h, const float *__restrict__ mu, int sets, float *__restrict__ prev,
-                                   size_t slot_stride, const int *__restrict__ req_of_token, const int *__restrict__ q_start,
-                                   const int *__restrict__ ctx_len, const int *__restrict__ state_slot, T *__restrict__ out, int n, int d) {
-    const int t = blockIdx.x, r = req_of_token[t], t0 = q_start[r], t1 = q_start[r + 1];
-    const bool first = t == t0, fresh = ctx_len[r] - (t1 - t0) == 0;
-    float *ps = prev + (size_t)state_slot[r] * slot_stride;
-    const float *row = h + (size_t)t * d, *last = h + (size_t)(t1 - 1) * d;
-    for (int c = threadIdx.x; c < d; c += blockDim.x) {
-        const float x = row[c];
-        float before;
-        if (first) {
-            before = fresh ? 0.f : ps[c];
-            ps[c] = last[c];
-        } else {
-            before = row[c - d];
+// V neighbouring channels a thread, TB tokens one after the other (the weights are loaded once for them, and a token's own row is
+// the next one's row before).
+template <class T, int V> struct alignas(V * sizeof(T)) WkVec { T v[V]; };
+
+template <class T, int V, int TB>
+__global__ void __launch_bounds__(256)
+token_shift_kernel(const float *__restrict__ h, const float *__restrict__ mu, int sets, float *__restrict__ prev, size_t slot_stride,
+                   const int *__restrict__ req_of_token, const int *__restrict__ q_start, const int *__restrict__ ctx_len,
+                   const int *__restrict__ state_slot, T *__restrict__ out, int n, int d) {
+    constexpr int SETS = 8;                                    // weights kept in registers; more sets are walked in turn
+    const int c = (blockIdx.y * 256 + threadIdx.x) * V, t_first = blockIdx.x * TB, t_end = min(n, t_first + TB);
+    if (c >= d) return;
+    for (int s0 = 0; s0 < sets; s0 += SETS) {
+        WkVec<float, V> m[SETS];
+#pragma unroll
+        for (int s = 0; s < SETS; ++s)
+            if (s0 + s < sets) m[s] = *(const WkVec<float, V> *)(mu + (size_t)(s0 + s) * d + c);
+        WkVec<float, V> before = {};
+#pragma unroll
+        for (int b = 0; b < TB; ++b) {
+            const int t = t_first + b;
+            if (t >= t_end) break;
+            const int r = req_of_token[t], t0 = q_start[r], t1 = q_start[r + 1];
+            const WkVec<float, V> x = *(const WkVec<float, V> *)(h + (size_t)t * d + c);
+            if (t == t0) {
+                WkVec<float, V> *ps = (WkVec<float, V> *)(prev + (size_t)state_slot[r] * slot_stride + c);
+                before = *ps;
+                if (ctx_len[r] - (t1 - t0) == 0)
+#pragma unroll
+                    for (int e = 0; e < V; ++e) before.v[e] = 0.f;
+                if (s0 + SETS >= sets) *ps = *(const WkVec<float, V> *)(h + (size_t)(t1 - 1) * d + c);
+            } else if (b == 0) {
+                before = *(const WkVec<float, V> *)(h + (size_t)(t - 1) * d + c);
+            }
+#pragma unroll
+            for (int s = 0; s < SETS; ++s) {
+                if (s0 + s >= sets) break;
+                WkVec<T, V> o;
+#pragma unroll
+                for (int e = 0; e < V; ++e) o.v[e] = from_f32<T>(fmaf(before.v[e] - x.v[e], m[s].v[e], x.v[e]));
+                *(WkVec<T, V> *)(out + ((size_t)(s0 + s) * n + t) * d + c) = o;
+            }
+            before = x;
         }
-        const float diff = before - x;
-        for (int s = 0; s < sets; ++s) out[((size_t)s * n + t) * d + c] = from_f32<T>(fmaf(diff, mu[(size_t)s * d + c], x));
     }
 }
 
@@ -63,68 +88,87 @@ LCU_API int lcu_token_shift(const float *h, const float *mu, int sets, float *pr
                             hipStream_t stream) {
     if (n <= 0) return LCU_OK;
     if (d <= 0 || sets <= 0 || slot_stride < d || !h || !mu || !prev || !out) return LCU_BAD_ARGUMENT;
-    int threads = (d + 63) / 64 * 64;
-    if (threads > 512) threads = 512;
-#define GO(T) token_shift_kernel<T><<<dim3(n), dim3(threads), 0, stream>>>(h, mu, sets, prev, (size_t)slot_stride, req_of_token, q_start, ctx_len, state_slot, (T *)out, n, d)
-    if (out_type == LCU_F32) GO(float);
-    else if (out_type == LCU_BF16) GO(bf16_t);
+    const bool four = d % 4 == 0 && slot_stride % 4 == 0 && (uintptr_t)h % 16 == 0 && (uintptr_t)mu % 16 == 0 && (uintptr_t)prev % 16 == 0 &&
+                      (uintptr_t)out % 16 == 0;
+    const int v = four ? 4 : 1, tb = n >= 512 ? 4 : 1;
+    const dim3 grid((n + tb - 1) / tb, (d + 256 * v - 1) / (256 * v)), block(256);
+#define GO(T, V, TB) token_shift_kernel<T, V, TB><<<grid, block, 0, stream>>>(h, mu, sets, prev, (size_t)slot_stride, req_of_token, q_start, ctx_len, state_slot, (T *)out, n, d)
+#define SIZES(T)                          \
+    do {                                  \
+        if (four && tb == 4) GO(T, 4, 4); \
+        else if (four) GO(T, 4, 1);       \
+        else if (tb == 4) GO(T, 1, 4);    \
+        else GO(T, 1, 1);                 \
+    } while (0)
+    if (out_type == LCU_F32) SIZES(float);
+    else if (out_type == LCU_BF16) SIZES(bf16_t);
     else return LCU_BAD_ARGUMENT;
+#undef SIZES
 #undef GO
     LCU_LAUNCH_CHECK();
     return LCU_OK;
 }
 
 // ---------------------------------------------------------------- prep
-__host__ __device__ constexpr int wk_pad_keys(int d) { return d <= 64 ? 64 : d <= 128 ? 128 : 256; }      // key channels in a row: r, k and w each
+__host__ __device__ constexpr int wk_pad_keys(int d) { return d <= 64 ? 64 : d <= 128 ? 128 : 256; }      // key channels of a row of w (zeros behind the true ones)
 __host__ __device__ constexpr int wk_pad_cols(int dv) { return (dv + WK_COLS - 1) / WK_COLS * WK_COLS; }
-// a row: r, k, w (D each, zeros behind the true channels), b and three zeros, v (padded to whole workgroups' columns)
-__host__ __device__ constexpr int wk_row(int D, int DV) { return 3 * D + 4 + DV; }
 
-// rows: [n, row_stride] with r, k (heads * d) and v (heads * dv) at their columns; low: [n, ld_low] 32-bit; w2t: [rank, heads * d].
+// rows: [n, row_stride] with r and k (heads * d) at their columns; low: [n, ld_low] 32-bit; w2t: [rank, heads * d].  To w: [heads][n][D]
+// and bonus: [heads][n].
+// A workgroup has 256 threads, D of them a head: 256 / D heads of WK_PREP_TOK tokens, a thread per key channel.  The rank's numbers
+// lie in LDS with the tokens side by side: every thread reads the same four at a time.
 template <class T>
-__global__ void wkv_prep_kernel(const T *__restrict__ rows, int row_stride, int r_off, int k_off, int v_off, const float *__restrict__ low,
-                                int ld_low, const float *__restrict__ w2t, const float *__restrict__ w0, const float *__restrict__ u,
-                                float *__restrict__ prep, int n, int heads, int d, int dv, int rank, int D, int DV) {
-    __shared__ float th[WK_PREP_TOK * WK_MAX_RANK];
-    __shared__ float part[WK_PREP_TOK][4];
-    const int t0 = blockIdx.x * WK_PREP_TOK, h = blockIdx.y, nt = min(WK_PREP_TOK, n - t0);
-    for (int x = threadIdx.x; x < nt * rank; x += blockDim.x) th[x] = tanhf(low[(size_t)(t0 + x / rank) * ld_low + x % rank]);
+__global__ void __launch_bounds__(256)
+wkv_prep_kernel(const T *__restrict__ rows, int row_stride, int r_off, int k_off, const float *__restrict__ low, int ld_low,
+                const float *__restrict__ w2t, const float *__restrict__ w0, const float *__restrict__ u, float *__restrict__ w_out,
+                float *__restrict__ bonus, int n, int heads, int d, int rank, int D) {
+    constexpr int TB = WK_PREP_TOK;
+    extern __shared__ float4 th4[];                            // [rank][TB]
+    __shared__ float part[TB][4];
+    float *th = (float *)th4;
+    const int t0 = blockIdx.x * TB, nt = min(TB, n - t0);
+    for (int x = threadIdx.x; x < TB * rank; x += 256) {
+        const int b = x / rank, j = x % rank;                  // (neighbouring threads, neighbouring addresses in memory)
+        th[j * TB + b] = b < nt ? tanhf(low[(size_t)(t0 + b) * ld_low + j]) : 0.f;
+    }
     __syncthreads();
-    const int i = threadIdx.x, c = h * d + i;                  // blockDim.x == D: a thread per key channel
-    const bool live = i < d;
-    float z[WK_PREP_TOK];
+    const int h = blockIdx.y * (256 / D) + threadIdx.x / D, i = threadIdx.x % D, c = h * d + i;
+    const bool live = i < d && h < heads;
+    float z[TB];
 #pragma unroll
-    for (int b = 0; b < WK_PREP_TOK; ++b) z[b] = live ? w0[c] : 0.f;
+    for (int b = 0; b < TB; ++b) z[b] = live ? w0[c] : 0.f;
     if (live) {
 #pragma unroll 4
         for (int j = 0; j < rank; ++j) {
             const float w = w2t[(size_t)j * heads * d + c];
 #pragma unroll
-            for (int b = 0; b < WK_PREP_TOK; ++b) z[b] = fmaf(w, b < nt ? th[b * rank + j] : 0.f, z[b]);
+            for (int b = 0; b < TB; b += 4) {
+                const float4 q = th4[(j * TB + b) / 4];
+                z[b] = fmaf(w, q.x, z[b]);
+                z[b + 1] = fmaf(w, q.y, z[b + 1]);
+                z[b + 2] = fmaf(w, q.z, z[b + 2]);
+                z[b + 3] = fmaf(w, q.w, z[b + 3]);
+            }
         }
     }
-    const int R = wk_row(D, DV);
     const float uu = live ? u[c] : 0.f;
+    float own[TB];                                             // r u k of the thread's channel
 #pragma unroll
-    for (int b = 0; b < WK_PREP_TOK; ++b) {
-        if (b >= nt) break;
-        const T *row = rows + (size_t)(t0 + b) * row_stride;
-        float *o = prep + ((size_t)h * n + t0 + b) * R;
-        const float rr = live ? to_f32(row[r_off + c]) : 0.f, kk = live ? to_f32(row[k_off + c]) : 0.f;
-        o[i] = rr;
-        o[D + i] = kk;
-        o[2 * D + i] = live ? expf(-expf(z[b])) : 0.f;
-        for (int j = i; j < DV; j += D) o[3 * D + 4 + j] = j < dv ? to_f32(row[v_off + h * dv + j]) : 0.f;
-        const float s = wave_sum(rr * uu * kk);
-        if ((i & (WAVE - 1)) == 0) part[b][i / WAVE] = s;
+    for (int b = 0; b < TB; ++b) {
+        const T *row = rows + (size_t)(t0 + min(b, nt - 1)) * row_stride + (live ? c : 0);       // (no branch around a load)
+        own[b] = to_f32(row[r_off]) * uu * to_f32(row[k_off]);
+    }
+#pragma unroll
+    for (int b = 0; b < TB; ++b) {
+        const float s = wave_sum_in_place(own[b]);
+        if ((threadIdx.x & (WAVE - 1)) == 0) part[b][threadIdx.x / WAVE] = s;
+        if (h < heads && b < nt) w_out[((size_t)h * n + t0 + b) * D + i] = live ? expf(-expf(z[b])) : 0.f;
     }
     __syncthreads();
-    if (i < 4 * nt) {
-        const int b = i / 4;
+    if (i < nt && h < heads) {
         float s = 0.f;
-        if (i % 4 == 0)
-            for (int w = 0; w < D / WAVE; ++w) s += part[b][w];
-        prep[((size_t)h * n + t0 + b) * R + 3 * D + i % 4] = s;
+        for (int w = 0; w < D / WAVE; ++w) s += part[i][threadIdx.x / D * (D / WAVE) + w];
+        bonus[(size_t)h * n + t0 + i] = s;
     }
 }
 
@@ -138,17 +182,20 @@ __device__ __forceinline__ int wk_long_index(const int *__restrict__ q_start, in
 
 // MODE 0: a request of fewer than WK_LONG tokens in one chain; 1: a run from zeros, leaves B in run_b and the product of its w in
 // run_p; 2: a run from run_in, with outputs.  o: [heads][n][DV].  run_b, run_in: [long request][run][heads][d][dv], run_p: [..][heads][d].
-template <int DPL, int MODE>
+// FOUR: d, dv and every column and stride are multiples of 4 (r, k and v are loaded four at a time).
+template <class T> struct alignas(4 * sizeof(T)) WkQuad { T v[4]; };
+
+template <class T, int DPL, int MODE, bool FOUR>
 __global__ void __launch_bounds__(WK_THREADS)
-wkv_scan_kernel(const float *__restrict__ prep, float *__restrict__ state, size_t slot_stride, float *__restrict__ o_out,
+wkv_scan_kernel(const T *__restrict__ rows, int row_stride, int r_off, int k_off, int v_off, const float *__restrict__ w_in,
+                const float *__restrict__ bonus, float *__restrict__ state, size_t slot_stride, float *__restrict__ o_out,
                 const int *__restrict__ q_start, const int *__restrict__ ctx_len, const int *__restrict__ state_slot,
                 float *__restrict__ run_b, float *__restrict__ run_p, const float *__restrict__ run_in, int n, int nh, int d, int dv, int DV) {
     constexpr int D = WK_LANES * DPL, TOK = WK_TOK;
-    constexpr int HEAD = 3 * D + 4;                            // floats of a token's row in front of v
-    constexpr int V4 = TOK * HEAD / 4;                         // float4s of a stage before its values
-    constexpr int STAGE4 = V4 + TOK * WK_COLS / 4;
-    constexpr int PER = (STAGE4 + WK_THREADS - 1) / WK_THREADS;
-    __shared__ float4 lds[2][STAGE4];
+    constexpr int G = (2 * D + WK_COLS) / 4;                   // groups of four of a token: r, k, the workgroup's columns of v
+    constexpr int PER = (TOK * G + WK_THREADS - 1) / WK_THREADS, PER_W = (TOK * D / 4 + WK_THREADS - 1) / WK_THREADS;
+    __shared__ float4 lds[2][TOK][G], lds_w[2][TOK][D / 4];
+    __shared__ float lds_b[2][TOK];
     const int r = MODE == 0 ? blockIdx.z : blockIdx.z / WK_RUNS, run = MODE == 0 ? 0 : blockIdx.z % WK_RUNS;
     const int h = blockIdx.y, col0 = blockIdx.x * WK_COLS;
     int t0 = q_start[r], t1 = q_start[r + 1];
@@ -172,47 +219,68 @@ wkv_scan_kernel(const float *__restrict__ prep, float *__restrict__ state, size_
 #pragma unroll
         for (int c = 0; c < WK_CPL; ++c) s[e][c] = (from && i < d && col + c < dv) ? from[(size_t)i * dv + col + c] : 0.f;
     }
-    const int R4 = (HEAD + DV) / 4;
-    const float4 *src = (const float4 *)prep + (size_t)h * n * R4;
-    // element x of a stage: the rows of its tokens up to their values, then the workgroup's columns of the values.  Beyond the
-    // last token everything is zero and w is 1, which leaves the state.
-    auto fetch = [&](int base, int x) -> float4 {
-        const bool is_v = x >= V4;
-        const int tt = is_v ? (x - V4) / (WK_COLS / 4) : x / (HEAD / 4), at = is_v ? (x - V4) % (WK_COLS / 4) : x % (HEAD / 4);
-        const int t = base + tt;
-        if (x >= STAGE4 || t >= t1) {
-            const float fill = !is_v && at >= D / 2 && at < 3 * D / 4 ? 1.f : 0.f;
-            return make_float4(fill, fill, fill, fill);
+    // a stage's numbers on their way: the loads stand under no branch (a place beyond the last token or channel is clamped), and
+    // what they brought is converted when it goes to LDS.  Beyond the last token r, k and v are zero and w is 1, which leaves
+    // the state.
+    WkQuad<T> next[PER];
+    float4 next_w[PER_W];
+    float next_b = 0.f;
+    auto fetch = [&](int base) {
+#pragma unroll
+        for (int p = 0; p < PER; ++p) {
+            const int x = threadIdx.x + p * WK_THREADS, t = min(base + x / G, t1 - 1), g = x % G;
+            const bool is_r = g < D / 4, is_v = g >= D / 2;
+            const int at = is_r ? 4 * g : is_v ? col0 + 4 * g - 2 * D : 4 * g - D, limit = is_v ? dv : d;
+            const T *from_row = rows + (size_t)t * row_stride + (is_r ? r_off + h * d : is_v ? v_off + h * dv : k_off + h * d);
+            if (FOUR) next[p] = *(const WkQuad<T> *)(from_row + min(at, limit - 4));
+            else
+#pragma unroll
+                for (int e = 0; e < 4; ++e) next[p].v[e] = from_row[min(at + e, limit - 1)];
         }
-        return src[(size_t)t * R4 + (is_v ? HEAD / 4 + col0 / 4 + at : at)];
+#pragma unroll
+        for (int p = 0; p < PER_W; ++p) {
+            const int x = threadIdx.x + p * WK_THREADS, t = min(base + x / (D / 4), t1 - 1);
+            next_w[p] = *(const float4 *)(w_in + ((size_t)h * n + t) * D + x % (D / 4) * 4);
+        }
+        next_b = bonus[(size_t)h * n + min(base + (int)threadIdx.x, t1 - 1)];
     };
-    float4 next[PER];
+    auto put = [&](int base, int to) {
 #pragma unroll
-    for (int k = 0; k < PER; ++k) next[k] = fetch(t0, threadIdx.x + k * WK_THREADS);
+        for (int p = 0; p < PER; ++p) {
+            const int x = threadIdx.x + p * WK_THREADS, tt = x / G, g = x % G;
+            const bool is_r = g < D / 4, is_v = g >= D / 2;
+            const int at = is_r ? 4 * g : is_v ? col0 + 4 * g - 2 * D : 4 * g - D, limit = base + tt < t1 ? (is_v ? dv : d) : 0;
+            if (TOK * G % WK_THREADS && x >= TOK * G) break;
+            lds[to][tt][g] = make_float4(at < limit ? to_f32(next[p].v[0]) : 0.f, at + 1 < limit ? to_f32(next[p].v[1]) : 0.f,
+                                         at + 2 < limit ? to_f32(next[p].v[2]) : 0.f, at + 3 < limit ? to_f32(next[p].v[3]) : 0.f);
+        }
 #pragma unroll
-    for (int k = 0; k < PER; ++k)
-        if (threadIdx.x + k * WK_THREADS < STAGE4) lds[0][threadIdx.x + k * WK_THREADS] = next[k];
+        for (int p = 0; p < PER_W; ++p) {
+            const int x = threadIdx.x + p * WK_THREADS, tt = x / (D / 4);
+            if (TOK * D / 4 % WK_THREADS && x >= TOK * D / 4) break;
+            lds_w[to][tt][x % (D / 4)] = base + tt < t1 ? next_w[p] : make_float4(1.f, 1.f, 1.f, 1.f);
+        }
+        if (threadIdx.x < TOK) lds_b[to][threadIdx.x] = next_b;
+    };
+    fetch(t0);
+    put(t0, 0);
     __syncthreads();
     int buf = 0;
     for (int base = t0; base < t1; base += TOK, buf ^= 1) {
         const int nt = min(TOK, t1 - base);
         const bool more = base + TOK < t1;
-        if (more) {
-#pragma unroll
-            for (int k = 0; k < PER; ++k) next[k] = fetch(base + TOK, threadIdx.x + k * WK_THREADS);
-        }
-        const float4 *cur = lds[buf];
+        if (more) fetch(base + TOK);
         float acc[TOK][WK_CPL];
 #pragma unroll
         for (int tt = 0; tt < TOK; ++tt) {
-            const float4 *row = cur + tt * (HEAD / 4) + sub * (DPL / 4);
-            const float4 v4 = cur[V4 + tt * (WK_COLS / 4) + cg];
+            const float4 *row = lds[buf][tt] + sub * (DPL / 4), *w_row = lds_w[buf][tt] + sub * (DPL / 4);
+            const float4 v4 = lds[buf][tt][D / 2 + cg];
             const float v[4] = {v4.x, v4.y, v4.z, v4.w};
 #pragma unroll
             for (int c = 0; c < WK_CPL; ++c) acc[tt][c] = 0.f;
 #pragma unroll
             for (int e4 = 0; e4 < DPL / 4; ++e4) {
-                const float4 k4 = row[D / 4 + e4], w4 = row[D / 2 + e4];
+                const float4 k4 = row[D / 4 + e4], w4 = w_row[e4];
                 const float4 r4 = MODE == 1 ? make_float4(0.f, 0.f, 0.f, 0.f) : row[e4];
                 const float kk[4] = {k4.x, k4.y, k4.z, k4.w}, ww[4] = {w4.x, w4.y, w4.z, w4.w}, rr[4] = {r4.x, r4.y, r4.z, r4.w};
 #pragma unroll
@@ -238,17 +306,13 @@ wkv_scan_kernel(const float *__restrict__ prep, float *__restrict__ state, size_
                     if (sub == tt) mine[c] = a;
                 }
             if (sub < nt) {
-                const float b = cur[sub * (HEAD / 4) + 3 * D / 4].x;
-                const float4 v4 = cur[V4 + sub * (WK_COLS / 4) + cg];
+                const float b = lds_b[buf][sub];
+                const float4 v4 = lds[buf][sub][D / 2 + cg];
                 *(float4 *)(o_out + ((size_t)h * n + base + sub) * DV + col) =
                     make_float4(fmaf(b, v4.x, mine[0]), fmaf(b, v4.y, mine[1]), fmaf(b, v4.z, mine[2]), fmaf(b, v4.w, mine[3]));
             }
         }
-        if (more) {
-#pragma unroll
-            for (int k = 0; k < PER; ++k)
-                if (threadIdx.x + k * WK_THREADS < STAGE4) lds[buf ^ 1][threadIdx.x + k * WK_THREADS] = next[k];
-        }
+        if (more) put(base + TOK, buf ^ 1);
         __syncthreads();
     }
     if (MODE == 2 && run != WK_RUNS - 1) return;
@@ -286,27 +350,27 @@ __global__ void wkv_chain_kernel(const float *__restrict__ state, size_t slot_st
 }
 
 // ---------------------------------------------------------------- out
-// One wave per (token, head): o / rms(o) * weight * silu(gate).
+// One wave per (token, head), four to a workgroup: o / rms(o) * weight * silu(gate).
 template <class TG, class T>
-__global__ void __launch_bounds__(WAVE)
+__global__ void __launch_bounds__(256)
 wkv_out_kernel(const float *__restrict__ o, int DV, const TG *__restrict__ rows, int row_stride, int g_off, const float *__restrict__ weight,
                T *__restrict__ out, int n, int nh, int dv, float eps) {
-    const int t = blockIdx.x, h = blockIdx.y;
+    const int t = blockIdx.x, h = blockIdx.y * 4 + threadIdx.x / WAVE, lane = threadIdx.x & (WAVE - 1);
+    if (h >= nh) return;
     const float *oh = o + ((size_t)h * n + t) * DV;
-    float x[4], ss = 0.f;
+    float x[4], z[4], ss = 0.f;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-        const int j = threadIdx.x + WAVE * i;
+        const int j = lane + WAVE * i;
         x[i] = j < dv ? oh[j] : 0.f;
+        z[i] = j < dv ? to_f32(rows[(size_t)t * row_stride + g_off + h * dv + j]) : 0.f;
         ss += x[i] * x[i];
     }
-    const float f = 1.0f / sqrtf(wave_sum(ss) / (float)dv + eps);
+    const float f = 1.0f / sqrtf(wave_sum_in_place(ss) / (float)dv + eps);
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-        const int j = threadIdx.x + WAVE * i, c = h * dv + j;
-        if (j >= dv) break;
-        const float z = to_f32(rows[(size_t)t * row_stride + g_off + c]);
-        out[(size_t)t * nh * dv + c] = from_f32<T>(x[i] * f * weight[c] * (z / (1.0f + expf(-z))));
+        const int j = lane + WAVE * i, c = h * dv + j;
+        if (j < dv) out[(size_t)t * nh * dv + c] = from_f32<T>(x[i] * f * weight[c] * (z[i] / (1.0f + expf(-z[i]))));
     }
 }
 
@@ -404,9 +468,7 @@ wkv_single_kernel(const TG *__restrict__ rows, int row_stride, int r_off, int k_
 }
 
 // The floats of the scratch arrays for a step of n tokens whose `n_long` requests feed at least WK_LONG of them.
-LCU_API long long lcu_wkv_prep_floats(int n, int heads, int d, int dv) {
-    return (long long)n * heads * wk_row(wk_pad_keys(d), wk_pad_cols(dv));
-}
+LCU_API long long lcu_wkv_prep_floats(int n, int heads, int d) { return (long long)n * heads * (wk_pad_keys(d) + 1); }
 LCU_API long long lcu_wkv_out_floats(int n, int heads, int dv) { return (long long)n * heads * wk_pad_cols(dv); }
 LCU_API long long lcu_wkv_run_floats(int n_long, int heads, int d, int dv) {
     return (long long)n_long * WK_RUNS * heads * d * (2ll * dv + 1);
@@ -429,34 +491,47 @@ LCU_API int lcu_wkv(const void *rows, int rows_type, int row_stride, int r_off, 
     if (!wkv_sizes_ok(heads, d, dv, rank, slot_stride) || !prep || !o || n_long < 0 || (n_long > 0 && !runs) || n_req * WK_RUNS > 65535)
         return LCU_BAD_ARGUMENT;
     const int D = wk_pad_keys(d), DV = wk_pad_cols(dv);
-    const dim3 pg((n + WK_PREP_TOK - 1) / WK_PREP_TOK, heads);
-    if (rows_type == LCU_F32)
-        wkv_prep_kernel<float><<<pg, dim3(D), 0, stream>>>((const float *)rows, row_stride, r_off, k_off, v_off, low, ld_low, w2t, w0, u, prep, n, heads, d, dv, rank, D, DV);
-    else if (rows_type == LCU_BF16)
-        wkv_prep_kernel<bf16_t><<<pg, dim3(D), 0, stream>>>((const bf16_t *)rows, row_stride, r_off, k_off, v_off, low, ld_low, w2t, w0, u, prep, n, heads, d, dv, rank, D, DV);
-    else
-        return LCU_BAD_ARGUMENT;
-    LCU_LAUNCH_CHECK();
+    const dim3 pg((n + WK_PREP_TOK - 1) / WK_PREP_TOK, (heads + 256 / D - 1) / (256 / D));
+    const size_t plds = (size_t)rank * WK_PREP_TOK * sizeof(float);
+    float *w_buf = prep, *bonus = prep + (size_t)n * heads * D;
     const size_t one = (size_t)n_long * WK_RUNS * heads * d;
     float *run_b = runs, *run_in = runs ? runs + one * dv : nullptr, *run_p = runs ? run_in + one * dv : nullptr;
-#define SCAN(DPL, MODE, Z) wkv_scan_kernel<DPL, MODE><<<dim3(DV / WK_COLS, heads, Z), dim3(WK_THREADS), 0, stream>>>(prep, state, (size_t)slot_stride, o, q_start, ctx_len, state_slot, run_b, run_p, run_in, n, heads, d, dv, DV)
-#define MODES(DPL)                                                                                                              \
+    const bool four = d % 4 == 0 && dv % 4 == 0 && row_stride % 4 == 0 && r_off % 4 == 0 && k_off % 4 == 0 && v_off % 4 == 0 && (uintptr_t)rows % 16 == 0;
+#define SCAN(T, DPL, MODE, Z)                                                                                                                     \
+    do {                                                                                                                                        \
+        if (four) SCAN_AS(T, DPL, MODE, true, Z);                                                                                               \
+        else SCAN_AS(T, DPL, MODE, false, Z);                                                                                                   \
+    } while (0)
+#define SCAN_AS(T, DPL, MODE, FOUR, Z)                                                                                                            \
+    wkv_scan_kernel<T, DPL, MODE, FOUR><<<dim3(DV / WK_COLS, heads, Z), dim3(WK_THREADS), 0, stream>>>((const T *)rows, row_stride, r_off, k_off, \
+        v_off, w_buf, bonus, state, (size_t)slot_stride, o, q_start, ctx_len, state_slot, run_b, run_p, run_in, n, heads, d, dv, DV)
+#define MODES(T, DPL)                                                                                                           \
     do {                                                                                                                        \
-        if (n_long < n_req) SCAN(DPL, 0, n_req);                                                                                \
+        if (n_long < n_req) SCAN(T, DPL, 0, n_req);                                                                             \
         if (n_long > 0) {                                                                                                       \
-            SCAN(DPL, 1, n_req * WK_RUNS);                                                                                      \
+            SCAN(T, DPL, 1, n_req * WK_RUNS);                                                                                   \
             wkv_chain_kernel<<<dim3((d * dv + 255) / 256, heads, n_req), dim3(256), 0, stream>>>(state, (size_t)slot_stride,   \
                 run_b, run_p, run_in, q_start, ctx_len, state_slot, heads, d, dv);                                              \
-            SCAN(DPL, 2, n_req * WK_RUNS);                                                                                      \
+            SCAN(T, DPL, 2, n_req * WK_RUNS);                                                                                   \
         }                                                                                                                       \
     } while (0)
-    if (D == 64) MODES(4);
-    else if (D == 128) MODES(8);
-    else MODES(16);
+#define ALL(T)                                                                                                                                  \
+    do {                                                                                                                                        \
+        wkv_prep_kernel<T><<<pg, dim3(256), plds, stream>>>((const T *)rows, row_stride, r_off, k_off, low, ld_low, w2t, w0, u, w_buf, bonus, n, \
+                                                            heads, d, rank, D);                                                                 \
+        if (D == 64) MODES(T, 4);                                                                                                               \
+        else if (D == 128) MODES(T, 8);                                                                                                         \
+        else MODES(T, 16);                                                                                                                      \
+    } while (0)
+    if (rows_type == LCU_F32) ALL(float);
+    else if (rows_type == LCU_BF16) ALL(bf16_t);
+    else return LCU_BAD_ARGUMENT;
+#undef ALL
 #undef MODES
 #undef SCAN
+#undef SCAN_AS
     LCU_LAUNCH_CHECK();
-#define OUT(TG, T) wkv_out_kernel<TG, T><<<dim3(n, heads), dim3(WAVE), 0, stream>>>(o, DV, (const TG *)rows, row_stride, g_off, weight, (T *)out, n, heads, dv, eps)
+#define OUT(TG, T) wkv_out_kernel<TG, T><<<dim3(n, (heads + 3) / 4), dim3(256), 0, stream>>>(o, DV, (const TG *)rows, row_stride, g_off, weight, (T *)out, n, heads, dv, eps)
     if (rows_type == LCU_F32 && out_type == LCU_F32) OUT(float, float);
     else if (rows_type == LCU_F32 && out_type == LCU_BF16) OUT(float, bf16_t);
     else if (rows_type == LCU_BF16 && out_type == LCU_BF16) OUT(bf16_t, bf16_t);

@@ -1687,7 +1687,7 @@ def wkv(rows: torch.Tensor, offsets: Dict[str, int], low: torch.Tensor, w2_t: to
         f.restype = ctypes.c_longlong
     n_long = sum(1 for q in step.q_lens if q >= lib.lcu_wkv_long())
     f32 = lambda size: torch.empty(size, dtype=torch.float32, device=rows.device)
-    prep, o = f32(lib.lcu_wkv_prep_floats(n, heads, dim, dim)), f32(lib.lcu_wkv_out_floats(n, heads, dim))
+    prep, o = f32(lib.lcu_wkv_prep_floats(n, heads, dim)), f32(lib.lcu_wkv_out_floats(n, heads, dim))
     runs = f32(lib.lcu_wkv_run_floats(n_long, heads, dim, dim)) if n_long else None
     _check(lib.lcu_wkv(*head, _ptr(prep), _ptr(o), _ptr(runs), n_long, *slot, n, step.n_req, heads, dim, dim, rank, ctypes.c_float(eps),
                        _stream()), "wkv")
