@@ -448,21 +448,21 @@ def mufotar_config(z, positions):
 def gefudra_config(z, positions):
     """As many layer runs as the Llama model beside it has layers, each with its dense feed-forward: latent attention (a latent of
     128, one head of the matrix-core attention kernels' largest size; queries through a latent of 3/8 of the width; a window
-    of 1,024), then the recurrent mixer (heads of 64), latent attention and differential attention (two maps of half a
-    Llama head over values of a whole one) as a loop that runs twice where there are eight runs, then latent attention."""
+    of 1,024), differential attention (two maps of half a Llama head over values of a whole one) and the recurrent mixer
+    (heads of 64) as a loop that runs twice where there are eight runs, then latent attention."""
     from llama_cu_amd.config import GefudraConfig
     inter = (z["top"] * 2 * z["ff"] // 3 + 127) // 128 * 128
     d, h, g, w = z["dim"], z["heads"], z["kv_heads"], z["width"]
     latent = {"type": "latent_attention", "mixer": {"heads": h, "dim": d, "vdim": d, "kv_rank": 128, "q_rank": 3 * w // 8, "scale": d ** -0.5,
                                                     "mask": {"size": 1024}}}
     mixer = {"type": "wkv", "mixer": {"heads": w // 64, "dim": 64, "rank": 64}}
-    differential = {"type": "attention", "mixer": {"heads": h, "kv_heads": g, "dim": d // 2, "vdim": d, "scale": (d // 2) ** -0.5, "diff": 0.5,
-                                                   "softcap": 30.0, "rot": {"dims": d // 2, "base": 50000.0}}}
-    times, left = divmod(z["layers"] - 1, 3)
-    layers = [latent, mixer, latent, differential] + [latent] * left
-    return GefudraConfig.from_dict({"architecture": "Gefudra", "vocab": z["vocab"], "width": w, "norm": {"eps": 1e-6}, "residual_mult": 0.5,
-                                    "logit_scale": 0.5, "layers": [dict(l, mlp={"kind": "dense", "ff": inter, "limit": 7.0}) for l in layers],
-                                    "loop": {"start": 1, "stop": 4, "times": times}, "max_positions": positions})
+    differential = {"type": "attention", "mixer": {"heads": h, "kv_heads": g, "dim": d // 2, "vdim": d, "scale": (d // 2) ** -0.5, "diff": 0.6,
+                                                   "softcap": 50.0, "rot": {"dims": d // 2, "base": 10000.0}}}
+    times = (z["layers"] - 1) // 3
+    layers = [latent, differential, mixer] + [latent] * (z["layers"] - 3 * times)
+    return GefudraConfig.from_dict({"architecture": "Gefudra", "vocab": z["vocab"], "width": w, "norm": {"eps": 1e-5}, "residual_mult": 0.7,
+                                    "logit_scale": 0.25, "layers": [dict(l, mlp={"kind": "dense", "ff": inter, "limit": 7.0}) for l in layers],
+                                    "loop": {"start": 0, "stop": 3, "times": times}, "max_positions": positions})
 
 
 DESIGN_CONFIGS = {"divasun": lambda z, p: divasun_config(z, p), "llama": lambda z, p: llama_like(z, p),
