@@ -190,8 +190,6 @@ def test_latent_attention_without_positions(dtype, m, page, folded):
     d, eps = 64, 1e-5
     cfg = config(16, d, [layer("latent_attention", m)], eps)
     w = mixer_weights(cfg, 11)
-    if page % 16 and dtype == "bfloat16":
-        page = 16
     part = built("mixer", "latent_attention", {
         "hidden_size": d, "heads": m["heads"], "head_dim": m["dim"], "rot_dim": 0, "value_dim": m["vdim"], "kv_rank": m["kv_rank"],
         "q_rank": m["q_rank"], "scale": m["scale"], "norm_eps": eps, "window": m["mask"]["size"] if "mask" in m else 0, "sink": True,
