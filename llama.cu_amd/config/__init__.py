@@ -7,9 +7,10 @@ from .lozezen import LozezenConfig
 from .ralepel import RalepelConfig
 from .mufotar import MufotarConfig
 from .gefudra import GefudraConfig
+from .lapunex import LapunexConfig
 from .registry import (Architecture, architecture_of, register_architecture, registered_architectures, load_config,
                        load_plugins, load_plugins_from_env, PLUGINS_ENV)
 
-__all__ = ["ConfigError", "read_config_json", "LlamaConfig", "DivasunConfig", "LozezenConfig", "RalepelConfig", "MufotarConfig", "GefudraConfig", "Architecture", "architecture_of",
+__all__ = ["ConfigError", "read_config_json", "LlamaConfig", "DivasunConfig", "LozezenConfig", "RalepelConfig", "MufotarConfig", "GefudraConfig", "LapunexConfig", "Architecture", "architecture_of",
            "register_architecture", "registered_architectures", "load_config", "load_plugins", "load_plugins_from_env",
            "PLUGINS_ENV"]

@@ -5,13 +5,13 @@
 #include "gate_act.h"
 
 // ---------------------------------------------------------------- embedding gather
-// out[i, :] = table[ids[i], :] * scale (the product in 32-bit).  An id outside the table writes NaN into the row
+// out[i, k, :] = table[ids[i], :] * scale for k < copies (the product in 32-bit).  An id outside the table writes NaN into the row
 // (the host checks ids before; this keeps a bad id from reading out of bounds).
 template <class TT, class TO>
 __global__ void embedding_gather_kernel(TO *__restrict__ out, const TT *__restrict__ table,
-                                        const int *__restrict__ ids, int d, int vocab, float scale) {
+                                        const int *__restrict__ ids, int d, int vocab, float scale, int copies) {
     const int row = blockIdx.x;
-    const int id = ids[row];
+    const int id = ids[row / copies];
     TO *o = out + (size_t)row * d;
     if (id < 0 || id >= vocab) {
         for (int c = threadIdx.x; c < d; c += blockDim.x) o[c] = from_f32<TO>(__uint_as_float(0x7fc00000u));
@@ -35,11 +35,11 @@ __global__ void embedding_gather_kernel(TO *__restrict__ out, const TT *__restri
 }
 
 LCU_API int lcu_embedding_gather(void *out, int out_type, const void *table, int table_type,
-                                 const int *ids, int n, int d, int vocab, float scale, hipStream_t stream) {
+                                 const int *ids, int n, int d, int vocab, float scale, int copies, hipStream_t stream) {
     if (n <= 0) return LCU_OK;
-    if (d <= 0 || vocab <= 0) return LCU_BAD_ARGUMENT;
-    dim3 grid(n), block(256);
-#define GO(TT, TO) embedding_gather_kernel<TT, TO><<<grid, block, 0, stream>>>((TO *)out, (const TT *)table, ids, d, vocab, scale)
+    if (d <= 0 || vocab <= 0 || copies <= 0) return LCU_BAD_ARGUMENT;
+    dim3 grid((unsigned)n * copies), block(256);
+#define GO(TT, TO) embedding_gather_kernel<TT, TO><<<grid, block, 0, stream>>>((TO *)out, (const TT *)table, ids, d, vocab, scale, copies)
     if (table_type == LCU_F32 && out_type == LCU_F32) GO(float, float);
     else if (table_type == LCU_BF16 && out_type == LCU_F32) GO(bf16_t, float);
     else if (table_type == LCU_BF16 && out_type == LCU_BF16) GO(bf16_t, bf16_t);

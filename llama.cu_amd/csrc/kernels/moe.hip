@@ -3,13 +3,13 @@
 //   route:   z = W_router h (+ bias) (32-bit), the `top` experts with the largest z (ties: the lower
 //            index), each with the weight sigmoid(z) (a token's weights are not made to add up to one) or,
 //            in the other mode, with the softmax over the chosen logits alone; or, in a third, with scores s = softmax(z)
-//            over all experts, the choice by s + a correction per expert, and the chosen scores divided by their sum as
-//            weights; rows of the router's matrix behind the experts' are gates: sigmoid of their logit goes out per
+//            over all experts, the choice by s + a correction per expert, and the chosen scores divided by their sum (or as
+//            they are) times a factor as weights; the choice may be limited to the experts of the best groups; rows of the router's matrix behind the experts' are gates: sigmoid of their logit goes out per
 //            token; the last experts may be identity experts, which have no matrices and return their input;
 //   group:   the (token, choice) pairs sorted by expert and cut into tiles of up to 16 or 64 rows of
 //            one expert, on the device (nothing comes back to the host);
 //   up:      act = gelu(W_up[e] (weight * h))    the weight scales what goes INTO the expert; or, gated:
-//            act = silu(W_gate[e] h) * (W_up[e] h), and the weight scales what comes OUT of the expert
+//            act = silu(W_gate[e] h) * (W_up[e] h) (or the limited form, gate_act.h), and the weight scales what comes OUT of the expert
 //   down:    y = W_down[e] act, added to the token's output row (32-bit), in the gated form times the weight
 //            and beside a shared expert's row times its gate.
 // The products run on the matrix cores: bfloat16 operands with v_mfma_f32_16x16x32_bf16, or
@@ -17,6 +17,7 @@
 // row and its expert alone (never on which rows share its tile), so it does not depend on
 // the batch.
 #include "common.h"
+#include "gate_act.h"
 
 constexpr int MOE_MAX_EXPERTS = 1024;
 constexpr int MOE_TILE_ROWS = 64;        // rows of a tile of the kernel for many rows; the kernel for few rows takes 16
@@ -35,13 +36,16 @@ constexpr int ROUTE_CHUNKS = 8;                  // rows of up to 8 * 512 elemen
 
 // bias: null or [experts], added to the logits.  mode 0: the weight of a chosen expert is sigmoid(z); 1: the softmax over
 // the chosen logits; 2: s = softmax(z) over all experts, the choice goes by s + bias (the bias is not added to the
-// logits), the weights are the chosen s divided by their sum + 1e-20.  extra: rows of `router` behind the experts' (at most MOE_MAX_EXTRA); gates [n, extra] takes sigmoid
+// logits), the weights are the chosen s divided by their sum + 1e-20 (renorm 0: as they are), times `scale`.  groups > 1 (mode 2):
+// the experts are so many groups of neighbours, a group counts as its best expert's s + bias, and only experts of the `keep` best
+// groups (ties: the lower index) can be chosen.  extra: rows of `router` behind the experts' (at most MOE_MAX_EXTRA); gates [n, extra] takes sigmoid
 // of their logits (they are no experts and are never chosen).
 constexpr int MOE_MAX_EXTRA = 8;
 template <class T, int THREADS>
 __global__ void __launch_bounds__(THREADS)
 moe_route_kernel(const T *__restrict__ h, const float *__restrict__ router, const float *__restrict__ bias, int *__restrict__ ids,
-                 float *__restrict__ wts, float *__restrict__ gates, int d, int n_experts, int top, int mode, int extra) {
+                 float *__restrict__ wts, float *__restrict__ gates, int d, int n_experts, int top, int mode, int extra, int groups, int keep,
+                 int renorm, float scale) {
     __shared__ float z[MOE_MAX_EXPERTS + MOE_MAX_EXTRA];
     __shared__ float zc[MOE_MAX_EXPERTS];
     __shared__ float sc[MOE_MAX_EXPERTS];
@@ -103,6 +107,23 @@ moe_route_kernel(const T *__restrict__ h, const float *__restrict__ router, cons
             }
         }
         __syncthreads();
+        if (groups > 1) {
+            // every group's best (in zc), then every group's place among them; the experts of a group behind the kept ones are out
+            const int per = n_experts / groups;
+            for (int g = threadIdx.x; g < groups; g += THREADS) {
+                float best = z[g * per];
+                for (int e = 1; e < per; ++e) best = fmaxf(best, z[g * per + e]);
+                zc[g] = best;
+            }
+            __syncthreads();
+            for (int g = threadIdx.x; g < groups; g += THREADS) {
+                int before = 0;
+                for (int o = 0; o < groups; ++o) before += zc[o] > zc[g] || (zc[o] == zc[g] && o < g);
+                if (before >= keep)
+                    for (int e = 0; e < per; ++e) z[g * per + e] = -INFINITY;
+            }
+            __syncthreads();
+        }
     }
     for (int k = 0; k < top; ++k) {                  // the first wave chooses; the others only keep the barriers
         if (wave == 0) {
@@ -131,8 +152,8 @@ moe_route_kernel(const T *__restrict__ h, const float *__restrict__ router, cons
     if (mode == 2 && wave == 0) {                    // the chosen scores, made to add up to one
         float part = 0.f;
         for (int k = lane; k < top; k += WAVE) part += zc[k];
-        const float sum = wave_sum(part) + 1e-20f;
-        for (int k = lane; k < top; k += WAVE) wts[(size_t)t * top + k] = zc[k] / sum;
+        const float sum = renorm ? wave_sum(part) + 1e-20f : 1.f;
+        for (int k = lane; k < top; k += WAVE) wts[(size_t)t * top + k] = zc[k] / sum * scale;
     }
     if (mode == 1 && wave == 0) {                    // the softmax over the chosen logits (the first is the largest)
         const float z0 = zc[0];
@@ -214,7 +235,6 @@ template <> struct Mma<float> {
 __device__ __forceinline__ float gelu_erf(float z) { return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f)); }
 
 enum { MOE_UP = 0, MOE_DOWN = 1, MOE_UP_GATED = 2 };
-__device__ __forceinline__ float silu_f(float z) { return z / (1.0f + expf(-z)); }
 
 // Both kernels below multiply the rows of a tile (sorted rows of one expert) with that expert's matrix
 // w[e] ([N, K], row-major) on the matrix cores.  The weight is the instruction's first operand (16
@@ -227,7 +247,7 @@ __device__ __forceinline__ float silu_f(float z) { return z / (1.0f + expf(-z));
 //             (add == 0: stored) or at the pair's token (add == 1: added; only with top == 1).
 //   MOE_UP_GATED: x = h [n, K], not scaled; w[e] holds N = 2 * features rows, in turns 16 rows of the gate matrix and the
 //             16 rows of the up matrix that meet them; out_t = act [total, N / 2] at the sorted row,
-//             silu(gate) * up.
+//             silu(gate) * up, or with limit > 0 the limited form with alpha and limit.
 template <class T, int MODE>
 __device__ __forceinline__ void moe_store(const f32x4 &acc, int dst, int col0, int N, T *__restrict__ out_t,
                                           float *__restrict__ out_f, int out_stride, int add) {
@@ -252,7 +272,7 @@ moe_gemm_few_kernel(const T *__restrict__ x, int x_stride, const T *__restrict__
                     const int *__restrict__ sorted_to_flat, const float *__restrict__ wts,
                     const int *__restrict__ tile_expert, const int *__restrict__ tile_begin,
                     const int *__restrict__ tile_rows, const int *__restrict__ n_tiles, int /* max_tiles */, T *__restrict__ out_t,
-                    float *__restrict__ out_f, int out_stride, int top, int add) {
+                    float *__restrict__ out_f, int out_stride, int top, int add, float alpha, float limit) {
     typedef Mma<T> M;
     typedef typename M::frag frag;
     const int tile = blockIdx.x;
@@ -304,7 +324,7 @@ moe_gemm_few_kernel(const T *__restrict__ x, int x_stride, const T *__restrict__
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
             const int col = f0 + 4 * g + i;
-            if (col < NF) out_t[(size_t)dst * out_stride + col] = from_f32<T>(silu_f(acc[i]) * acc2[i]);
+            if (col < NF) out_t[(size_t)dst * out_stride + col] = from_f32<T>(gate_up_of(acc[i], acc2[i], alpha, limit));
         }
     } else {
         moe_store<T, MODE>(acc, dst, f0 + 4 * g, N, out_t, out_f, out_stride, add);
@@ -320,7 +340,7 @@ moe_gemm_many_kernel(const T *__restrict__ x, int x_stride, const T *__restrict_
                      const int *__restrict__ sorted_to_flat, const float *__restrict__ wts,
                      const int *__restrict__ tile_expert, const int *__restrict__ tile_begin,
                      const int *__restrict__ tile_rows, const int *__restrict__ n_tiles, int max_tiles, T *__restrict__ out_t,
-                     float *__restrict__ out_f, int out_stride, int top, int add) {
+                     float *__restrict__ out_f, int out_stride, int top, int add, float alpha, float limit) {
     typedef Mma<T> M;
     typedef typename M::frag frag;
     constexpr int PL = M::PER_LANE;                 // elements in 16 bytes
@@ -417,7 +437,7 @@ moe_gemm_many_kernel(const T *__restrict__ x, int x_stride, const T *__restrict_
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 const int col = (n0 + 32 * wave) / 2 + 4 * g + i;
-                if (col < N / 2) out_t[(size_t)dst * out_stride + col] = from_f32<T>(silu_f(acc[0][m][i]) * acc[1][m][i]);
+                if (col < N / 2) out_t[(size_t)dst * out_stride + col] = from_f32<T>(gate_up_of(acc[0][m][i], acc[1][m][i], alpha, limit));
             }
             continue;
         }
@@ -456,13 +476,15 @@ LCU_API int lcu_moe_tile_rows(int total, int experts) { return (long long)total 
 // bias: null or [experts] 32-bit; mode 0: sigmoid weights, 1: softmax over the chosen; extra, gates: see the kernel
 // (router then has experts + extra rows).
 LCU_API int lcu_moe_route(const void *h, int type, const float *router, const float *bias, int *ids, float *wts, float *gates,
-                          int n, int d, int experts, int top, int mode, int extra, hipStream_t stream) {
+                          int n, int d, int experts, int top, int mode, int extra, int groups, int keep, int renorm, float scale,
+                          hipStream_t stream) {
     if (n <= 0) return LCU_OK;
     if (d <= 0 || experts <= 0 || experts > MOE_MAX_EXPERTS || top <= 0 || top > experts || mode < 0 || mode > 2 ||
-        extra < 0 || extra > MOE_MAX_EXTRA || (extra && !gates))
+        extra < 0 || extra > MOE_MAX_EXTRA || (extra && !gates) || groups < 1 ||
+        (groups > 1 && (mode != 2 || experts % groups || keep < 1 || keep > groups || top > keep * (experts / groups))))
         return LCU_BAD_ARGUMENT;
     const bool few = n <= 256 && experts > 4;
-#define GO(T, TH) moe_route_kernel<T, TH><<<dim3(n), dim3(TH), 0, stream>>>((const T *)h, router, bias, ids, wts, gates, d, experts, top, mode, extra)
+#define GO(T, TH) moe_route_kernel<T, TH><<<dim3(n), dim3(TH), 0, stream>>>((const T *)h, router, bias, ids, wts, gates, d, experts, top, mode, extra, groups, keep, renorm, scale)
     if (type == LCU_F32) { if (few) GO(float, 1024); else GO(float, 256); }
     else if (type == LCU_BF16) { if (few) GO(bf16_t, 1024); else GO(bf16_t, 256); }
     else return LCU_BAD_ARGUMENT;
@@ -477,13 +499,13 @@ LCU_API int lcu_moe_route(const void *h, int type, const float *router, const fl
 // [total, d] 32-bit (only read and written when top > 1 or gated).  out: [n, d] 32-bit, added to.
 // gated: w_up is [experts, 2 * ff, d], in turns 16 rows of the gate matrix and the 16 rows of the up matrix that meet
 // them (ff a multiple of 16); act = silu(gate h) * (up h), and the weight scales what comes out; fresh: out is written
-// and not added to.  identity: ids may name experts + identity experts; the last `identity` have no matrices and return the
+// and not added to; limit > 0: the limited activation (gate_act.h) with alpha and limit instead of silu.  identity: ids may name experts + identity experts; the last `identity` have no matrices and return the
 // token's input.  shared (null or
 // [n, d] of `type`) with shared_gate (null or [n] 32-bit): rows that are added beside the experts', times the gate.
 LCU_API int lcu_moe_experts(const void *h, int type, const int *ids, const float *wts, int *ints, int max_tiles,
                             const void *w_up, const void *w_down, void *act, float *y, float *out, int n, int d, int ff,
                             int experts, int top, int gated, const void *shared, const float *shared_gate, int fresh,
-                            int identity, hipStream_t stream) {
+                            int identity, float alpha, float limit, hipStream_t stream) {
     if (n <= 0) return LCU_OK;
     const int per = type == LCU_BF16 ? 8 : 4;
     if (d <= 0 || ff <= 0 || d % per || ff % per || experts <= 0 || experts > MOE_MAX_EXPERTS || top <= 0 || max_tiles <= 0 ||
@@ -508,12 +530,12 @@ LCU_API int lcu_moe_experts(const void *h, int type, const int *ids, const float
 #define GO(KERNEL, T)                                                                                                              \
     if (gated)                                                                                                                     \
         KERNEL<T, MOE_UP_GATED><<<gu, block, 0, stream>>>((const T *)h, d, (const T *)w_up, (size_t)up_rows * d, up_rows, d, sorted, wts, \
-                                                      t_exp, t_beg, t_rows, n_tiles, max_tiles, (T *)act, nullptr, ff, top, 0);       \
+                                                      t_exp, t_beg, t_rows, n_tiles, max_tiles, (T *)act, nullptr, ff, top, 0, alpha, limit);       \
     else                                                                                                                           \
         KERNEL<T, MOE_UP><<<gu, block, 0, stream>>>((const T *)h, d, (const T *)w_up, (size_t)ff * d, ff, d, sorted, wts, t_exp, t_beg, \
-                                                t_rows, n_tiles, max_tiles, (T *)act, nullptr, ff, top, 0);                         \
+                                                t_rows, n_tiles, max_tiles, (T *)act, nullptr, ff, top, 0, 0.f, 0.f);                         \
     KERNEL<T, MOE_DOWN><<<gd, block, 0, stream>>>((const T *)act, ff, (const T *)w_down, (size_t)ff * d, d, ff, sorted, wts, t_exp, \
-                                                  t_beg, t_rows, n_tiles, max_tiles, nullptr, down_to, d, top, add)
+                                                  t_beg, t_rows, n_tiles, max_tiles, nullptr, down_to, d, top, add, 0.f, 0.f)
     if (type == LCU_BF16) {
         if (tile_rows == 16) { GO(moe_gemm_few_kernel, bf16_t); } else { GO(moe_gemm_many_kernel, bf16_t); }
     } else {

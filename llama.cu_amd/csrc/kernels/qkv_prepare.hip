@@ -3,6 +3,7 @@
 //
 //   q, k, v <- product + bias                                           (bias: one vector over the row's columns)
 //   q, k    <- x * rsqrt(mean over the head's dims of x^2 + eps) * w     (w [dh], shared by all heads; one for q, one for k)
+//              or x * rsqrt(mean over all heads' dims of x^2 + eps) * w   (w [heads * dh]; a kernel of its own)
 //   q, k    <- the first rot_dim dims of every head turned by the angle of the token's position (tables
 //              [max_pos, rot_dim / 2]; pairing 0: (i, i + rot_dim/2), 1: (2i, 2i + 1)); the other dims pass
 //   q -> q_out [n, nh * dhp]; k, v -> the token's place in its page
@@ -252,24 +253,143 @@ LCU_API int lcu_qkv_prepare(const void *rows, int in_type, int n, int row_stride
     return LCU_OK;
 }
 
-// The output of every head times sigmoid of the head's gate: out[t, h, :] *= sigmoid(gate[t, h]), the gate's rows
-// [n, gate_stride] with the heads' numbers from column g_off.  The factor is 32-bit.
-template <class TG, class T>
-__global__ void head_gate_kernel(T *__restrict__ out, const TG *__restrict__ gate, int gate_stride, int g_off, int nh, int dv) {
-    const int t = blockIdx.x;
-    for (int c = threadIdx.x; c < nh * dv; c += blockDim.x) {
-        const float g = to_f32(gate[(size_t)t * gate_stride + g_off + c / dv]);
-        T *o = out + (size_t)t * nh * dv + c;
-        *o = from_f32<T>(to_f32(*o) / (1.0f + expf(-g)));
+// A norm over the whole projection of the queries, and one over that of the keys, needs a token's whole row: a workgroup per token.
+// The row is read twice, the second time from the caches.  V dims a piece (1: any sizes, either pairing).
+template <class TI, class T, int V>
+__global__ void __launch_bounds__(512)
+qkv_prepare_rows_kernel(const TI *__restrict__ rows, int row_stride, int q_off, int k_off, int v_off, const float *__restrict__ q_norm,
+                        const float *__restrict__ k_norm, float eps, const int *__restrict__ positions, const float *__restrict__ cos_t,
+                        const float *__restrict__ sin_t, int max_pos, int rot_dim, int pairing, T *__restrict__ q_out,
+                        const int *__restrict__ slots, T *__restrict__ cache, int nh, int nkvh, int dh, int dhp, int dv, int dvp, int page,
+                        int store_kv) {
+    struct alignas(V * sizeof(TI)) In { TI v[V]; };
+    struct alignas(V * sizeof(T)) Out { T v[V]; };
+    struct alignas(V * sizeof(float)) F32 { float v[V]; };
+    __shared__ float scratch[16], scratch_k[16];
+    const int t = blockIdx.x, threads = blockDim.x, nq = nh * dh, nk = store_kv ? nkvh * dh : 0;
+    const TI *row = rows + (size_t)t * row_stride;
+    float sq = 0.f, sk = 0.f;
+    for (int c = threadIdx.x * V; c < nq + nk; c += threads * V) {
+        const In a = *(const In *)(row + (c < nq ? q_off + c : k_off + c - nq));
+        float part = 0.f;
+#pragma unroll
+        for (int e = 0; e < V; ++e) part += to_f32(a.v[e]) * to_f32(a.v[e]);
+        if (c < nq) sq += part;
+        else sk += part;
+    }
+    const float fq = rsqrtf(block_sum(sq, scratch) / (float)nq + eps);
+    const float fk = nk ? rsqrtf(block_sum(sk, scratch_k) / (float)nk + eps) : 0.f;
+    const int slot = store_kv ? slots[t] : -1, tok = slot < 0 ? 0 : slot % page;
+    T *pg = slot < 0 ? nullptr : cache + (size_t)(slot / page) * kv_page_elems(nkvh, dhp, dvp, page);
+    const int pos = cos_t ? positions[t] : 0, half = rot_dim / 2;
+    const bool in_table = pos >= 0 && pos < max_pos;
+    // the pieces of a stored head: its turned pairs, its other dims, its zeros; of a value head: its dims with zeros behind them
+    const int turned = half / V, passed = (dh - rot_dim) / V, items = turned + passed + (dhp - dh) / V;
+    const int n_q = nh * items, n_k = slot < 0 ? 0 : nkvh * items, n_v = slot < 0 ? 0 : nkvh * ((dvp + V - 1) / V);
+    for (int i = threadIdx.x; i < n_q + n_k + n_v; i += threads) {
+        if (i >= n_q + n_k) {
+            const int per = (dvp + V - 1) / V, kvh = (i - n_q - n_k) / per, c = (i - n_q - n_k) % per * V;
+            In a = {};
+            if (c < dv) a = *(const In *)(row + v_off + kvh * dv + c);
+#pragma unroll
+            for (int e = 0; e < V; ++e) pg[kv_value_offset(nkvh, kvh, tok, c + e, dhp, dvp, page)] = from_f32<T>(to_f32(a.v[e]));
+            continue;
+        }
+        const bool is_key = i >= n_q;
+        const int head = (is_key ? i - n_q : i) / items, item = (is_key ? i - n_q : i) % items;
+        const TI *x = row + (is_key ? k_off : q_off) + head * dh;
+        const float *w = (is_key ? k_norm : q_norm) + head * dh;
+        const float f = is_key ? fk : fq;
+        auto at_dim = [&](int c) -> Out * { return (Out *)(is_key ? pg + kv_key_offset(head, tok, c, dhp, page) : q_out + (size_t)t * nh * dhp + (size_t)head * dhp + c); };
+        auto normed = [&](int c, float *o) {
+            const In a = *(const In *)(x + c);
+            const F32 wv = *(const F32 *)(w + c);
+#pragma unroll
+            for (int e = 0; e < V; ++e) o[e] = to_f32(a.v[e]) * f * wv.v[e];
+        };
+        float a[V], b[V];
+        Out oa, ob;
+        if (item < turned) {
+            const int i0 = item * V, ca = pairing == 0 ? i0 : 2 * i0, cb = pairing == 0 ? half + i0 : 2 * i0 + 1;      // (neighbours: V is 1)
+            normed(ca, a);
+            normed(cb, b);
+            const size_t tab = (size_t)(in_table ? pos : 0) * half + i0;
+            const F32 cs = *(const F32 *)(cos_t + tab), sn = *(const F32 *)(sin_t + tab);
+#pragma unroll
+            for (int e = 0; e < V; ++e) {
+                float ra, rb;
+                rotate_pair(a[e], b[e], cs.v[e], sn.v[e], ra, rb);
+                if (!in_table) ra = rb = __uint_as_float(0x7fc00000u);        // a position outside the table gives NaN, not a wrong value
+                oa.v[e] = from_f32<T>(ra);
+                ob.v[e] = from_f32<T>(rb);
+            }
+            *at_dim(ca) = oa;
+            *at_dim(cb) = ob;
+        } else {
+            const int c = rot_dim + (item - turned) * V;
+            if (c < dh) normed(c, a);
+#pragma unroll
+            for (int e = 0; e < V; ++e) oa.v[e] = from_f32<T>(c < dh ? a[e] : 0.f);
+            *at_dim(c) = oa;
+        }
     }
 }
 
-LCU_API int lcu_head_gate(void *out, int type, const void *gate, int gate_type, int gate_stride, int g_off, int n, int nh,
-                          int dv, hipStream_t stream) {
+// rows, q_out, cache and the rest as lcu_qkv_prepare (no bias, no maps); q_norm [nh * dh], k_norm [nkvh * dh].
+LCU_API int lcu_qkv_prepare_rows(const void *rows, int in_type, int n, int row_stride, int q_off, int k_off, int v_off, const float *q_norm,
+                                 const float *k_norm, float eps, const int *positions, const float *cos_t, const float *sin_t, int max_pos,
+                                 int rot_dim, int pairing, void *q_out, int type, const int *slots, void *cache, int nh, int nkvh, int dh,
+                                 int dhp, int dv, int dvp, int page, int store_kv, hipStream_t stream) {
     if (n <= 0) return LCU_OK;
-    if (nh <= 0 || dv <= 0 || !out || !gate) return LCU_BAD_ARGUMENT;
+    if (nh <= 0 || nkvh <= 0 || dh <= 0 || dhp < dh || dhp % 8 || dhp > QP_MAX_DIM || dv <= 0 || dvp < dv || dvp > QP_MAX_DIM || page <= 0 ||
+        page % 8 || rot_dim < 0 || rot_dim % 2 || rot_dim > dh || (pairing != 0 && pairing != 1) || !rows || !q_out || !q_norm || !k_norm ||
+        (cos_t && (!sin_t || !positions || rot_dim == 0)) || (store_kv && (!cache || !slots)))
+        return LCU_BAD_ARGUMENT;
+    const int rot = cos_t ? rot_dim : 0;
+    const bool four = (pairing == 0 || !rot) && dh % 4 == 0 && rot % 8 == 0 && dv % 4 == 0 && dvp % 4 == 0 && row_stride % 4 == 0 && q_off % 4 == 0 &&
+                      k_off % 4 == 0 && v_off % 4 == 0 && (uintptr_t)rows % 16 == 0 && (uintptr_t)q_out % 16 == 0 && (uintptr_t)cache % 16 == 0 &&
+                      (uintptr_t)cos_t % 16 == 0 && (uintptr_t)sin_t % 16 == 0 && (uintptr_t)q_norm % 16 == 0 && (uintptr_t)k_norm % 16 == 0;
+    dim3 grid(n), block(n <= 192 ? 512 : 256);
+#define GO(TI, T, V) qkv_prepare_rows_kernel<TI, T, V><<<grid, block, 0, stream>>>((const TI *)rows, row_stride, q_off, k_off, v_off, q_norm, k_norm, eps, positions, cos_t, sin_t, max_pos, rot, pairing, (T *)q_out, slots, (T *)cache, nh, nkvh, dh, dhp, dv, dvp, page, store_kv)
+#define EITHER(TI, T) do { if (four) GO(TI, T, 4); else GO(TI, T, 1); } while (0)
+    if (in_type == LCU_F32 && type == LCU_F32) EITHER(float, float);
+    else if (in_type == LCU_F32 && type == LCU_BF16) EITHER(float, bf16_t);
+    else if (in_type == LCU_BF16 && type == LCU_BF16) EITHER(bf16_t, bf16_t);
+    else return LCU_BAD_ARGUMENT;
+#undef EITHER
+#undef GO
+    LCU_LAUNCH_CHECK();
+    return LCU_OK;
+}
+
+// The output of every head times sigmoid of the head's gate: out[t, h, :] = factor * sigmoid(gate[t, h]) * x[t, h, :], the gate's rows
+// [n, gate_stride] with the heads' numbers from column g_off, out's rows out_stride apart (out may be x).  The factor is 32-bit.
+template <class TG, class T, int V>
+__global__ void __launch_bounds__(256)
+head_gate_kernel(T *out, int out_stride, const T *x, const TG *__restrict__ gate, int gate_stride, int g_off, int nh, int dv, float factor) {
+    struct alignas(V * sizeof(T)) Piece { T v[V]; };
+    const int t = blockIdx.x;
+    for (int c = threadIdx.x * V; c < nh * dv; c += blockDim.x * V) {
+        const float g = to_f32(gate[(size_t)t * gate_stride + g_off + c / dv]);
+        const float f = factor / (1.0f + expf(-g));
+        Piece p = *(const Piece *)(x + (size_t)t * nh * dv + c);
+#pragma unroll
+        for (int e = 0; e < V; ++e) p.v[e] = from_f32<T>(to_f32(p.v[e]) * f);
+        *(Piece *)(out + (size_t)t * out_stride + c) = p;
+    }
+}
+
+LCU_API int lcu_head_gate(void *out, int out_stride, const void *x, int type, const void *gate, int gate_type, int gate_stride, int g_off, int n,
+                          int nh, int dv, float factor, hipStream_t stream) {
+    if (n <= 0) return LCU_OK;
+    if (nh <= 0 || dv <= 0 || !out || !x || !gate || out_stride < nh * dv) return LCU_BAD_ARGUMENT;
     dim3 grid(n), block(256);
-#define GO(TG, T) head_gate_kernel<TG, T><<<grid, block, 0, stream>>>((T *)out, (const TG *)gate, gate_stride, g_off, nh, dv)
+    const bool four = dv % 4 == 0 && out_stride % 4 == 0 && (uintptr_t)out % 16 == 0 && (uintptr_t)x % 16 == 0;
+#define GO(TG, T)                                                                                                                                      \
+    do {                                                                                                                                               \
+        if (four) head_gate_kernel<TG, T, 4><<<grid, block, 0, stream>>>((T *)out, out_stride, (const T *)x, (const TG *)gate, gate_stride, g_off, nh, dv, factor); \
+        else head_gate_kernel<TG, T, 1><<<grid, block, 0, stream>>>((T *)out, out_stride, (const T *)x, (const TG *)gate, gate_stride, g_off, nh, dv, factor);     \
+    } while (0)
     if (gate_type == LCU_F32 && type == LCU_F32) GO(float, float);
     else if (gate_type == LCU_F32 && type == LCU_BF16) GO(float, bf16_t);
     else if (gate_type == LCU_BF16 && type == LCU_BF16) GO(bf16_t, bf16_t);

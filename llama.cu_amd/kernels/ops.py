@@ -132,17 +132,19 @@ def _check(rc: int, name: str) -> None:
 # ------------------------------------------------------------------ elementwise
 
 
-def embedding_gather(table: torch.Tensor, ids: torch.Tensor, out: torch.Tensor, scale: float = 1.0) -> torch.Tensor:
-    """``out[i, :] = table[ids[i], :] * scale`` (the product in 32-bit, converted to ``out``'s type)."""
+def embedding_gather(table: torch.Tensor, ids: torch.Tensor, out: torch.Tensor, scale: float = 1.0,
+                     copies: int = 1) -> torch.Tensor:
+    """``out[i, :] = table[ids[i], :] * scale`` (the product in 32-bit, converted to ``out``'s type); ``copies``: each row of
+    ``out`` holds so many of them side by side."""
     _gpu(table, ids, out)
     _rows(table, "embedding table"); _contig(table, "embedding table"); _contig(out, "embedding out")
     n = ids.numel()
     _i32(ids, "token ids")
-    if out.shape != (n, table.shape[1]):
-        raise KernelError(f"embedding out: shape {tuple(out.shape)}, expected {(n, table.shape[1])}")
+    if copies < 1 or out.shape != (n, copies * table.shape[1]):
+        raise KernelError(f"embedding out: shape {tuple(out.shape)}, expected {(n, copies * table.shape[1])}")
     lib = build.load("elementwise")
     _check(lib.lcu_embedding_gather(_ptr(out), _type(out, "embedding out"), _ptr(table), _type(table, "embedding table"),
-                                    _ptr(ids), n, table.shape[1], table.shape[0], ctypes.c_float(scale), _stream()), "embedding_gather")
+                                    _ptr(ids), n, table.shape[1], table.shape[0], ctypes.c_float(scale), int(copies), _stream()), "embedding_gather")
     return out
 
 
@@ -1286,12 +1288,13 @@ def delta_rule(proj: torch.Tensor, offsets: Dict[str, int], w2_t: torch.Tensor, 
 
 
 def moe_route(h: torch.Tensor, router: torch.Tensor, top: int, bias: Optional[torch.Tensor] = None, softmax_chosen: bool = False,
-              extra: int = 0, softmax_all: bool = False):
+              extra: int = 0, softmax_all: bool = False, groups: int = 1, keep: int = 1, renorm: bool = True, scale: float = 1.0):
     """``(ids, weights)``, each ``[n, top]``: every row's ``top`` experts by ``router @ h + bias`` (32-bit; ties go to the
     lower index), largest first, with the weight ``sigmoid`` of that logit or, with ``softmax_chosen``, the softmax over
     the chosen logits alone; with ``softmax_all`` the scores are ``s = softmax(router @ h)`` over all experts, the choice goes
     by ``s + bias`` (the bias is a correction of the choice and not of the logits) and the weights are the chosen ``s``
-    divided by their sum + 1e-20.  ``extra``: the last ``extra`` rows of ``router`` are no experts but gates; then a third
+    divided by their sum + 1e-20 (``renorm=False``: as they are), times ``scale``; of ``groups`` > 1 equal groups of neighbouring
+    experts only those of the ``keep`` with the largest best ``s + bias`` can be chosen.  ``extra``: the last ``extra`` rows of ``router`` are no experts but gates; then a third
     result ``[n, extra]`` holds ``sigmoid`` of their logits."""
     _gpu(h, router, bias)
     _rows(h, "moe input"); _contig(h, "moe input"); _contig(router, "router")
@@ -1304,25 +1307,32 @@ def moe_route(h: torch.Tensor, router: torch.Tensor, top: int, bias: Optional[to
     _f32_vec(bias, "router bias", experts)
     if softmax_all and softmax_chosen:
         raise KernelError("moe_route: the softmax runs over all experts or over the chosen ones, not both")
+    if (groups != 1 or not renorm or scale != 1.0) and not softmax_all:
+        raise KernelError("moe_route: groups, a factor and weights as they are go with scores over all experts")
+    if groups < 1 or experts % groups or not 1 <= keep <= groups or top > keep * (experts // groups):
+        raise KernelError(f"moe_route: top {top} of the experts of {keep} of {groups} groups of {experts} experts is not supported")
     ids = torch.empty((n, top), dtype=torch.int32, device=h.device)
     wts = torch.empty((n, top), dtype=torch.float32, device=h.device)
     gates = torch.empty((n, extra), dtype=torch.float32, device=h.device) if extra else None
     lib = build.load("moe")
     _check(lib.lcu_moe_route(_ptr(h), _type(h, "moe input"), _ptr(router), _ptr(bias), _ptr(ids), _ptr(wts), _ptr(gates), n, d,
-                             experts, top, 2 if softmax_all else int(bool(softmax_chosen)), int(extra), _stream()), "moe_route")
+                             experts, top, 2 if softmax_all else int(bool(softmax_chosen)), int(extra), int(groups), int(keep), int(bool(renorm)),
+                             ctypes.c_float(scale), _stream()), "moe_route")
     return (ids, wts, gates) if extra else (ids, wts)
 
 
 def moe_experts(h: torch.Tensor, ids: torch.Tensor, wts: torch.Tensor, w_up: torch.Tensor, w_down: torch.Tensor,
                 out: torch.Tensor, gated: bool = False, shared: Optional[torch.Tensor] = None,
-                shared_gate: Optional[torch.Tensor] = None, fresh: bool = False, identity: int = 0) -> torch.Tensor:
+                shared_gate: Optional[torch.Tensor] = None, fresh: bool = False, identity: int = 0,
+                act_alpha: float = 1.0, act_limit: float = 0.0) -> torch.Tensor:
     """``out[t] += sum over t's experts e of  w_down[e] @ gelu(w_up[e] @ (weight * h[t]))`` (the exact gelu; the
     weight scales what goes INTO the expert, not what comes out).  ``w_up [experts, ff, d]``, ``w_down [experts, d, ff]`` in ``h``'s type,
     ``out`` float32 ``[n, d]``.  ``gated``: ``out[t] += sum_e weight * w_down[e] @ (silu(gate[e] @ h[t]) * (up[e] @ h[t]))``
     with ``w_up [experts, 2 * ff, d]`` holding in turns 16 rows of the gate matrix and the 16 up rows that meet them
     (``gated_rows`` lays them out so); ``shared [n, d]`` (with ``shared_gate [n]`` float32, or ones) is added beside;
     ``fresh``: ``out`` is written, not added to (it need not hold anything).  ``identity``: ``ids`` may name ``experts +
-    identity`` experts, of which the last ``identity`` have no matrices: their output is ``weight * h[t]`` (gated form only)."""
+    identity`` experts, of which the last ``identity`` have no matrices: their output is ``weight * h[t]`` (gated form only).
+    ``act_limit`` > 0: the limited activation (``swiglu``) with ``act_alpha`` instead of silu."""
     _gpu(h, ids, wts, w_up, w_down, out, shared, shared_gate)
     _rows(h, "moe input")
     for t, what in ((h, "moe input"), (ids, "moe ids"), (wts, "moe weights"), (w_up, "moe up"), (w_down, "moe down"), (out, "moe out")):
@@ -1342,6 +1352,8 @@ def moe_experts(h: torch.Tensor, ids: torch.Tensor, wts: torch.Tensor, w_up: tor
         raise KernelError(f"moe_experts: the width {d} and the experts' {ff} must be multiples of {per} ({16 if gated else per} for the experts')")
     if fresh and not gated:
         raise KernelError("moe_experts: only the gated form writes its output afresh")
+    if act_limit and not (gated and act_limit > 0):
+        raise KernelError("moe_experts: the limited activation goes with gated experts and needs a positive limit")
     identity = int(identity)
     if identity < 0 or (identity and not gated) or experts + identity > 1024:
         raise KernelError("moe_experts: identity experts go with gated experts, and all together are at most 1024")
@@ -1360,8 +1372,8 @@ def moe_experts(h: torch.Tensor, ids: torch.Tensor, wts: torch.Tensor, w_up: tor
     y = torch.empty((total, d), dtype=torch.float32, device=h.device) if (top > 1 or gated) else None
     _check(lib.lcu_moe_experts(_ptr(h), _type(h, "moe input"), _ptr(ids), _ptr(wts), _ptr(ints), max_tiles, _ptr(w_up),
                                _ptr(w_down), _ptr(act), _ptr(y), _ptr(out), n, d, ff, experts, top, int(bool(gated)),
-                               _ptr(shared), _ptr(shared_gate if shared is not None else None), int(bool(fresh)), identity, _stream()),
-           "moe_experts")
+                               _ptr(shared), _ptr(shared_gate if shared is not None else None), int(bool(fresh)), identity, ctypes.c_float(act_alpha),
+                               ctypes.c_float(act_limit), _stream()), "moe_experts")
     return out
 
 
@@ -1492,16 +1504,59 @@ def qkv_prepare(rows: torch.Tensor, offsets, n_heads: int, n_kv_heads: int, head
     return q
 
 
-def head_gate(out: torch.Tensor, gate_rows: torch.Tensor, g_off: int, n_heads: int, value_dim: int) -> torch.Tensor:
-    """``out[t, h, :] *= sigmoid(gate_rows[t, g_off + h])`` for ``out [n, n_heads * value_dim]``, in place."""
-    _gpu(out, gate_rows)
-    _rows(out, "attention out"); _contig(out, "attention out"); _rows(gate_rows, "gate rows")
-    n = out.shape[0]
-    if out.shape[1] != n_heads * value_dim or gate_rows.shape[0] != n or g_off < 0 or g_off + n_heads > gate_rows.shape[1]:
+def qkv_prepare_rows(rows: torch.Tensor, offsets, n_heads: int, n_kv_heads: int, head_dim: int, value_dim: int, stored_dim: int,
+                     stored_value_dim: int, dtype: torch.dtype, q_norm: torch.Tensor, k_norm: torch.Tensor, eps: float,
+                     positions: Optional[torch.Tensor] = None, cos: Optional[torch.Tensor] = None, sin: Optional[torch.Tensor] = None,
+                     rot_dim: int = 0, pairing: int = 0, cache: Optional[torch.Tensor] = None, slots: Optional[torch.Tensor] = None,
+                     page_size: int = 16) -> torch.Tensor:
+    """``qkv_prepare`` with a norm over the whole projection: all of a token's queries are divided by their one root mean square and
+    multiplied by ``q_norm`` (float32 ``[n_heads * head_dim]``), all of its keys likewise (``k_norm``), before the rotation."""
+    _gpu(rows, positions, q_norm, k_norm, cos, sin, cache, slots)
+    _rows(rows, "qkv rows")
+    n, width = rows.shape
+    store = cache is not None
+    q_off, k_off, v_off = (int(o) for o in offsets)
+    if q_off < 0 or q_off + n_heads * head_dim > width or (store and (k_off < 0 or k_off + n_kv_heads * head_dim > width
+                                                                      or v_off < 0 or v_off + n_kv_heads * value_dim > width)):
+        raise KernelError(f"qkv_prepare_rows: the columns of q, k or v lie outside the rows' {width} columns")
+    if stored_dim % 8 or stored_dim < head_dim or stored_value_dim < value_dim or max(stored_dim, stored_value_dim) > QKV_PREPARE_MAX_DIM:
+        raise KernelError(f"qkv_prepare_rows: stored head sizes {stored_dim} / {stored_value_dim} do not fit {head_dim} / {value_dim} (keys a multiple of 8, at most {QKV_PREPARE_MAX_DIM})")
+    _f32_vec(q_norm, "query norm weight", n_heads * head_dim); _f32_vec(k_norm, "key norm weight", n_kv_heads * head_dim)
+    max_pos = 0
+    if cos is not None:
+        if sin is None or cos.shape != sin.shape or cos.dtype != torch.float32 or sin.dtype != torch.float32 or positions is None \
+                or cos.dim() != 2 or cos.shape[1] * 2 != rot_dim or not cos.is_contiguous() or not sin.is_contiguous():
+            raise KernelError("rotation tables must be two contiguous float32 tensors [max_pos, rot_dim/2], with the positions")
+        _i32(positions, "positions", n)
+        max_pos = cos.shape[0]
+    if store:
+        _i32(slots, "cache slots", n)
+        _contig(cache, "cache")
+        if cache.dtype != dtype or cache.dim() != 3 or cache.shape[1] * cache.shape[2] != n_kv_heads * (stored_dim + stored_value_dim) * page_size:
+            raise KernelError(f"cache: {cache.dtype} {tuple(cache.shape)} does not hold pages of {n_kv_heads} x ({stored_dim} + {stored_value_dim}) x {page_size} {dtype}")
+    q = torch.empty((n, n_heads * stored_dim), dtype=dtype, device=rows.device)
+    lib = build.load("qkv_prepare")
+    _check(lib.lcu_qkv_prepare_rows(_ptr(rows), _type(rows, "qkv rows"), n, rows.stride(0), q_off, k_off, v_off, _ptr(q_norm), _ptr(k_norm),
+                                    ctypes.c_float(eps), _ptr(positions), _ptr(cos), _ptr(sin), max_pos, int(rot_dim), int(pairing), _ptr(q),
+                                    _type(q, "q"), _ptr(slots), _ptr(cache), n_heads, n_kv_heads, head_dim, stored_dim, value_dim,
+                                    stored_value_dim, page_size, int(store), _stream()), "qkv_prepare_rows")
+    return q
+
+
+def head_gate(x: torch.Tensor, gate_rows: torch.Tensor, g_off: int, n_heads: int, value_dim: int, out: Optional[torch.Tensor] = None,
+              factor: float = 1.0) -> torch.Tensor:
+    """``out[t, h, :] = factor * sigmoid(gate_rows[t, g_off + h]) * x[t, h, :]`` for ``x [n, n_heads * value_dim]``; ``out`` (None: in
+    place) may be columns of a wider row."""
+    out = x if out is None else out
+    _gpu(out, x, gate_rows)
+    _rows(x, "attention out"); _contig(x, "attention out"); _rows(out, "gated rows"); _rows(gate_rows, "gate rows")
+    n = x.shape[0]
+    if x.shape[1] != n_heads * value_dim or out.shape != x.shape or out.dtype != x.dtype or gate_rows.shape[0] != n or g_off < 0 \
+            or g_off + n_heads > gate_rows.shape[1]:
         raise KernelError("head_gate: the output or the gates' columns do not fit")
     lib = build.load("qkv_prepare")
-    _check(lib.lcu_head_gate(_ptr(out), _type(out, "attention out"), _ptr(gate_rows), _type(gate_rows, "gate rows"),
-                             gate_rows.stride(0), int(g_off), n, n_heads, value_dim, _stream()), "head_gate")
+    _check(lib.lcu_head_gate(_ptr(out), out.stride(0), _ptr(x), _type(x, "attention out"), _ptr(gate_rows), _type(gate_rows, "gate rows"),
+                             gate_rows.stride(0), int(g_off), n, n_heads, value_dim, ctypes.c_float(factor), _stream()), "head_gate")
     return out
 
 
@@ -1926,3 +1981,124 @@ def gated_delta_rule(qkv: torch.Tensor, rows: torch.Tensor, off_a: int, off_b: i
                                     _type(out, "gated delta out"), _ptr(step.q_start), _ptr(step.ctx_len), _ptr(step.state_slot), n,
                                     step.n_req, heads, qk_heads, key_dim, value_dim, ctypes.c_float(eps), _stream()), "gated_delta_rule")
     return out
+
+
+# ------------------------------------------------------------------ several residual streams
+
+
+STREAMS_MAX = 8
+
+
+def streams_norm(x: torch.Tensor, streams: int, weight: torch.Tensor, eps: float, out_dtype: torch.dtype, delta: Optional[torch.Tensor] = None,
+                 mix: Optional[torch.Tensor] = None, out_weights: Optional[torch.Tensor] = None, read: Optional[torch.Tensor] = None,
+                 write_back: bool = True) -> torch.Tensor:
+    """``x [n, streams * d]`` float32: the streams of every row side by side.  With ``delta`` (a sublayer's output ``[n, d]``, or
+    float32 planes ``[planes, n, d]``) they become ``x_t = sum_s mix[s, t] x_s + out_weights[t] delta``, all at once, in place
+    (``write_back``); returns the rows ``u * rsqrt(mean(u^2) + eps) * weight`` of ``u = sum_s read[s] x_s`` (``read`` None: ones) in
+    ``out_dtype``.  The vectors are float32."""
+    _gpu(x, weight, delta, mix, out_weights, read)
+    _rows(x, "streams"); _contig(x, "streams")
+    if not 1 <= streams <= STREAMS_MAX or x.dtype != torch.float32 or x.shape[1] % streams:
+        raise KernelError(f"streams_norm: {streams} streams in rows of {x.shape[1]} {x.dtype} are not supported (1 to {STREAMS_MAX}, float32)")
+    n, d = x.shape[0], x.shape[1] // streams
+    _f32_vec(weight, "norm weight", d); _f32_vec(read, "reading weights", streams); _f32_vec(out_weights, "writing weights", streams)
+    planes, dt = 1, F32
+    if delta is not None:
+        _contig(delta, "streams delta")
+        if delta.dim() == 3:
+            planes = delta.shape[0]
+            if delta.dtype != torch.float32:
+                raise KernelError("streams_norm: planes of partial sums are float32")
+        if delta.shape[-2:] != (n, d) or mix is None or out_weights is None:
+            raise KernelError(f"streams_norm: an output {tuple(delta.shape)} needs the shape {(n, d)} and the matrix and weights that it enters by")
+        if mix.dtype != torch.float32 or mix.shape != (streams, streams) or not mix.is_contiguous():
+            raise KernelError(f"streams_norm: the matrix between the streams must be contiguous float32 [{streams}, {streams}]")
+        dt = _type(delta, "streams delta")
+    out = torch.empty((n, d), dtype=out_dtype, device=x.device)
+    lib = build.load("streams")
+    _check(lib.lcu_streams_norm(_ptr(x), int(streams), _ptr(delta), dt, planes, _ptr(mix), _ptr(out_weights), _ptr(read), _ptr(weight), _ptr(out),
+                                _type(out, "norm out"), n, d, ctypes.c_float(eps), int(bool(write_back)), _stream()), "streams_norm")
+    return out
+
+
+# ------------------------------------------------------------------ linear attention with a decay per head and token
+
+
+def decay_scan(rows: torch.Tensor, offsets: Dict[str, int], state: torch.Tensor, step, heads: int, key_dim: int, value_dim: int,
+               weight: torch.Tensor, eps: float, out: torch.Tensor, scale: float = 1.0, silu: bool = False, factor: float = 1.0,
+               decay: Optional[torch.Tensor] = None, log_decay: Optional[torch.Tensor] = None, gates: Optional[torch.Tensor] = None,
+               gate_bias=None, cap: float = 0.0, scaled_rows: bool = False) -> Optional[torch.Tensor]:
+    """``S <- a S + b k v^T``, ``o = scale * S^T q`` per head over the step's rows, request by request from each request's state.
+    ``rows [n, *]`` holds q, k (``heads * key_dim``), v and the output's gate g (``heads * value_dim``) at the columns ``offsets``;
+    ``silu``: q, k and v pass through silu.  ``state [slots, floats]`` float32 (``decay_state_floats``; views of a wider state will
+    do), taken as zero at a request's position 0.
+
+    ``decay`` (float32 ``[heads]``, with its logarithm in two parts, ``log_decay [heads, 2]``): ``a = decay``, ``b = 1``, and the heads'
+    outputs side by side, divided by their root mean square, times ``weight``, times ``sigmoid(g)`` go to ``out``.  Else ``gates [n, 2
+    heads]`` (float32: the input gates' projections, then the forget gates') with ``gate_bias`` (two float32 ``[heads]``) and
+    ``cap``: ``i = cap tanh(. / cap)``, ``f = log sigmoid(cap tanh(. / cap))``, a running maximum ``m = max(f + m, i)``, ``a = exp(f +
+    m' - m)``, ``b = exp(i - m)``, a normaliser ``n`` that sums ``k`` as ``S`` does, and each head's ``o / (max(|scale n . q|, exp(-m)) +
+    1e-6)`` divided by its root mean square, times ``weight``, times ``sigmoid(g)``.
+
+    ``out [n, heads * value_dim]`` of the rows' type may be columns of a wider row and takes the result times ``factor``.  ``rows`` may
+    be float32 beside a bfloat16 ``out`` in a step of single tokens.  ``scaled_rows`` (``decay``, a step of single tokens): the norm over all heads is
+    left to whoever multiplies the rows; returns the heads' shares ``[n, heads]`` of their sums of squares."""
+    gated = decay is None
+    _gpu(rows, state, weight, out, decay, log_decay, gates)
+    _rows(rows, "scan rows"); _rows(out, "scan out"); _rows(state, "scan state")
+    n, width = rows.shape
+    hk, hv = heads * key_dim, heads * value_dim
+    for name, w in (("q", hk), ("k", hk), ("v", hv), ("g", hv)):
+        if name not in offsets or offsets[name] < 0 or offsets[name] + w > width:
+            raise KernelError(f"decay_scan: the columns of {name!r} lie outside the rows' {width} columns")
+    if key_dim > 256 or value_dim > 512:
+        raise KernelError(f"decay_scan: heads of {key_dim} (values {value_dim}) are not supported (at most 256 and 512)")
+    if state.dtype != torch.float32 or state.shape[1] < decay_state_floats(heads, key_dim, value_dim, gated):
+        raise KernelError(f"decay_scan: a slot of the state must hold {decay_state_floats(heads, key_dim, value_dim, gated)} float32")
+    if n != step.n or max(step.state_slots, default=0) >= state.shape[0]:
+        raise KernelError("decay_scan: the rows are not the step's, or a request's slot lies outside the state")
+    single = step.decode_only
+    if out.shape != (n, hv) or (out.dtype != rows.dtype and not (single and rows.dtype == torch.float32)):
+        raise KernelError(f"decay_scan: out {out.dtype} {tuple(out.shape)} does not fit rows of {rows.dtype}")
+    _f32_vec(weight, "scan norm weight", hv)
+    if gated:
+        bi, bf = gate_bias
+        _gpu(bi, bf)
+        _f32_vec(bi, "input gate bias", heads); _f32_vec(bf, "forget gate bias", heads)
+        _rows(gates, "gate rows")
+        if gates.dtype != torch.float32 or gates.shape != (n, 2 * heads) or not cap > 0:
+            raise KernelError(f"decay_scan: the gates must be float32 {(n, 2 * heads)} with a positive cap")
+        zp, ldz, bip, bfp = _ptr(gates), gates.stride(0), _ptr(bi), _ptr(bf)
+    else:
+        _f32_vec(decay, "decay", heads)
+        if log_decay is None or log_decay.dtype != torch.float32 or log_decay.shape != (heads, 2) or not log_decay.is_contiguous():
+            raise KernelError(f"decay_scan: the decays' logarithms must be contiguous float32 [{heads}, 2]")
+        zp, ldz, bip, bfp = _ptr(None), 0, _ptr(None), _ptr(None)
+    if scaled_rows and (gated or not single or factor != 1.0):
+        raise KernelError("decay_scan: rows that wait for their norm come of a fixed decay in a step of single tokens")
+    lib = build.load("decay_scan")
+    rt, ot = _type(rows, "scan rows"), _type(out, "scan out")
+    cols = (rows.stride(0), offsets["q"], offsets["k"], offsets["v"], offsets["g"], int(bool(silu)))
+    f32 = lambda count: torch.empty(int(count), dtype=torch.float32, device=rows.device)
+    tail = (_ptr(step.q_start), _ptr(step.ctx_len), _ptr(step.state_slot))
+    sizes = (heads, key_dim, value_dim, ctypes.c_float(scale), ctypes.c_float(eps), ctypes.c_float(factor), _stream())
+    stride = ctypes.c_longlong(state.stride(0))
+    if single:
+        sumsq = None if gated else torch.empty((n, heads), dtype=torch.float32, device=rows.device)
+        _check(lib.lcu_decay_scan_single(_ptr(rows), rt, *cols, _ptr(decay), zp, ldz, bip, bfp, ctypes.c_float(cap), _ptr(state), stride,
+                                         _ptr(weight), _ptr(out), ot, out.stride(0), _ptr(sumsq), int(not scaled_rows), *tail, step.n_req,
+                                         *sizes), "decay_scan_single")
+        return sumsq if scaled_rows else None
+    n_long = sum(1 for q in step.q_lens if q >= lib.lcu_decay_scan_long())
+    lib.lcu_decay_scan_run_floats.restype = ctypes.c_longlong
+    o = f32(heads * n * lib.lcu_decay_scan_out_cols(value_dim, int(gated)))
+    runs = f32(lib.lcu_decay_scan_run_floats(n_long, heads, key_dim, value_dim, int(gated))) if n_long else None
+    scratch = f32(3 * heads * n) if gated else None
+    _check(lib.lcu_decay_scan(_ptr(rows), rt, *cols, _ptr(log_decay), zp, ldz, bip, bfp, ctypes.c_float(cap), _ptr(scratch), _ptr(o), _ptr(runs),
+                              n_long, _ptr(state), stride, _ptr(weight), _ptr(out), out.stride(0), *tail, n, step.n_req, *sizes), "decay_scan")
+    return None
+
+
+def decay_state_floats(heads: int, key_dim: int, value_dim: int, gated: bool) -> int:
+    """What a request's state takes in ``decay_scan``: the matrices, and with gates a normaliser and a maximum per head."""
+    return heads * key_dim * value_dim + (heads * (key_dim + 1) if gated else 0)

@@ -50,7 +50,7 @@ class Attention(Part):
         general path: one product for all projections with 32-bit output, then ``ops.qkv_prepare``.
         ``value_dim``: the values' head size if it is not ``head_dim``.  ``projection_norm_eps``: queries and keys
         are divided by the root mean square over their whole projection (all heads at once) and multiplied by a
-        weight per column (tensors ``q_norm``, ``k_norm``).  ``query_temperature = (coef, every)``: the query at
+        weight per column (tensors ``q_norm``, ``k_norm``), before any rotation (with a rotation the general path runs).  ``query_temperature = (coef, every)``: the query at
         position ``p`` is multiplied by ``1 + coef * ln(floor((p + 1) / every) + 1)``."""
         if heads % kv_heads:
             raise ValueError(f"attention: {heads} heads are no multiple of {kv_heads} key/value heads")
@@ -91,11 +91,16 @@ class Attention(Part):
         self.graph_safe = self.position.graph_safe
         rot = self.position.rotated_dims()
         self.general = bool(self.bias or self.head_gate or self.head_norm_eps is not None or self.chunk
-                            or self.values_are_keys or self.sink or self.out_bias
+                            or self.values_are_keys or self.sink or self.out_bias or (rot and self.norm_eps is not None)
                             or (rot and (self.value_dim != self.head_dim or self.padded_dim != self.head_dim)))
-        if self.general and (self.shares_kv or self.norm_eps is not None or self.q_temp is not None):
+        if self.general and (self.shares_kv or self.q_temp is not None):
             raise ValueError("attention: biases, head norms, chunks, a head gate or values of their own size under a rotation "
-                             "do not go together with shared keys and values, a norm over the whole projection or a query temperature")
+                             "do not go together with shared keys and values or a query temperature")
+        if self.general and self.norm_eps is not None and (self.bias or self.head_norm_eps is not None or self.values_are_keys):
+            raise ValueError("attention: on the general path a norm over the whole projection does not go together with biases, head norms or "
+                             "values that are the keys")
+        # the gate's kernel may write the output product's operand anywhere, times a factor
+        self.splits_output = self.general and self.head_gate and not self.out_bias
         # what a head takes in the cache and in the kernels: the true sizes filled up with dims of zeros (general path)
         self.stored_dim, self.stored_value_dim = self.padded_dim, self.value_dim
         self.w_qkv = self.w_o = None
@@ -179,6 +184,8 @@ class Attention(Part):
             self.k_head_norm = tensors[nm["k_head_norm"]].float().contiguous()
         elif self.head_norm_eps is not None:                  # a norm without a weight: the kernel multiplies by ones
             self.q_head_norm = self.k_head_norm = torch.ones(dh, dtype=torch.float32, device=build.device)
+        if self.norm_eps is not None:
+            self.q_norm, self.k_norm = tensors[nm["q_norm"]].float().contiguous(), tensors[nm["k_norm"]].float().contiguous()
         if self.sink:
             self.sinks = tensors[nm["sink"]].float().contiguous()
         if self.out_bias:
@@ -197,7 +204,8 @@ class Attention(Part):
                     break
             else:
                 ops.say_once(f"attention with {nh} heads of {dh} (values {dv}) in {nkv} groups runs on the generic kernel, not on the matrix cores")
-        self.w_o = Weight(w_o.contiguous(), build)
+        self.output_matrix, self.output_width = w_o.contiguous(), nh * self.stored_value_dim
+        self.w_o = Weight(self.output_matrix, build) if self.own_output else None
         self.position.load({}, build)
         if type(self.position).apply is not Part.apply:
             raise ValueError("attention: the general path takes a rotation, a bias inside the scores or no position encoding")
@@ -212,7 +220,8 @@ class Attention(Part):
     # forward(..., bias_later=True) leaves the output projection's bias (``output_bias``, float32, or None) to the caller
     ends_in_bias = True
 
-    def _forward_general(self, h, step, cache, out_dtype=None, bias_later=False):
+    def _heads_general(self, h, step, cache):
+        """(the attention's output before any gate, the input product's rows)"""
         nh, nkv = self.heads, self.kv_heads
         if not cache.writes:
             raise ops.KernelError("attention: the general path needs a cache of its own")
@@ -220,17 +229,30 @@ class Attention(Part):
         rot = self.position.rotary_tables()
         cos, sin, rot_dim, pairing = rot if rot is not None else (None, None, 0, 0)
         rows = linear(h, self.w_in, out_dtype=torch.float32)
-        q = ops.qkv_prepare(rows, self.offsets, nh, nkv, self.head_dim, self.value_dim, self.stored_dim, self.stored_value_dim,
-                            self.dtype, positions=step.positions, bias=self.bias_vec, q_norm=self.q_head_norm,
-                            k_norm=self.k_head_norm, eps=self.head_norm_eps or 0.0, cos=cos, sin=sin, rot_dim=rot_dim,
-                            pairing=pairing, cache=cache.pages, slots=step.slots(cache.group), page_size=page_size)
+        if self.norm_eps is not None:
+            q = ops.qkv_prepare_rows(rows, self.offsets, nh, nkv, self.head_dim, self.value_dim, self.stored_dim, self.stored_value_dim,
+                                     self.dtype, self.q_norm, self.k_norm, self.norm_eps, positions=step.positions, cos=cos, sin=sin,
+                                     rot_dim=rot_dim, pairing=pairing, cache=cache.pages, slots=step.slots(cache.group), page_size=page_size)
+        else:
+            q = ops.qkv_prepare(rows, self.offsets, nh, nkv, self.head_dim, self.value_dim, self.stored_dim, self.stored_value_dim,
+                                self.dtype, positions=step.positions, bias=self.bias_vec, q_norm=self.q_head_norm,
+                                k_norm=self.k_head_norm, eps=self.head_norm_eps or 0.0, cos=cos, sin=sin, rot_dim=rot_dim,
+                                pairing=pairing, cache=cache.pages, slots=step.slots(cache.group), page_size=page_size)
         out = torch.empty((rows.shape[0], nh * self.stored_value_dim), dtype=self.dtype, device=rows.device)
         ops.paged_attention(q, out, cache.pages, step, cache.group, nh, nkv, self.stored_dim, page_size, self.scale,
                             self.window, value_dim=self.stored_value_dim, chunk=self.chunk,
                             force_generic=not self._matrix_cores(page_size), head_slopes=self.position.score_slopes(),
                             sinks=self.sinks)
+        return out, rows
+
+    def forward_rows(self, h, step, cache, out, factor: float = 1.0, state=None) -> None:
+        heads, rows = self._heads_general(h, step, cache)
+        ops.head_gate(heads, rows, self.g_off, self.heads, self.stored_value_dim, out=out, factor=factor)
+
+    def _forward_general(self, h, step, cache, out_dtype=None, bias_later=False, planes_ok=False):
+        out, rows = self._heads_general(h, step, cache)
         if self.head_gate:
-            ops.head_gate(out, rows, self.g_off, nh, self.stored_value_dim)
+            ops.head_gate(out, rows, self.g_off, self.heads, self.stored_value_dim)
         if self.output_bias is not None and not bias_later:
             return ops.row_bias(linear(out, self.w_o, out_dtype=out_dtype or torch.float32), self.output_bias)
         return linear(out, self.w_o, out_dtype=out_dtype or self.dtype)

@@ -33,7 +33,7 @@ import torch
 class TensorSpec:
     """One tensor a part binds: its shape, and how a random model fills it: the name of an
     initialiser (``normal``: N(0, std); ``one_plus_normal``: 1 + N(0, std), for norm weights;
-    ``zeros``; ``ones``; or one that ``weights.register_initialiser`` has made known).
+    ``identity_plus_normal``; ``zeros``; ``ones``; or one that ``weights.register_initialiser`` has made known).
     ``integer`` tensors are kept as int32, all others follow the weight policy."""
     shape: Tuple[int, ...]
     init: str = "normal"
@@ -232,6 +232,18 @@ class NormedRows:
     rows: torch.Tensor
 
 
+@dataclass
+class StreamUpdate:
+    """A sublayer's output on its way into several residual streams (``parts/streams.py``): ``x_t <- sum_s mix[s, t] x_s + out[t] *
+    delta``, all streams at once.  Whoever norms next lets it in."""
+    delta: torch.Tensor         # [n, width] in the compute type or float32, or float32 planes [planes, n, width]
+    mix: torch.Tensor           # [streams, streams] float32: from, to
+    out: torch.Tensor           # [streams] float32
+
+    def at_rows(self, gather) -> "StreamUpdate":
+        return StreamUpdate(gather(self.delta), self.mix, self.out)
+
+
 class Part:
     # Whether a step through this part may be captured into a graph and replayed: true only
     # if all it does is launch work on the current stream whose shape depends on the batch's
@@ -262,6 +274,14 @@ class Part:
     deferrable = False
     delta_scale = 1.0
     reads_float32 = False
+    # embedding, block, final norm: how many residual streams a row holds side by side (all three agree)
+    streams = 1
+    # mixer: ``splits_output``: its last step is a product with ``output_matrix`` ([width, output_width], known after ``load``), and
+    # ``forward_rows(h, step, cache, out, factor, state=)`` writes what it would multiply, times ``factor``, into the columns ``out``
+    # instead: several such mixers' rows side by side are one product.  ``own_output`` False (set before ``load``): somebody else
+    # multiplies, so the part keeps no matrix of its own for it.
+    splits_output = False
+    own_output = True
     takes_planes = False
     ends_in_norm = False
     ends_in_planes = False

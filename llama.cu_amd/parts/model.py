@@ -15,18 +15,18 @@ from typing import Dict, List, Optional
 import torch
 
 from ..kernels import ops
-from .base import BuildContext, ModelSpec, Part, ScaledRows, TensorSpec, make_part, prefixed, register_part
+from .base import BuildContext, ModelSpec, Part, ScaledRows, StreamUpdate, TensorSpec, make_part, prefixed, register_part
 from .linear import Weight, linear, linear_scaled, skinny_takes
 
 
 class TokenEmbedding(Part):
     graph_safe = True
 
-    def __init__(self, vocab_size: int, hidden_size: int, scale: float = 1.0, tensor: str = "weight"):
+    def __init__(self, vocab_size: int, hidden_size: int, scale: float = 1.0, tensor: str = "weight", streams: int = 1):
         """``scale``: every row is multiplied by it (in 32-bit) on its way into the residual stream.
-        ``tensor``: the table's name under the part's."""
+        ``tensor``: the table's name under the part's.  ``streams``: so many residual streams, all equal at the start."""
         self.vocab_size, self.hidden_size = int(vocab_size), int(hidden_size)
-        self.scale, self.tensor = float(scale), str(tensor)
+        self.scale, self.tensor, self.streams = float(scale), str(tensor), int(streams)
         self.weight = None
 
     def tensors(self):
@@ -36,9 +36,9 @@ class TokenEmbedding(Part):
         self.weight = tensors[self.tensor].contiguous()
 
     def forward(self, tokens: torch.Tensor) -> torch.Tensor:
-        """The residual stream of the step's tokens, float32 ``[n, d]``."""
-        out = torch.empty((tokens.numel(), self.hidden_size), dtype=torch.float32, device=tokens.device)
-        return ops.embedding_gather(self.weight, tokens, out, self.scale)
+        """The residual stream of the step's tokens, float32 ``[n, d]`` (several: ``[n, streams * d]``)."""
+        out = torch.empty((tokens.numel(), self.streams * self.hidden_size), dtype=torch.float32, device=tokens.device)
+        return ops.embedding_gather(self.weight, tokens, out, self.scale, copies=self.streams)
 
 
 class OutputHead(Part):
@@ -90,6 +90,10 @@ class DecoderModel:
         self.head = make_part("head", spec.head)
         self.streams: List[Part] = [make_part("stream", s) for s in spec.streams]
         self.graph_safe = all(p.graph_safe for p in [self.embedding, self.final_norm, self.head] + self.layers + self.streams)
+        counts = {p.streams for p in [self.embedding, self.final_norm] + self.layers}
+        if len(counts) != 1 or (counts != {1} and self.streams):
+            raise ValueError(f"the embedding, the layers and the final norm keep {sorted(counts)} residual streams: they must agree (and parts "
+                             f"that change the stream between layers know one)")
         n = len(self.layers)
         for i, e in enumerate(spec.run_order):
             if not 0 <= e.layer < n:
@@ -203,6 +207,7 @@ class DecoderModel:
                 xs, ps = x, pending
             else:
                 xs = ops.gather_rows(x, step.logit_rows)
-                ps = ops.gather_rows(pending, step.logit_rows) if pending is not None else None
+                gather = lambda t: ops.gather_rows(t, step.logit_rows)
+                ps = pending.at_rows(gather) if isinstance(pending, StreamUpdate) else gather(pending) if pending is not None else None
             y = self.final_norm.forward(xs, ps)
             return self.head.forward(y)

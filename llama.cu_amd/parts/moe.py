@@ -90,6 +90,10 @@ class GatedMoE(Part):
     are chosen (``correction``: a tensor ``[experts]`` that moves the choice and nothing else), and the weights are the chosen
     ``s`` divided by their sum + 1e-20.  ``identity``: so many more outputs of the router, behind the experts', stand for
     identity experts, which have no tensors and whose output is the input itself (times the weight).
+    ``renormalize=False``: the weights are the chosen ``s`` as they are; ``scale``: times a factor; ``groups``, ``keep_groups``: the experts
+    are so many groups of neighbours, and a token's come from the ``keep_groups`` whose best expert's score is largest (all three with
+    ``softmax_all``).  ``activation="limited"``: with ``g = min(W_gate h, limit)`` and ``u`` = ``W_up h`` held within ``-limit .. limit`` an
+    expert is ``W_down (g sigmoid(alpha g) (u + 1))``.
     ``shared_gated=False``: the shared expert is added as it is, without a gate.  ``forward(h, add_to=)`` adds the output
     into 32-bit rows that hold another branch's output already."""
     graph_safe = True
@@ -101,7 +105,8 @@ class GatedMoE(Part):
 
     def __init__(self, hidden_size: int, expert_size: int, experts: int, top: int, shared_size: Optional[int] = None,
                  router_bias: bool = True, names: Optional[Dict[str, str]] = None, scoring: str = "softmax_chosen",
-                 correction: bool = False, identity: int = 0, shared_gated: bool = True):
+                 correction: bool = False, identity: int = 0, shared_gated: bool = True, renormalize: bool = True, scale: float = 1.0,
+                 groups: int = 1, keep_groups: int = 1, activation: str = "silu", alpha: float = 1.0, limit: float = 0.0):
         self.hidden_size, self.expert_size = int(hidden_size), int(expert_size)
         self.experts, self.top, self.identity = int(experts), int(top), int(identity)
         self.outputs = self.experts + self.identity          # what the router chooses among
@@ -113,6 +118,16 @@ class GatedMoE(Part):
         if correction and scoring != "softmax_all":
             raise ValueError("moe: a correction of the choice goes with scores over all experts")
         self.scoring, self.correction, self.shared_gated = scoring, bool(correction), bool(shared_gated)
+        self.choice = {}
+        if not renormalize or float(scale) != 1.0 or int(groups) != 1:
+            if scoring != "softmax_all" or self.outputs % int(groups) or not 1 <= int(keep_groups) <= int(groups) \
+                    or self.top > int(keep_groups) * (self.outputs // int(groups)):
+                raise ValueError(f"moe: weights as they are, a factor and groups go with scores over all experts; top {top} of {keep_groups} of "
+                                 f"{groups} groups of {self.outputs} is not supported")
+            self.choice = {"renorm": bool(renormalize), "scale": float(scale), "groups": int(groups), "keep": int(keep_groups)}
+        if activation not in ("silu", "limited") or (activation == "limited" and not limit > 0):
+            raise ValueError(f"moe: the experts' activation is 'silu', or 'limited' with a positive limit, not {activation!r} ({limit})")
+        self.act = {"act_alpha": float(alpha), "act_limit": float(limit)} if activation == "limited" else {}
         self.names = dict(self.NAMES, **(names or {}))
         self.router_bias = bool(router_bias)
         self.shared = None
@@ -166,6 +181,15 @@ class GatedMoE(Part):
             gate = torch.cat([gate, gate.new_zeros(n, pad, d)], dim=1)
             up = torch.cat([up, up.new_zeros(n, pad, d)], dim=1)
             self.w_down = torch.cat([self.w_down, self.w_down.new_zeros(n, d, pad)], dim=2).contiguous()
+        # the products load 16 bytes at a time along the width too: a width that does not fill them gets columns of zeros
+        per = 8 if build.dtype == torch.bfloat16 else 4
+        self.pad_width = -d % per
+        if self.pad_width:
+            if self.shared is not None:
+                raise ValueError(f"moe: a width of {d}, no multiple of {per}, together with a shared expert is not supported")
+            fill = lambda t, dims: torch.nn.functional.pad(t, dims)
+            gate, up, self.router = fill(gate, (0, self.pad_width)), fill(up, (0, self.pad_width)), fill(self.router, (0, self.pad_width)).contiguous()
+            self.w_down = fill(self.w_down, (0, 0, 0, self.pad_width)).contiguous()
         self.w_gate_up = ops.gated_rows(gate.contiguous(), up.contiguous())
         if self.shared is not None:
             self.shared.load(tensors, build)
@@ -173,17 +197,23 @@ class GatedMoE(Part):
 
     def forward(self, h, add_to: Optional[torch.Tensor] = None):
         """``add_to``: float32 ``[n, d]`` that takes the output in (and is returned); without it the output is new rows."""
+        if self.pad_width:
+            out = self._experts(torch.nn.functional.pad(h, (0, self.pad_width)), None)[:, :self.hidden_size].contiguous()
+            return out if add_to is None else ops.scaled_sum(add_to, out, 1.0)
+        return self._experts(h, add_to)
+
+    def _experts(self, h, add_to):
         over_all = self.scoring == "softmax_all"
         routed = ops.moe_route(h, self.router, self.top, bias=self.bias, softmax_chosen=not over_all, softmax_all=over_all,
-                               extra=self.gates)
+                               extra=self.gates, **self.choice)
         ids, wts = routed[0], routed[1]
         fresh = add_to is None
-        out = add_to if not fresh else torch.empty((h.shape[0], self.hidden_size), dtype=torch.float32, device=h.device)
+        out = add_to if not fresh else torch.empty((h.shape[0], h.shape[1]), dtype=torch.float32, device=h.device)
         if self.shared is not None:
             ops.moe_experts(h, ids, wts, self.w_gate_up, self.w_down, out, gated=True, shared=self.shared.forward(h),
-                            shared_gate=routed[2] if self.gates else None, fresh=fresh, identity=self.identity)
+                            shared_gate=routed[2] if self.gates else None, fresh=fresh, identity=self.identity, **self.act)
         else:
-            ops.moe_experts(h, ids, wts, self.w_gate_up, self.w_down, out, gated=True, fresh=fresh, identity=self.identity)
+            ops.moe_experts(h, ids, wts, self.w_gate_up, self.w_down, out, gated=True, fresh=fresh, identity=self.identity, **self.act)
         return out
 
 

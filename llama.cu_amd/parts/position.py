@@ -64,8 +64,15 @@ class Rotary(NoPosition):
     """
 
     def __init__(self, head_dim: int, theta: float, max_positions: int, interleaved: bool = False,
-                 rot_dim: int = 0, scaling_factor: float = 1.0):
-        """``scaling_factor``: linear scaling, every frequency is divided by it (in 32-bit)."""
+                 rot_dim: int = 0, scaling_factor: float = 1.0, yarn=None):
+        """``scaling_factor``: linear scaling, every frequency is divided by it (in 32-bit).  ``yarn`` (``{"factor", "original", "fast",
+        "slow"}``): frequencies blended between themselves and themselves divided by ``factor``.  The pair whose angle makes ``t`` turns
+        in ``original`` positions is ``pair(t) = rot_dim ln(original / (2 pi t)) / (2 ln theta)``; pairs up to ``floor(pair(fast))`` keep their
+        frequency, pairs from ``ceil(pair(slow))`` on have it divided, in between the share is linear; cosine and sine are multiplied by ``0.1
+        ln(factor) + 1``."""
+        self.yarn = None if yarn is None else tuple(float(yarn[k]) for k in ("factor", "original", "fast", "slow"))
+        if self.yarn is not None and (min(self.yarn) <= 0 or float(theta) in (0.0, 1.0) or float(scaling_factor) != 1.0):
+            raise ValueError(f"rotary: blended frequencies {yarn} need positive numbers, a base that is not 1 and no other scaling")
         self.head_dim = int(head_dim)
         self.scaling_factor = float(scaling_factor)
         if not self.scaling_factor > 0:
@@ -78,8 +85,25 @@ class Rotary(NoPosition):
         self.interleaved = bool(interleaved)
         self.cos = self.sin = None
 
+    def yarn_frequencies(self):
+        """(frequencies [rot_dim / 2] in 64-bit, the factor on cosine and sine)"""
+        factor, original, fast, slow = self.yarn
+
+        def pair(turns):
+            return self.rot_dim * np.log(original / (2.0 * np.pi * turns)) / (2.0 * np.log(self.theta))
+
+        i = np.arange(self.rot_dim // 2, dtype=np.float64)
+        freq = np.power(self.theta, -2.0 * i / self.rot_dim)
+        low, high = max(np.floor(pair(fast)), 0.0), min(np.ceil(pair(slow)), self.rot_dim - 1.0)
+        share = np.clip((i - low) / max(high - low, 0.001), 0.0, 1.0)
+        return freq / factor * share + freq * (1.0 - share), 0.1 * np.log(factor) + 1.0
+
     def host_tables(self):
         half = self.rot_dim // 2
+        if self.yarn is not None:               # in 64-bit, rounded once
+            freq, size = self.yarn_frequencies()
+            ang = np.arange(self.max_positions, dtype=np.float64)[:, None] * freq[None, :]
+            return (size * np.cos(ang)).astype(np.float32), (size * np.sin(ang)).astype(np.float32)
         # 32-bit throughout, as the reference: theta.powf(-((2 * i) as f32 / dh as f32))
         expo = -(np.float32(2.0) * np.arange(half, dtype=np.float32) / np.float32(self.rot_dim))
         freq = np.power(np.float32(self.theta), expo.astype(np.float32)).astype(np.float32)
@@ -90,7 +114,7 @@ class Rotary(NoPosition):
         return np.cos(ang).astype(np.float32), np.sin(ang).astype(np.float32)
 
     def load(self, tensors, build: BuildContext) -> None:
-        key = (self.theta, self.rot_dim, self.max_positions, str(torch.device(build.device)), self.scaling_factor)
+        key = (self.theta, self.rot_dim, self.max_positions, str(torch.device(build.device)), self.scaling_factor, self.yarn)
         tables = _tables.get(key)
         if tables is None:
             cos, sin = self.host_tables()

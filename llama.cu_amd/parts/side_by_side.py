@@ -1,6 +1,8 @@
 """Several mixers side by side: all read the same input, and the mixer's output is the sum of theirs, each times a
 factor: ``out = sum_i scale_i * mixer_i(h)``.  Each mixer keeps its own tensors under its own name and its own cache
-need; at most one of them may hold keys and values in pages (``SeveralNeeds``).  The sum is 32-bit.
+need; at most one of them may hold keys and values in pages (``SeveralNeeds``).  The sum is 32-bit.  Where every mixer can hand over the
+rows that its output product would multiply (``splits_output``), they are written side by side, each times its factor, and the output
+products and the sum are one product.
 """
 from __future__ import annotations
 
@@ -10,6 +12,7 @@ import torch
 
 from ..kernels import ops
 from .base import BuildContext, Part, PartSpec, SeveralNeeds, TensorSpec, make_part, prefixed, register_part
+from .linear import Weight, finish
 
 
 class SideBySide(Part):
@@ -21,6 +24,10 @@ class SideBySide(Part):
         self.scales = [float(x) for x in scales]
         self.graph_safe = all(m.graph_safe for m in self.mixers)
         # under which name each mixer with a need finds a state of its own in the one LayerCache (SeveralNeeds)
+        self.joint = all(m.splits_output for m in self.mixers)
+        if self.joint:
+            for m in self.mixers:
+                m.own_output = False
         self._state_of, kept = {}, 0
         for i, m in enumerate(self.mixers):
             if m.cache_need() is not None:
@@ -45,6 +52,10 @@ class SideBySide(Part):
             pre = spec.name + "." if spec.name else ""
             m.load({k[len(pre):]: v for k, v in tensors.items() if k.startswith(pre)}, build)
         self.dtype = build.dtype
+        if self.joint:
+            self.w_o = Weight(torch.cat([m.output_matrix for m in self.mixers], dim=1).contiguous(), build)
+            for m in self.mixers:
+                m.output_matrix = None
 
     def cache_need(self):
         kept = [n for n in (m.cache_need() for m in self.mixers) if n is not None]
@@ -57,7 +68,19 @@ class SideBySide(Part):
     def decode_splits(self, batch: int, max_ctx_len: int) -> int:
         return max(int(m.decode_splits(batch, max_ctx_len)) for m in self.mixers)
 
-    def forward(self, h, step, cache, out_dtype=None):
+    @property
+    def ends_in_planes(self):
+        return self.joint
+
+    def forward(self, h, step, cache, out_dtype=None, planes_ok=False):
+        if self.joint:
+            both = torch.empty((h.shape[0], self.w_o.shape[1]), dtype=self.dtype, device=h.device)
+            at = 0
+            for i, (m, scale) in enumerate(zip(self.mixers, self.scales)):
+                state = cache.more.get(self._state_of.get(i))
+                m.forward_rows(h, step, cache, both[:, at:at + m.output_width], scale, state=state)
+                at += m.output_width
+            return finish(both, self.w_o, self.dtype, planes_ok=planes_ok, out_dtype=out_dtype)
         total = None
         for i, (m, scale) in enumerate(zip(self.mixers, self.scales)):
             kw = {}

@@ -85,6 +85,8 @@ def registered_initialisers() -> List[str]:
 
 register_initialiser("normal", lambda out, key, std: fill_normal(out, key, std))                   # N(0, std): matrices
 register_initialiser("one_plus_normal", lambda out, key, std: fill_normal(out, key, std, 1.0))    # 1 + N(0, std): norm weights
+register_initialiser("identity_plus_normal",                                                         # I + N(0, std): a square map that keeps most
+                     lambda out, key, std: fill_normal(out, key, std).add_(torch.eye(out.shape[0], dtype=out.dtype, device=out.device)))
 register_initialiser("zeros", lambda out, key, std: out.zero_())
 register_initialiser("ones", lambda out, key, std: out.fill_(1.0))
 
