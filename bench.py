@@ -465,9 +465,33 @@ def gefudra_config(z, positions):
                                     "loop": {"start": 0, "stop": 3, "times": times}, "max_positions": positions})
 
 
+def lapunex_config(z, positions):
+    """As many layer runs as the Llama model beside it has layers, over four residual streams: linear attention with a fixed decay and the
+    dense feed-forward; then as a loop that runs as often as fits linear attention with a mixture of experts (in four groups of
+    which two are kept) and the side-by-side mixer (attention with half of each head rotated and a sink beside a matrix memory,
+    half of the heads each) with the dense feed-forward; then linear attention with experts.  A token's experts have about as many weights as
+    Llama's feed-forward."""
+    from llama_cu_amd.config import LapunexConfig
+    inter = (z["top"] * 2 * z["ff"] // 3 + 127) // 128 * 128
+    d, h, g, w = z["dim"], z["heads"], z["kv_heads"], z["width"]
+    lightning = {"type": "lightning", "mixer": {"heads": h, "dim": d, "vdim": d, "decay": [1.0 - 0.3 / (1 + k) ** 2 for k in range(h)]}}
+    left = {"heads": h // 2, "kv_heads": g // 2, "dim": d, "vdim": d, "scale": d ** -0.5,
+            "rot": {"base": 10000.0, "dims": d // 2, "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}
+    parallel = {"type": "parallel", "mixer": {"left": left, "right": {"heads": h // 2, "dim": d, "vdim": d, "gate_cap": 15.0},
+                                              "left_scale": 0.75, "right_scale": 1.25}}
+    dense = {"kind": "dense", "ff": inter}
+    moe = {"kind": "moe", "expert": {"ff": inter // z["top"] // 64 * 64, "limit": 7.0},
+           "router": {"experts": z["experts"], "top": z["top"], "scale": 2.5, "groups": {"count": 4, "keep": 2}}}
+    return LapunexConfig.from_dict({"architecture": "Lapunex", "vocab": z["vocab"], "width": w, "streams": 4, "norm": {"eps": 1e-5},
+                                    "embedding": {"scale": 2.0}, "max_positions": positions,
+                                    "layers": [dict(lightning, mlp=dense), dict(lightning, mlp=moe), dict(parallel, mlp=dense), dict(lightning, mlp=moe)],
+                                    "loop": {"start": 1, "stop": 3, "times": (z["layers"] - 2) // 2}})
+
+
 DESIGN_CONFIGS = {"divasun": lambda z, p: divasun_config(z, p), "llama": lambda z, p: llama_like(z, p),
                   "lozezen": lambda z, p: lozezen_config(z, p), "ralepel": lambda z, p: ralepel_config(z, p),
-                  "mufotar": lambda z, p: mufotar_config(z, p), "gefudra": lambda z, p: gefudra_config(z, p)}
+                  "mufotar": lambda z, p: mufotar_config(z, p), "gefudra": lambda z, p: gefudra_config(z, p),
+                  "lapunex": lambda z, p: lapunex_config(z, p)}
 
 
 def llama_like(z, positions):
@@ -594,10 +618,10 @@ def main() -> int:
                          "decode while a prompt of 16 tokens arrives every second step (host time and the GPU's busy "
                          "fraction per kind of step)")
     ap.add_argument("--designs", default="divasun,llama", metavar="NAMES",
-                    help="with --workload designs: which designs are measured side by side, of divasun, lozezen, ralepel, mufotar, gefudra and llama "
+                    help="with --workload designs: which designs are measured side by side, of divasun, lozezen, ralepel, mufotar, gefudra, lapunex and llama "
                          "(default: divasun,llama)")
     ap.add_argument("--designs-one", metavar="DESIGN:SIZE:WHAT", default=None,
-                    help="with --workload designs, for a profiler: only DESIGN (divasun, lozezen, ralepel, mufotar, gefudra or llama) at SIZE (w2048, w4096), and "
+                    help="with --workload designs, for a profiler: only DESIGN (divasun, lozezen, ralepel, mufotar, gefudra, lapunex or llama) at SIZE (w2048, w4096), and "
                          "only WHAT: 'prefill' (three steps of 2,048 tokens) or a number of requests that decode ten steps over "
                          "prompts of 512 tokens; steps are launched one kernel at a time, not replayed from graphs")
     ap.add_argument("--no-points", action="store_true", help="skip decoding at batch 1 and 64, the prefill and the check")
