@@ -20,6 +20,9 @@
 // transposed), shared by the workgroup's waves.  Products of 32-bit operands (S, the weighted scores, the weighted values)
 // with bfloat16 ones are made of three bfloat16 products, of the operand's upper, middle and lower eight bits, which loses
 // nothing of its 24; in float32 all products run on the 32-bit matrix instruction.  L is summed in 64-bit and kept in two parts.
+// The weights exp(L_t - L_s) b_s are made once a chunk for all waves, few of them: those of a tile's own 16 tokens one by one, those of
+// tokens in an earlier tile as exp(L_t - L_e) times exp(L_e - L_s) b_s, e that tile's last token (neither factor exceeds 1 where
+// no decay does).
 // A request that feeds DS_LONG tokens or more is cut into up to DS_RUNS runs that are walked side by side, twice: first
 // from zeros, which gives what a run adds to any state; a small kernel chains the runs' starts; the second walk gives the outputs.
 //
@@ -32,8 +35,9 @@
 #include "lane_moves.h"
 
 constexpr int DS_RUNS = 16;
-constexpr int DS_LONG = 512;
-constexpr int DS_WAVES = 4;                       // waves of a chunk workgroup at most
+constexpr int DS_LONG = 256;                     // (not fewer: steps of up to 256 tokens are captured into graphs by their sizes, and of those only a
+                                                  // lone request's may be long)
+constexpr int DS_WAVES = 8;                       // waves of a chunk workgroup at most
 
 typedef __attribute__((ext_vector_type(4))) float f32x4;
 typedef __attribute__((ext_vector_type(4))) uint32_t u32x4;
@@ -43,6 +47,13 @@ typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
 __device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
 __device__ __forceinline__ float silu_f(float z) { return z / (1.0f + expf(-z)); }
 __device__ __forceinline__ float log_sigmoid_f(float z) { return fminf(z, 0.f) - log1pf(expf(-fabsf(z))); }
+
+// silu of a value that is rounded to T next: to bfloat16 with the hardware's exponential and reciprocal (an error of 2^-20 or so)
+template <class T> __device__ __forceinline__ float silu_for(float z);
+template <> __device__ __forceinline__ float silu_for<float>(float z) { return silu_f(z); }
+template <> __device__ __forceinline__ float silu_for<bf16_t>(float z) {
+    return z * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.44269504f * z));
+}
 
 template <class T, int V> struct alignas(V * sizeof(T)) DsVec { T v[V]; };
 
@@ -107,21 +118,23 @@ __device__ __forceinline__ int ds_run_len(int q) {          // a multiple of 64 
 
 // ---------------------------------------------------------------- the gates
 // z: [n, ld] 32-bit with the input gates' projections at z[., h] and the forget gates' at z[., heads + h].  To log_a, b, m: [heads][n].
-// A workgroup per (head, request): 256 tokens at a time, (F, M) = (sum of f, the maximum that tokens alone would leave) composed
+// A workgroup per (head, request): THREADS tokens at a time, (F, M) = (sum of f, the maximum that tokens alone would leave) composed
 // across the threads.
-__global__ void __launch_bounds__(256)
+template <int THREADS>
+__global__ void __launch_bounds__(THREADS)
 ds_gates_kernel(const float *__restrict__ z, int ld, const float *__restrict__ bias_i, const float *__restrict__ bias_f, float cap,
                 float *__restrict__ state, size_t slot_stride, size_t m_off, float *__restrict__ log_a, float *__restrict__ b_out,
                 float *__restrict__ m_out, const int *__restrict__ q_start, const int *__restrict__ ctx_len,
                 const int *__restrict__ state_slot, int n, int heads) {
-    __shared__ float wf[4], wm[4];
+    constexpr int WAVES = THREADS / WAVE;
+    __shared__ float wf[WAVES], wm[WAVES];
     const int h = blockIdx.x, r = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int t0 = q_start[r], t1 = q_start[r + 1];
     if (t1 <= t0) return;
     float *m_slot = state + (size_t)state_slot[r] * slot_stride + m_off + h;
     float m = ctx_len[r] - (t1 - t0) > 0 ? *m_slot : 0.f;
     const float bi = bias_i[h], bf = bias_f[h];
-    for (int base = t0; base < t1; base += 256) {
+    for (int base = t0; base < t1; base += THREADS) {
         const int t = base + tid;
         float gi = -INFINITY, f = 0.f;                     // beyond the last token: nothing changes
         if (t < t1) {
@@ -138,7 +151,8 @@ ds_gates_kernel(const float *__restrict__ z, int ld, const float *__restrict__ b
         if (lane == 63) { wf[wave] = F; wm[wave] = M; }
         __syncthreads();
         float start = m;                                   // the maximum in front of this wave's tokens, and behind all
-        for (int w = 0; w < 4; ++w) {
+#pragma unroll
+        for (int w = 0; w < WAVES; ++w) {
             if (w < wave) start = fmaxf(start + wf[w], wm[w]);
             m = fmaxf(m + wf[w], wm[w]);
         }
@@ -179,13 +193,17 @@ template <class T> struct DsChunk {
 // MODE 0: a request of fewer than DS_LONG tokens.  1: a run from zeros, leaves its own sum in run_b and the sum of its log a in run_l.
 // 2: a run from run_in, with outputs; the last one leaves the request's state.
 template <class T, int D, int MODE>
-__global__ void __launch_bounds__(DS_WAVES *WAVE)
+__global__ void __launch_bounds__(DS_WAVES *WAVE, 1)
 ds_chunk_kernel(DsArgs p) {
     typedef DsMma<T> M;
     typedef typename M::frag frag;
     constexpr int C = DsChunk<T>::tokens(D), PAD = 16 / sizeof(T), LDK = D + PAD, LDT = C + PAD;
     constexpr int TT = C / 16, KT = D / 16, TPS = M::PER / 4;                // tiles of tokens, of key channels; tiles a step of a product
     __shared__ __attribute__((aligned(16))) T qs[C * LDK], ks[C * LDK], kt[D * LDT];
+    // weights: [t][s % 16] of a tile's own tokens (rows of 20: no bank twice); t behind the end of each earlier tile; s up to the end of its tile; t from the chunk's
+    // start; s up to the chunk's end, and the whole chunk
+    __shared__ __attribute__((aligned(16))) float w_own[MODE == 1 ? 1 : C * 20], w_tile[MODE == 1 ? 1 : C], w_end[C];
+    __shared__ float w_behind[MODE == 1 ? 1 : TT * C], w_start[MODE == 1 ? 1 : C], w_all;
     __shared__ float l_hi[C], l_lo[C], b_s[C];
     const int r = MODE == 0 ? blockIdx.z : blockIdx.z / DS_RUNS, run = MODE == 0 ? 0 : blockIdx.z % DS_RUNS, h = blockIdx.y;
     int t0 = p.q_start[r], t1 = p.q_start[r + 1];
@@ -255,7 +273,7 @@ ds_chunk_kernel(DsArgs p) {
 #pragma unroll
                     for (int e = 0; e < 4; ++e) {
                         const bool in_row = t < nt && c0 + e < d;
-                        if (p.silu) { kv[a][e] = silu_f(kv[a][e]); qv[a][e] = silu_f(qv[a][e]); }
+                        if (p.silu) { kv[a][e] = silu_for<T>(kv[a][e]); qv[a][e] = silu_for<T>(qv[a][e]); }
                         if (!in_row) kv[a][e] = qv[a][e] = 0.f;
                     }
                     DsVec<T, 4> ko, qo;
@@ -308,12 +326,32 @@ ds_chunk_kernel(DsArgs p) {
             for (int i = 0; i < 4; ++i) {
                 const int t = 16 * x + 4 * g + i;
                 float e = to_f32(rows[(size_t)(base + min(t, nt - 1)) * p.row_stride + p.v_off + h * dv + min(col, dv - 1)]);
-                if (p.silu) e = silu_f(e);
+                if (p.silu) e = silu_for<T>(e);
                 v[x][i] = to_f32(from_f32<T>(t >= nt || col >= p.dvx ? 0.f : col < dv ? e : 1.f));
             }
         __syncthreads();
+        // ---- the weights
+        {
+            auto between = [&](int t, int u) { return expf((l_hi[t] - l_hi[u]) + (l_lo[t] - l_lo[u])); };
+            if (MODE != 1) {
+                for (int x = tid; x < C * 16; x += threads) {
+                    const int t = x / 16, u = t / 16 * 16 + x % 16;
+                    w_own[t * 20 + x % 16] = u <= t ? between(t, u) * b_s[u] : 0.f;
+                }
+                for (int x = tid; x < TT * C; x += threads) {
+                    const int c = x / C, t = x % C;
+                    if (t / 16 > c) w_behind[x] = between(t, 16 * c + 15);
+                }
+                for (int t = tid; t < C; t += threads) {
+                    w_tile[t] = between(t | 15, t) * b_s[t];
+                    w_start[t] = expf(l_hi[t] + l_lo[t]);
+                }
+            }
+            for (int t = tid; t < C; t += threads) w_end[t] = between(C - 1, t) * b_s[t];
+            if (tid == 0) w_all = expf(l_hi[C - 1] + l_lo[C - 1]);
+        }
+        __syncthreads();
         if (!active) continue;
-        const float end_hi = l_hi[C - 1], end_lo = l_lo[C - 1];
         if (MODE != 1) {
             // ---- what the chunk found in the state, and the scores
             f32x4 o[TT], sc[TT][TT];
@@ -345,17 +383,16 @@ ds_chunk_kernel(DsArgs p) {
 #pragma unroll
             for (int a = 0; a < TT; ++a) {
                 const int t = 16 * a + l16;
-                const float t_hi = l_hi[t], t_lo = l_lo[t];
-                o[a] *= expf(t_hi + t_lo);
+                o[a] *= w_start[t];
 #pragma unroll
                 for (int c0 = 0; c0 < TT; c0 += TPS) {
                     if (c0 > a) continue;
                     float w[M::PER], vv[M::PER];
 #pragma unroll
                     for (int j = 0; j < M::PER; ++j) {
-                        const int c = c0 + j / 4, u = 16 * c + 4 * g + j % 4;
-                        w[j] = 0.f;
-                        if (c <= a && u <= t) w[j] = sc[a][c][j % 4] * (expf((t_hi - l_hi[u]) + (t_lo - l_lo[u])) * b_s[u]);
+                        const int c = c0 + j / 4;
+                        const float own = c == a ? w_own[t * 20 + 4 * g + j % 4] : 0.f;
+                        w[j] = c < a ? sc[a][c][j % 4] * (w_behind[c * C + t] * w_tile[16 * c + 4 * g + j % 4]) : c == a ? sc[a][c][j % 4] * own : 0.f;
                         vv[j] = v[c][j % 4];
                     }
                     frag wf[M::SPLITS];
@@ -370,10 +407,10 @@ ds_chunk_kernel(DsArgs p) {
                 }
             }
         }
-        l_run += (double)end_hi + (double)end_lo;
+        l_run += (double)l_hi[C - 1] + (double)l_lo[C - 1];
         if (MODE == 2 && !last && base + C >= t1) break;                       // nobody reads the state behind this run
         // ---- the state behind the chunk
-        const float keep = expf(end_hi + end_lo);
+        const float keep = w_all;
 #pragma unroll
         for (int x = 0; x < KT; ++x) s[x] *= keep;
 #pragma unroll
@@ -382,7 +419,7 @@ ds_chunk_kernel(DsArgs p) {
 #pragma unroll
             for (int j = 0; j < M::PER; ++j) {
                 const int c = c0 + j / 4, u = 16 * c + 4 * g + j % 4;
-                w[j] = v[c][j % 4] * (expf((end_hi - l_hi[u]) + (end_lo - l_lo[u])) * b_s[u]);
+                w[j] = v[c][j % 4] * w_end[u];
             }
             frag wf[M::SPLITS];
             M::split(w, wf);
@@ -421,10 +458,15 @@ ds_chain_kernel(DsArgs p) {
     float at = 0.f;
     if (p.ctx_len[r] > q_len) at = col < p.dv ? slot[((size_t)h * p.d + key) * p.dv + col] : slot[p.n_off + (size_t)h * p.d + key];
     const size_t first = ((size_t)ds_long_index(p.q_start, r) * DS_RUNS) * p.heads + h;
-    for (int k = 0; k < runs; ++k) {
+    float b[DS_RUNS];                             // (all loads are on their way before the first is needed)
+#pragma unroll
+    for (int k = 0; k < DS_RUNS; ++k) b[k] = p.run_b[(first + (size_t)min(k, runs - 2) * p.heads) * per + e];
+#pragma unroll
+    for (int k = 0; k < DS_RUNS; ++k) {
+        if (k >= runs) break;
         const size_t no = first + (size_t)k * p.heads;
         p.run_in[no * per + e] = at;
-        if (k + 1 < runs) at = fmaf(expf(p.run_l[no]), at, p.run_b[no * per + e]);
+        if (k + 1 < runs) at = fmaf(expf(p.run_l[no]), at, b[k]);
     }
 }
 
@@ -533,13 +575,13 @@ ds_single_kernel(DsSingle p) {
     if (fresh) a = 0.f;                           // the state is zero: what the slot held is not used (it is not read either)
     for (int c = tid; c < d; c += 256) {
         float q = to_f32(row[p.q_off + h * d + c]), k = to_f32(row[p.k_off + h * d + c]);
-        if (p.silu) { q = silu_f(q); k = silu_f(k); }
+        if (p.silu) { q = silu_for<T>(q); k = silu_for<T>(k); }
         qk[0][c] = to_f32(from_f32<T>(q));
         qk[1][c] = to_f32(from_f32<T>(k));
     }
     for (int c = tid; c < dv; c += 256) {
         float v = to_f32(row[p.v_off + h * dv + c]);
-        if (p.silu) v = silu_f(v);
+        if (p.silu) v = silu_for<T>(v);
         vs[c] = to_f32(from_f32<T>(v));
     }
     __syncthreads();                              // (every thread has read m)
@@ -688,8 +730,11 @@ LCU_API int lcu_decay_scan(const void *rows, int type, int row_stride, int q_off
     if (gated) {
         float *la = gates, *b = gates + (size_t)heads * n;
         m = b + (size_t)heads * n;
-        ds_gates_kernel<<<dim3(heads, n_req), dim3(256), 0, stream>>>(z, ldz, bias_i, bias_f, cap, state, (size_t)slot_stride,
-                                                                      p.n_off + (size_t)heads * d, la, b, m, q_start, ctx_len, state_slot, n, heads);
+#define GATES(THREADS) ds_gates_kernel<THREADS><<<dim3(heads, n_req), dim3(THREADS), 0, stream>>>(z, ldz, bias_i, bias_f, cap, state, (size_t)slot_stride, \
+                                                                  p.n_off + (size_t)heads * d, la, b, m, q_start, ctx_len, state_slot, n, heads)
+        if (n > 256) GATES(1024);
+        else GATES(256);
+#undef GATES
         LCU_LAUNCH_CHECK();
         p.log_a = la;
         p.b = b;

@@ -51,27 +51,41 @@ LCU_API int lcu_embedding_gather(void *out, int out_type, const void *table, int
 }
 
 // ---------------------------------------------------------------- row gather
-template <class T>
-__global__ void gather_rows_kernel(T *__restrict__ out, const T *__restrict__ x,
-                                   const int *__restrict__ rows, int d, int n_src) {
-    const int r = rows[blockIdx.x];
-    T *o = out + (size_t)blockIdx.x * d;
+// V neighbouring elements a thread, the row shared out over blockIdx.y (few rows are gathered, often one: what counts is that all of
+// it is on its way at once).
+template <class T, int V>
+__global__ void __launch_bounds__(256)
+gather_rows_kernel(T *__restrict__ out, const T *__restrict__ x, const int *__restrict__ rows, int d, int n_src) {
+    struct alignas(V * sizeof(T)) Piece { T v[V]; };
+    const int r = rows[blockIdx.x], c = (blockIdx.y * 256 + threadIdx.x) * V;
+    if (c >= d) return;
+    Piece p;
     if (r < 0 || r >= n_src) {
-        for (int c = threadIdx.x; c < d; c += blockDim.x) o[c] = from_f32<T>(__uint_as_float(0x7fc00000u));
-        return;
+#pragma unroll
+        for (int e = 0; e < V; ++e) p.v[e] = from_f32<T>(__uint_as_float(0x7fc00000u));
+    } else {
+        p = *(const Piece *)(x + (size_t)r * d + c);
     }
-    const T *s = x + (size_t)r * d;
-    for (int c = threadIdx.x; c < d; c += blockDim.x) o[c] = s[c];
+    *(Piece *)(out + (size_t)blockIdx.x * d + c) = p;
 }
 
 LCU_API int lcu_gather_rows(void *out, const void *x, int type, const int *rows, int n_out, int d,
                             int n_src, hipStream_t stream) {
     if (n_out <= 0) return LCU_OK;
     if (d <= 0) return LCU_BAD_ARGUMENT;
-    dim3 grid(n_out), block(256);
-    if (type == LCU_F32) gather_rows_kernel<float><<<grid, block, 0, stream>>>((float *)out, (const float *)x, rows, d, n_src);
-    else if (type == LCU_BF16) gather_rows_kernel<bf16_t><<<grid, block, 0, stream>>>((bf16_t *)out, (const bf16_t *)x, rows, d, n_src);
+    const bool four = d % 4 == 0 && (uintptr_t)out % 16 == 0 && (uintptr_t)x % 16 == 0;
+    const int per = four ? 1024 : 256;
+    if ((d + per - 1) / per > 65535) return LCU_BAD_ARGUMENT;
+    dim3 grid(n_out, (d + per - 1) / per), block(256);
+#define GO(T)                                                                                                             \
+    do {                                                                                                                  \
+        if (four) gather_rows_kernel<T, 4><<<grid, block, 0, stream>>>((T *)out, (const T *)x, rows, d, n_src);           \
+        else gather_rows_kernel<T, 1><<<grid, block, 0, stream>>>((T *)out, (const T *)x, rows, d, n_src);                \
+    } while (0)
+    if (type == LCU_F32) GO(float);
+    else if (type == LCU_BF16) GO(bf16_t);
     else return LCU_BAD_ARGUMENT;
+#undef GO
     LCU_LAUNCH_CHECK();
     return LCU_OK;
 }

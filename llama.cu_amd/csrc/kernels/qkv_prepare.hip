@@ -265,7 +265,7 @@ qkv_prepare_rows_kernel(const TI *__restrict__ rows, int row_stride, int q_off, 
     struct alignas(V * sizeof(TI)) In { TI v[V]; };
     struct alignas(V * sizeof(T)) Out { T v[V]; };
     struct alignas(V * sizeof(float)) F32 { float v[V]; };
-    __shared__ float scratch[16], scratch_k[16];
+    __shared__ float sums[2][16];
     const int t = blockIdx.x, threads = blockDim.x, nq = nh * dh, nk = store_kv ? nkvh * dh : 0;
     const TI *row = rows + (size_t)t * row_stride;
     float sq = 0.f, sk = 0.f;
@@ -277,8 +277,13 @@ qkv_prepare_rows_kernel(const TI *__restrict__ rows, int row_stride, int q_off, 
         if (c < nq) sq += part;
         else sk += part;
     }
-    const float fq = rsqrtf(block_sum(sq, scratch) / (float)nq + eps);
-    const float fk = nk ? rsqrtf(block_sum(sk, scratch_k) / (float)nk + eps) : 0.f;
+    sq = wave_sum(sq);                            // both sums behind one barrier
+    sk = wave_sum(sk);
+    if (threadIdx.x % WAVE == 0) { sums[0][threadIdx.x / WAVE] = sq; sums[1][threadIdx.x / WAVE] = sk; }
+    __syncthreads();
+    sq = sk = 0.f;
+    for (int i = 0; i < threads / WAVE; ++i) { sq += sums[0][i]; sk += sums[1][i]; }
+    const float fq = rsqrtf(sq / (float)nq + eps), fk = nk ? rsqrtf(sk / (float)nk + eps) : 0.f;
     const int slot = store_kv ? slots[t] : -1, tok = slot < 0 ? 0 : slot % page;
     T *pg = slot < 0 ? nullptr : cache + (size_t)(slot / page) * kv_page_elems(nkvh, dhp, dvp, page);
     const int pos = cos_t ? positions[t] : 0, half = rot_dim / 2;

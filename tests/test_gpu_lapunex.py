@@ -190,7 +190,7 @@ def test_the_matrix_memory_against_its_recurrence(dtype, heads, dim, vdim, cap):
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("kind", ["lightning", "memory"])
 def test_long_portions_are_walked_in_runs(dtype, kind):
-    """Portions of 512 tokens and more are walked in runs side by side and chained: a long portion from the start beside a short
+    """Portions of 256 tokens and more are walked in runs side by side and chained: a long portion from the start beside a short
     request, a second long one that goes on from the first's state beside another that starts, then single tokens."""
     d = 40
     for shape in ([([0.99, 0.6], 32, 24), ([0.999], 130, 70)] if kind == "lightning" else [(2, 32, 24, 6.0), (1, 130, 70, 9.0)]):
