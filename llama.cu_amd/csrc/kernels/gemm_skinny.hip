@@ -36,13 +36,16 @@ typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
 typedef __attribute__((ext_vector_type(4))) float f32x4;
 typedef __attribute__((ext_vector_type(4))) uint32_t u32x4;
 
-enum { EPI_BF16 = 0, EPI_F32 = 1, EPI_ADD_F32 = 2, EPI_SWIGLU = 3, EPI_ADD_NORM = 4, EPI_QKV_ROPE = 5 };
+enum { EPI_BF16 = 0, EPI_F32 = 1, EPI_ADD_F32 = 2, EPI_SWIGLU = 3, EPI_ADD_NORM = 4, EPI_QKV_ROPE = 5, EPI_STREAMS = 6 };
 
 // What two epilogues need beside Y, so that no kernel stands between a projection that ends
 // a branch and the product that follows the next norm:
 //   EPI_ADD_NORM: Y is the float32 residual stream and takes the product in; the new rows times
 //     the norm's weight go to h_out as bfloat16, *not yet normalised*, and the workgroup's
 //     share of each row's sum of squares goes to sumsq_out[row][workgroup].
+//   EPI_STREAMS: the same for several residual streams side by side (Y [M, streams * N]): x_t <- sum_s mix[s, t] x_s + out_w[t] *
+//     product, all t at once, and h_out and sumsq_out are made of sum_s read[s] x_s (read null: ones).  The rows of X may wait for
+//     their normalisation.
 //   row scale (any other epilogue, sumsq_in not null): the rows of X are such rows; a row of
 //     the product is multiplied by rsqrt(sum of its shares / norm_width + eps) before the
 //     epilogue (the normalisation is a factor per row, so it commutes with the product).
@@ -75,6 +78,9 @@ struct SkinnyExtra {
     float res_scale;
     // EPI_SWIGLU: limit > 0 asks for the limited activation (gate_act.h)
     float act_alpha, act_limit;
+    // EPI_STREAMS
+    int streams;
+    const float *mix, *out_w, *read;
     // grouped products (group_rows 0: one matrix, one X)
     int group_rows;
     size_t x_group_stride;
@@ -314,6 +320,46 @@ gemm_skinny_kernel(const bf16_t *__restrict__ X, int ldx, const bf16_t *__restri
         }
         return;
     }
+    if (EPI == EPI_STREAMS) {
+        constexpr int MOST = 8;
+        const int S = ex.streams;
+#pragma unroll
+        for (int m = 0; m < MT; ++m) {
+            const int tok = 16 * m + l16;
+            float ss = 0.f;
+#pragma unroll
+            for (int t = 0; t < NT; ++t) {
+                const int c = n0 + 16 * t + 4 * grp;          // (N is a multiple of 4)
+                if (tok >= M || c >= N) continue;
+                float *res = (float *)Y + (size_t)tok * ldy + c;
+                f32x4 xs[MOST], u = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                for (int s = 0; s < MOST; ++s)
+                    if (s < S) xs[s] = *(const f32x4 *)(res + (size_t)s * N);
+#pragma unroll
+                for (int to = 0; to < MOST; ++to) {
+                    if (to >= S) break;
+                    f32x4 n = acc[t][m] * ex.out_w[to];
+#pragma unroll
+                    for (int s = 0; s < MOST; ++s)
+                        if (s < S) n += ex.mix[s * S + to] * xs[s];
+                    *(f32x4 *)(res + (size_t)to * N) = n;
+                    u += (ex.read ? ex.read[to] : 1.f) * n;
+                }
+                const f32x4 w = *(const f32x4 *)((const float *)ex.norm_w + c);
+#pragma unroll
+                for (int r = 0; r < 4; ++r) ss += u[r] * u[r];
+                uint2 h;
+                h.x = pack2_bf16(u[0] * w[0], u[1] * w[1]);
+                h.y = pack2_bf16(u[2] * w[2], u[3] * w[3]);
+                *(uint2 *)(ex.h_out + (size_t)tok * ex.ldh + c) = h;
+            }
+            ss += __shfl_xor(ss, 16, WAVE);               // every lane takes part: the others bring zero
+            ss += __shfl_xor(ss, 32, WAVE);
+            if (grp == 0 && tok < M) ex.sumsq_out[(size_t)tok * gridDim.x + blockIdx.x] = ss;
+        }
+        return;
+    }
     if (EPI == EPI_ADD_NORM) {
 #pragma unroll
         for (int m = 0; m < MT; ++m) {
@@ -390,6 +436,9 @@ static int launch_epi(const void *X, int ldx, const void *W, int ldw, void *Y, i
     case EPI_ADD_NORM:
         if constexpr (MT <= 2 && NT <= 2) { GO(EPI_ADD_NORM); break; }      // made for decoding: at most 32 rows
         return LCU_UNSUPPORTED;
+    case EPI_STREAMS:
+        if constexpr (MT <= 2 && NT <= 2) { GO(EPI_STREAMS); break; }
+        return LCU_UNSUPPORTED;
     case EPI_QKV_ROPE:
         if constexpr (MT <= 2 && NT == 2) {
             const dim3 rgrid((ex.heads + 2 * ex.kv_heads) * (ex.head_dim / 32));
@@ -461,7 +510,7 @@ static int skinny_bf16(const void *X, int ldx, const void *W, int ldw, void *Y, 
 
 LCU_API int lcu_gemm_skinny_bf16(const void *X, int ldx, const void *W, int ldw, void *Y, int ldy, int M, int N, int K,
                                  int epilogue, int tiles, int waves, int w_packed, float act_alpha, float act_limit, hipStream_t stream) {
-    if (epilogue == EPI_ADD_NORM) return LCU_BAD_ARGUMENT;
+    if (epilogue == EPI_ADD_NORM || epilogue == EPI_STREAMS) return LCU_BAD_ARGUMENT;
     SkinnyExtra ex = {};
     ex.act_alpha = act_alpha; ex.act_limit = act_limit;
     return skinny_bf16(X, ldx, W, ldw, Y, ldy, M, N, K, epilogue, tiles, waves, w_packed, ex, stream);
@@ -499,12 +548,30 @@ LCU_API int lcu_gemm_skinny_bf16_add_norm(const void *X, int ldx, const void *W,
     return skinny_bf16(X, ldx, W, ldw, res, ldres, M, N, K, EPI_ADD_NORM, tiles, waves, w_packed, ex, stream);
 }
 
+// The same between several residual streams: x [M, streams * N] (float32, rows ldx_s apart, N a multiple of 4); mix [streams, streams]
+// (from, to), out_w and read [streams] (read may be null), norm_w [N], all float32.  sumsq_in (may be null): the rows of X
+// wait for their normalisation.
+LCU_API int lcu_gemm_skinny_bf16_streams(const void *X, int ldx, const void *W, int ldw, float *x, int ldx_s, int streams, int M, int N, int K,
+                                         const float *mix, const float *out_w, const float *read, const float *norm_w, void *h_out, int ldh,
+                                         float *sumsq_out, int sumsq_cols, int tiles, int waves, int w_packed, const float *sumsq_in, int n_in,
+                                         int norm_width, float eps, hipStream_t stream) {
+    if (M > 32 || (tiles != 1 && tiles != 2) || !x || !mix || !out_w || !norm_w || !h_out || !sumsq_out || streams < 1 || streams > 8 || N % 4 ||
+        ldh < N || ldh % 4 || ldx_s < streams * N || ldx_s % 4 || (uintptr_t)x % 16 || (uintptr_t)norm_w % 16 || (uintptr_t)h_out % 8 ||
+        sumsq_cols != (N + 16 * tiles - 1) / (16 * tiles) || (sumsq_in && (n_in <= 0 || norm_width <= 0)))
+        return LCU_BAD_ARGUMENT;
+    SkinnyExtra ex = {};
+    ex.norm_w = norm_w; ex.norm_w_type = LCU_F32; ex.h_out = (bf16_t *)h_out; ex.ldh = ldh; ex.sumsq_out = sumsq_out;
+    ex.streams = streams; ex.mix = mix; ex.out_w = out_w; ex.read = read;
+    ex.sumsq_in = sumsq_in; ex.n_in = n_in; ex.norm_width = norm_width; ex.eps = eps;
+    return skinny_bf16(X, ldx, W, ldw, x, ldx_s, M, N, K, EPI_STREAMS, tiles, waves, w_packed, ex, stream);
+}
+
 // A product whose rows of X wait for their normalisation: row i of the product is multiplied by
 // rsqrt(sum(sumsq_in[i][0 .. n_in)) / norm_width + eps) before the epilogue (not EPI_ADD_NORM).
 LCU_API int lcu_gemm_skinny_bf16_scaled(const void *X, int ldx, const void *W, int ldw, void *Y, int ldy, int M, int N, int K,
                                         int epilogue, int tiles, int waves, int w_packed, const float *sumsq_in, int n_in,
                                         int norm_width, float eps, float act_alpha, float act_limit, hipStream_t stream) {
-    if (epilogue == EPI_ADD_NORM || !sumsq_in || n_in <= 0 || norm_width <= 0) return LCU_BAD_ARGUMENT;
+    if (epilogue == EPI_ADD_NORM || epilogue == EPI_STREAMS || !sumsq_in || n_in <= 0 || norm_width <= 0) return LCU_BAD_ARGUMENT;
     SkinnyExtra ex = {};
     ex.sumsq_in = sumsq_in; ex.n_in = n_in; ex.norm_width = norm_width; ex.eps = eps;
     ex.act_alpha = act_alpha; ex.act_limit = act_limit;

@@ -956,6 +956,42 @@ def gemm_skinny_add_norm(x: torch.Tensor, w: torch.Tensor, residual: torch.Tenso
     return h, sumsq
 
 
+def gemm_skinny_streams(x: torch.Tensor, w: torch.Tensor, streams: torch.Tensor, count: int, mix: torch.Tensor, out_weights: torch.Tensor,
+                        read: Optional[torch.Tensor], norm_weight: torch.Tensor, packed: bool = False, row_sumsq: Optional[torch.Tensor] = None,
+                        norm_width: int = 0, eps: float = 0.0):
+    """``gemm_skinny_add_norm`` between several residual streams (``streams [m, count * n]`` float32, in place): ``x_t = sum_s mix[s, t] x_s
+    + out_weights[t] * (x @ w.T)``, all at once; returns ``(h, sumsq)`` with ``h = bfloat16((sum_s read[s] x_s) * norm_weight)``, not
+    yet normalised (``read`` None: ones), and the shares of the rows' sums of squares.  ``row_sumsq``, ``norm_width``, ``eps``: the rows of ``x``
+    wait for their own normalisation (``gemm_skinny``).  The vectors are float32.  At most 32 rows."""
+    _gpu(x, w, streams, mix, out_weights, read, norm_weight, row_sumsq)
+    _rows(x, "skinny x"); _rows(w, "skinny w"); _rows(streams, "streams")
+    if packed and not (packable(w) and w.is_contiguous()):
+        raise KernelError("gemm_skinny_streams: a packed weight is a contiguous result of pack_weight")
+    m, k = x.shape
+    n = w.shape[0]
+    if w.shape[1] != k or m > ADD_NORM_MAX_ROWS or not skinny_supported(x, w, torch.float32) or n % 4:
+        raise KernelError(f"gemm_skinny_streams: x {tuple(x.shape)} {x.dtype} with w {tuple(w.shape)} {w.dtype} is not supported")
+    if not 1 <= count <= STREAMS_MAX or streams.dtype != torch.float32 or streams.shape != (m, count * n) or streams.stride(0) % 4:
+        raise KernelError(f"gemm_skinny_streams: the streams must be float32 {(m, count * n)} (at most {STREAMS_MAX})")
+    if mix.dtype != torch.float32 or mix.shape != (count, count) or not mix.is_contiguous():
+        raise KernelError(f"gemm_skinny_streams: the matrix between the streams must be contiguous float32 [{count}, {count}]")
+    _f32_vec(out_weights, "writing weights", count); _f32_vec(read, "reading weights", count); _f32_vec(norm_weight, "norm weight", n)
+    if row_sumsq is not None and (row_sumsq.dtype != torch.float32 or row_sumsq.dim() != 2 or row_sumsq.shape[0] != m
+                                  or not row_sumsq.is_contiguous() or norm_width <= 0):
+        raise KernelError("gemm_skinny_streams: row_sumsq must be a contiguous float32 [rows, parts] tensor, with the norm's width")
+    tiles = 1 if n <= TUNING.skinny_eight_waves_to else 2
+    waves = 8 if n <= TUNING.skinny_eight_waves_to else 4
+    parts = (n + 16 * tiles - 1) // (16 * tiles)
+    h = torch.empty((m, n), dtype=torch.bfloat16, device=x.device)
+    sumsq = torch.empty((m, parts), dtype=torch.float32, device=x.device)
+    lib = build.load("gemm_skinny")
+    _check(lib.lcu_gemm_skinny_bf16_streams(_ptr(x), x.stride(0), _ptr(w), w.stride(0), _ptr(streams), streams.stride(0), int(count), m, n, k,
+                                            _ptr(mix), _ptr(out_weights), _ptr(read), _ptr(norm_weight), _ptr(h), h.stride(0), _ptr(sumsq), parts,
+                                            tiles, waves, int(packed), _ptr(row_sumsq), 0 if row_sumsq is None else row_sumsq.shape[1],
+                                            int(norm_width), ctypes.c_float(eps), _stream()), "gemm_skinny_streams")
+    return h, sumsq
+
+
 MID_ADD_NORM_MAX_ROWS = 64
 
 

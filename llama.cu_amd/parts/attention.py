@@ -15,8 +15,8 @@ import torch
 
 from ..kernels import ops
 from .base import BuildContext, PagedKV, Part, PartSpec, ScaledRows, TensorSpec, make_part, register_part
-from .linear import (Weight, linear, linear_into_norm, linear_planes, linear_qkv_rope, linear_scaled, mid_qkv_takes, mid_takes,
-                     skinny_takes)
+from .linear import (Weight, end_in_norm, linear, linear_planes, linear_qkv_rope, linear_scaled, mid_qkv_takes, mid_takes,
+                     project, skinny_takes)
 from ..weights.loader import fused_rows
 
 
@@ -228,7 +228,7 @@ class Attention(Part):
         page_size = cache.page_size or self.page_size
         rot = self.position.rotary_tables()
         cos, sin, rot_dim, pairing = rot if rot is not None else (None, None, 0, 0)
-        rows = linear(h, self.w_in, out_dtype=torch.float32)
+        rows = project(h, self.w_in, torch.float32)
         if self.norm_eps is not None:
             q = ops.qkv_prepare_rows(rows, self.offsets, nh, nkv, self.head_dim, self.value_dim, self.stored_dim, self.stored_value_dim,
                                      self.dtype, self.q_norm, self.k_norm, self.norm_eps, positions=step.positions, cos=cos, sin=sin,
@@ -317,7 +317,8 @@ class Attention(Part):
         plain rows: only where the kernel for few rows is the faster one for the q, k, v
         product anyway."""
         if self.general:
-            return False
+            return (self.dtype == torch.bfloat16 and n_rows <= ops.ADD_NORM_MAX_ROWS
+                    and skinny_takes(n_rows, self.w_in, preferred=True))
         return self.dtype == torch.bfloat16 and n_rows <= ops.ADD_NORM_MAX_ROWS and skinny_takes(n_rows, self.w_qkv, preferred=True)
 
     def forward(self, h, step, cache, into=None, planes_ok=False, out_dtype=None, bias_later=False):
@@ -368,10 +369,9 @@ class Attention(Part):
         if out_dtype is not None and out_dtype != self.dtype:
             return linear(out, self.w_o, out_dtype=out_dtype)
         if into is not None:
-            residual, norm = into
-            fused = linear_into_norm(out, self.w_o, residual, norm.weight, scale=norm.delta_scale)
+            fused = end_in_norm(out, self.w_o, into)
             if fused is not None:
-                return ScaledRows(fused[0], fused[1], norm.size, norm.eps)
+                return fused
         if planes_ok and self.dtype == torch.bfloat16 and mid_takes(n_rows, self.w_o):
             return linear_planes(out, self.w_o)
         return linear(out, self.w_o, out_dtype=self.dtype)

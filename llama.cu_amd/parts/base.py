@@ -244,6 +244,18 @@ class StreamUpdate:
         return StreamUpdate(gather(self.delta), self.mix, self.out)
 
 
+@dataclass
+class StreamsEnd:
+    """What ``forward(..., into=)`` of a branch takes instead of ``(residual, norm)`` where there are several residual streams: the
+    branch's last product may let its output into them (``mix``, ``out`` as in ``StreamUpdate``) and return ScaledRows made with
+    ``norm`` of the sum of the streams weighted with ``read`` (None: ones)."""
+    x: torch.Tensor
+    norm: Any                   # parts.streams.StreamsNorm
+    read: Optional[torch.Tensor]
+    mix: torch.Tensor
+    out: torch.Tensor
+
+
 class Part:
     # Whether a step through this part may be captured into a graph and replayed: true only
     # if all it does is launch work on the current stream whose shape depends on the batch's
@@ -260,7 +272,7 @@ class Part:
     #        of partial sums as ``delta``;
     #        ``delta_scale``: what ``delta`` is multiplied by before it is added to the stream, also by a
     #        product that ends in this norm.
-    # mixer, feed-forward:  ``ends_in_norm``: ``forward(..., into=(residual, norm))`` may add its output to
+    # mixer, feed-forward:  ``ends_in_norm``: ``forward(..., into=(residual, norm))`` (or a StreamsEnd) may add its output to
     #        the residual stream itself and return ScaledRows made with ``norm``;
     #        ``ends_in_planes``: ``forward(..., planes_ok=True)`` may return float32 planes;
     #        ``takes_scaled_rows(n_rows)``: whether ``forward`` takes ScaledRows of that many rows;

@@ -22,14 +22,15 @@ import torch
 
 from ..kernels import ops
 from ..weights.loader import fused_rows
-from .base import BuildContext, Part, ScaledRows, SlotState, TensorSpec, register_part
-from .linear import Weight, finish, linear, linear_scaled, skinny_takes
+from .base import BuildContext, Part, ScaledRows, SlotState, StreamsEnd, TensorSpec, register_part
+from .linear import Weight, end_in_norm, finish, linear_scaled, project, skinny_takes
 
 
 class _DecayScan(Part):
     graph_safe = True
     splits_output = True
     ends_in_planes = True
+    ends_in_norm = True
     GATED = False
     IN = ()                       # the input matrices, in the order of their rows in the one product
 
@@ -70,10 +71,17 @@ class _DecayScan(Part):
             raise ops.KernelError("decay scan: the layer was given no state slots")
         return state
 
-    def forward(self, h, step, cache, out_dtype=None, planes_ok=False, state: Optional[torch.Tensor] = None):
-        out = torch.empty((h.shape[0], self.output_width), dtype=self.dtype, device=h.device)
+    def takes_scaled_rows(self, n_rows: int) -> bool:
+        return self.dtype == torch.bfloat16 and n_rows <= ops.ADD_NORM_MAX_ROWS and skinny_takes(n_rows, self.w_in, preferred=True)
+
+    def _operand(self, h):
+        rows = h.rows if isinstance(h, ScaledRows) else h
+        return torch.empty((rows.shape[0], self.output_width), dtype=self.dtype, device=rows.device)
+
+    def forward(self, h, step, cache, out_dtype=None, planes_ok=False, into=None, state: Optional[torch.Tensor] = None):
+        out = self._operand(h)
         self.forward_rows(h, step, cache, out, 1.0, state)
-        return finish(out, self.w_o, self.dtype, planes_ok=planes_ok, out_dtype=out_dtype)
+        return finish(out, self.w_o, self.dtype, into=into, planes_ok=planes_ok, out_dtype=out_dtype)
 
 
 class Lightning(_DecayScan):
@@ -98,22 +106,24 @@ class Lightning(_DecayScan):
         self.decay_vec = torch.tensor(self.decay, dtype=torch.float32, device=build.device)
 
     def _scan(self, h, step, cache, out, factor, state, scaled_rows=False):
-        rows = linear(h, self.w_in, out_dtype=self.dtype)
+        rows = project(h, self.w_in, self.dtype)
         return ops.decay_scan(rows, self.offsets, self._state(cache, state), step, self.heads, self.head_dim, self.value_dim, self.weight,
                               self.norm_eps, out, silu=True, factor=factor, decay=self.decay_vec, log_decay=self.log_decay, scaled_rows=scaled_rows)
 
     def forward_rows(self, h, step, cache, out, factor: float = 1.0, state: Optional[torch.Tensor] = None) -> None:
         self._scan(h, step, cache, out, factor, state)
 
-    def forward(self, h, step, cache, out_dtype=None, planes_ok=False, state: Optional[torch.Tensor] = None):
-        n = h.shape[0]
+    def forward(self, h, step, cache, out_dtype=None, planes_ok=False, into=None, state: Optional[torch.Tensor] = None):
+        n = step.n
         if step.decode_only and self.dtype == torch.bfloat16 and out_dtype in (None, self.dtype) and n <= ops.ADD_NORM_MAX_ROWS \
                 and skinny_takes(n, self.w_o, preferred=True):
             # few single tokens: the norm over the heads is a factor per row, which the output product applies
-            out = torch.empty((n, self.output_width), dtype=self.dtype, device=h.device)
+            out = self._operand(h)
             sumsq = self._scan(h, step, cache, out, 1.0, state, scaled_rows=True)
-            return linear_scaled(ScaledRows(out, sumsq, self.output_width, self.norm_eps), self.w_o, out_dtype=self.dtype)
-        return super().forward(h, step, cache, out_dtype=out_dtype, planes_ok=planes_ok, state=state)
+            scaled = ScaledRows(out, sumsq, self.output_width, self.norm_eps)
+            fused = end_in_norm(scaled, self.w_o, into) if isinstance(into, StreamsEnd) else None
+            return fused if fused is not None else linear_scaled(scaled, self.w_o, out_dtype=self.dtype)
+        return super().forward(h, step, cache, out_dtype=out_dtype, planes_ok=planes_ok, into=into, state=state)
 
 
 class MatrixMemory(_DecayScan):
@@ -146,10 +156,10 @@ class MatrixMemory(_DecayScan):
 
     def forward_rows(self, h, step, cache, out, factor: float = 1.0, state: Optional[torch.Tensor] = None) -> None:
         if step.decode_only or self.dtype == torch.float32:
-            both = linear(h, self.w_in, out_dtype=torch.float32)
+            both = project(h, self.w_in, torch.float32)
             rows, gates = both[:, :self.in_rows], both[:, self.in_rows:]
         else:
-            rows, gates = linear(h, self.w_rows, out_dtype=self.dtype), linear(h, self.w_gates, out_dtype=torch.float32)
+            rows, gates = project(h, self.w_rows, self.dtype), project(h, self.w_gates, torch.float32)
         ops.decay_scan(rows, self.offsets, self._state(cache, state), step, self.heads, self.head_dim, self.value_dim, self.weight, self.norm_eps,
                        out, scale=self.query_scale, factor=factor, gates=gates, gate_bias=self.gate_bias, cap=self.gate_cap)
 

@@ -15,7 +15,7 @@ import torch
 from ..kernels import ops
 from .base import BuildContext, Part, ScaledRows, TensorSpec, register_part
 from ..weights.loader import fused_rows
-from .linear import (Weight, library_friendly_rows, linear, linear_into_norm, linear_planes, linear_swiglu,
+from .linear import (Weight, end_in_norm, library_friendly_rows, linear, linear_planes, linear_swiglu,
                      linear_swiglu_mid, mid_swiglu_takes, mid_takes, skinny_row_limit, skinny_takes)
 
 
@@ -132,10 +132,9 @@ class SwiGLU(Part):
             return linear_planes(act, self.w_down)
         if into is not None and act.dtype == torch.bfloat16 and skinny_takes(act.shape[0], self.w_down, preferred=True):
             # only where the kernel for few rows is the faster one for this product anyway
-            residual, norm = into
-            fused = linear_into_norm(act, self.w_down, residual, norm.weight, scale=norm.delta_scale)
+            fused = end_in_norm(act, self.w_down, into)
             if fused is not None:
-                return ScaledRows(fused[0], fused[1], norm.size, norm.eps)
+                return fused
         return linear(act, self.w_down, out_dtype=self.dtype)
 
 

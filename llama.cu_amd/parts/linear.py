@@ -20,7 +20,7 @@ from typing import Optional, Union
 import torch
 
 from ..kernels import ops
-from .base import ScaledRows
+from .base import ScaledRows, StreamsEnd
 
 
 class Weight:
@@ -303,18 +303,37 @@ def project(h, weight: Union[torch.Tensor, Weight], dtype: torch.dtype) -> torch
     return linear(h, weight, out_dtype=dtype)
 
 
+def end_in_norm(a, weight: Union[torch.Tensor, Weight], into) -> Optional[ScaledRows]:
+    """A branch's last product with the residual sum and the next norm's weight in its epilogue: ``into = (residual, norm)``, or a
+    StreamsEnd for several residual streams; ``a``: rows, or (with a StreamsEnd) ScaledRows.  None if no kernel takes these operands
+    (then nothing has been done)."""
+    if not isinstance(into, StreamsEnd):
+        residual, norm = into
+        fused = linear_into_norm(a, weight, residual, norm.weight, scale=norm.delta_scale)
+        return None if fused is None else ScaledRows(fused[0], fused[1], norm.size, norm.eps)
+    rows = a.rows if isinstance(a, ScaledRows) else a
+    plain, packed = _split(weight)
+    norm = into.norm
+    if rows.dtype != torch.bfloat16 or plain.dtype != torch.bfloat16 or rows.shape[0] > ops.ADD_NORM_MAX_ROWS or norm.size % 4 \
+            or not ops.skinny_supported(rows, plain, torch.float32) or not skinny_takes(rows.shape[0], weight, preferred=True):
+        return None
+    kw = dict(row_sumsq=a.sumsq, norm_width=a.width, eps=a.eps) if isinstance(a, ScaledRows) else {}
+    h, sumsq = ops.gemm_skinny_streams(rows, plain if packed is None else packed, into.x, norm.streams, into.mix, into.out, into.read, norm.weight,
+                                       packed=packed is not None, **kw)
+    return ScaledRows(h, sumsq, norm.size, norm.eps)
+
+
 def finish(a: torch.Tensor, weight: Union[torch.Tensor, Weight], dtype: torch.dtype, into=None, planes_ok: bool = False,
            out_dtype: Optional[torch.dtype] = None):
-    """A branch's last product, ended as whoever called the branch allows: ``into = (residual, norm)``: the residual sum and that
+    """A branch's last product, ended as whoever called the branch allows: ``into`` (``end_in_norm``): the residual sum and the next
     norm's weight in its epilogue where a kernel for few rows takes it (ScaledRows); ``planes_ok``: float32 planes of
     partial sums where K is cut; else plain rows of ``out_dtype`` (``dtype``)."""
     if out_dtype is not None and out_dtype != dtype:
         return linear(a, weight, out_dtype=out_dtype)
     if into is not None:
-        residual, norm = into
-        fused = linear_into_norm(a, weight, residual, norm.weight, scale=norm.delta_scale)
+        fused = end_in_norm(a, weight, into)
         if fused is not None:
-            return ScaledRows(fused[0], fused[1], norm.size, norm.eps)
+            return fused
     if planes_ok and dtype == torch.bfloat16 and mid_takes(a.shape[0], weight):
         return linear_planes(a, weight)
     return linear(a, weight, out_dtype=dtype)

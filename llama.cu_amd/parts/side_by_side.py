@@ -11,7 +11,7 @@ from typing import Dict, Sequence
 import torch
 
 from ..kernels import ops
-from .base import BuildContext, Part, PartSpec, SeveralNeeds, TensorSpec, make_part, prefixed, register_part
+from .base import BuildContext, Part, PartSpec, ScaledRows, SeveralNeeds, TensorSpec, make_part, prefixed, register_part
 from .linear import Weight, finish
 
 
@@ -68,19 +68,28 @@ class SideBySide(Part):
     def decode_splits(self, batch: int, max_ctx_len: int) -> int:
         return max(int(m.decode_splits(batch, max_ctx_len)) for m in self.mixers)
 
+    # (with one product for all: it ends as a single mixer's would)
     @property
     def ends_in_planes(self):
         return self.joint
 
-    def forward(self, h, step, cache, out_dtype=None, planes_ok=False):
+    @property
+    def ends_in_norm(self):
+        return self.joint
+
+    def takes_scaled_rows(self, n_rows: int) -> bool:
+        return self.joint and all(m.takes_scaled_rows(n_rows) for m in self.mixers)
+
+    def forward(self, h, step, cache, out_dtype=None, planes_ok=False, into=None):
         if self.joint:
-            both = torch.empty((h.shape[0], self.w_o.shape[1]), dtype=self.dtype, device=h.device)
+            n = (h.rows if isinstance(h, ScaledRows) else h).shape[0]
+            both = torch.empty((n, self.w_o.shape[1]), dtype=self.dtype, device=self.w_o.plain.device)
             at = 0
             for i, (m, scale) in enumerate(zip(self.mixers, self.scales)):
                 state = cache.more.get(self._state_of.get(i))
                 m.forward_rows(h, step, cache, both[:, at:at + m.output_width], scale, state=state)
                 at += m.output_width
-            return finish(both, self.w_o, self.dtype, planes_ok=planes_ok, out_dtype=out_dtype)
+            return finish(both, self.w_o, self.dtype, into=into, planes_ok=planes_ok, out_dtype=out_dtype)
         total = None
         for i, (m, scale) in enumerate(zip(self.mixers, self.scales)):
             kw = {}

@@ -5,18 +5,19 @@ A sublayer reads a weighted sum of the streams and writes through a matrix betwe
     u = sum_s in[s] x_s,   y = f(norm(u)),   x_t <- sum_s mix[s, t] x_s + out[t] y        (all t at once from the old x)
 
 ``StreamsNorm`` makes ``norm(u)`` (without ``in``: of the sum of the streams, behind the last sublayer) and on its way there lets the
-last sublayer's output into the streams: ``pending`` between these parts is a ``StreamUpdate``, the output with the matrix and the weights
+last sublayer's output into the streams (a product of few rows may do both in its epilogue: ``StreamsEnd``): ``pending`` between these parts is a ``StreamUpdate``, the output with the matrix and the weights
 that it enters by, and the one kernel (``ops.streams_norm``) reads and writes every stream once between two sublayers.  ``StreamsBlock``
 is the arrangement of a mixer and a feed-forward in one layer.
 """
 from __future__ import annotations
 
+from dataclasses import dataclass
 from typing import Dict, Optional
 
 import torch
 
 from ..kernels import ops
-from .base import BuildContext, Part, PartSpec, StreamUpdate, TensorSpec, make_part, register_part
+from .base import BuildContext, Part, PartSpec, ScaledRows, StreamUpdate, StreamsEnd, TensorSpec, make_part, register_part
 from .block import _SublayersInTurn
 
 
@@ -24,6 +25,7 @@ class StreamsNorm(Part):
     """RMS norm of a weighted sum of the streams.  ``tensor``, ``one_plus``: as ``rmsnorm``."""
     graph_safe = True
     takes_planes = True
+    deferrable = True            # a product may end in it (``StreamsEnd``): a factor per row times a weight per column, of the weighted sum
 
     def __init__(self, size: int, eps: float, streams: int, tensor: str = "weight", one_plus: bool = False):
         self.size, self.eps, self.streams = int(size), float(eps), int(streams)
@@ -47,6 +49,13 @@ class StreamsNorm(Part):
                                 write_back=write_back)
 
 
+@dataclass(frozen=True)
+class StreamsRead:
+    """A norm with the weights that its sum of the streams is made with: what a block may end in."""
+    norm: StreamsNorm
+    read: Optional[torch.Tensor]
+
+
 class StreamsBlock(_SublayersInTurn):
     """A mixer and a feed-forward (which may be missing, with its norm) between several residual streams.  ``connections``: under
     which names the two sublayers' tensors ``in [streams]``, ``out [streams]`` and ``mix [streams, streams]`` (from, to) lie."""
@@ -54,6 +63,7 @@ class StreamsBlock(_SublayersInTurn):
     CHILDREN = ("norm1", "mixer", "norm2", "ffn")
     takes_planes = True          # ``pending``'s output may be float32 planes of partial sums
     ends_in_planes = True        # forward takes ``planes_ok``
+    ends_in_next_norm = True     # forward takes ``next_norm`` (a StreamsRead, or a StreamsNorm of the plain sum)
 
     def __init__(self, streams: int, norm1: PartSpec, mixer: PartSpec, norm2: Optional[PartSpec] = None, ffn: Optional[PartSpec] = None,
                  connections=("connection1", "connection2")):
@@ -84,17 +94,41 @@ class StreamsBlock(_SublayersInTurn):
         super().load(tensors, build)
         self.connections = [{k: tensors[f"{name}.{k}"].float().contiguous() for k in ("in", "out", "mix")} for name in self.names]
 
+    @property
+    def first_norm(self):
+        return StreamsRead(self.norm1, self.connections[0]["in"])
+
+    def takes_scaled_rows(self, n_rows: int) -> bool:
+        """Whether ``pending`` may be ScaledRows of so many rows made with ``first_norm``."""
+        return self.mixer.takes_scaled_rows(n_rows)
+
     def forward(self, x: torch.Tensor, pending, step, cache, next_norm=None, planes_ok=False):
         first = self.connections[0]
-        h = self.norm1.forward(x, pending, first["in"])
-        later = {"planes_ok": True} if self.mixer.ends_in_planes and (self.ffn is not None or planes_ok) else {}
-        pending = StreamUpdate(self.mixer.forward(h, step, cache, **later), first["mix"], first["out"])
-        if self.ffn is None:
-            return pending
-        second = self.connections[1]
-        h = self.norm2.forward(x, pending, second["in"])
-        later = {"planes_ok": True} if planes_ok and self.ffn.ends_in_planes else {}
-        return StreamUpdate(self.ffn.forward(h, **later), second["mix"], second["out"])
+        h = pending if isinstance(pending, ScaledRows) else self.norm1.forward(x, pending, first["in"])
+        n_rows = x.shape[0]
+        inner = self.ffn is not None
+        ahead = None if next_norm is None else next_norm if isinstance(next_norm, StreamsRead) else StreamsRead(next_norm, None)
+        second = self.connections[1] if inner else None
+        if inner:                # what the mixer may end in: the second norm, if the feed-forward takes such rows
+            target = StreamsRead(self.norm2, second["in"]) if self.ffn.takes_scaled_rows(n_rows) else None
+        else:
+            target = ahead
+        h = self._ended(x, self.mixer, (h, step, cache), target, inner or planes_ok, first)
+        if not inner:
+            return h
+        if not isinstance(h, ScaledRows):
+            h = self.norm2.forward(x, h, second["in"])
+        return self._ended(x, self.ffn, (h,), ahead, planes_ok, second)
+
+    @staticmethod
+    def _ended(x, part, args, target: Optional[StreamsRead], planes_ok: bool, connection):
+        """The output of ``part``: on its way into the streams (StreamUpdate), or, where its last product ended in the norm
+        ``target``, in them already (ScaledRows)."""
+        kw = {"planes_ok": True} if planes_ok and part.ends_in_planes else {}
+        if target is not None and part.ends_in_norm:
+            kw["into"] = StreamsEnd(x, target.norm, target.read, connection["mix"], connection["out"])
+        out = part.forward(*args, **kw)
+        return out if isinstance(out, ScaledRows) else StreamUpdate(out, connection["mix"], connection["out"])
 
 
 register_part("norm", "streams_rmsnorm", StreamsNorm)

@@ -70,6 +70,33 @@ def test_streams_refuse_what_does_not_fit():
             ops.streams_norm(x, bad.pop("streams", 3), w, 1e-5, torch.float32, **bad)
 
 
+@pytest.mark.parametrize("rows,packed,waits", [(3, True, False), (16, False, True), (29, True, True), (32, False, False)])
+@pytest.mark.parametrize("streams", [1, 3, 4, 7])
+def test_a_product_that_ends_in_the_streams_and_the_next_norm(rows, packed, waits, streams):
+    from llama_cu_amd.kernels import ops
+    n, k, eps = 192, 256, 1e-5
+    x, w = rnd(rows, k, seed=1).bfloat16(), rnd(n, k, seed=2, std=0.1).bfloat16()
+    X, mix, inn, out_w, nw = rnd(rows, streams, n, seed=3), rnd(streams, streams, seed=4), rnd(streams, seed=5), rnd(streams, seed=6), rnd(n, seed=7)
+    y = f64(x.float()) @ f64(w.float()).T
+    kw = {}
+    if waits:                                                # the rows' own norm is a factor that the product applies
+        shares = (x.float() ** 2).reshape(rows, 8, k // 8).sum(-1).contiguous()
+        kw = dict(row_sumsq=shares.cuda(), norm_width=k, eps=eps)
+        y = P.rms_div(f64(x.float()), eps) @ f64(w.float()).T
+    want = P.update_streams(f64(X), f64(mix), f64(out_w), y)
+    wg = ops.pack_weight(w.cuda()) if packed else w.cuda()
+    for read in (inn, None):
+        xs = X.reshape(rows, -1).cuda()
+        h, sumsq = ops.gemm_skinny_streams(x.cuda(), wg, xs, streams, mix.cuda(), out_w.cuda(), None if read is None else read.cuda(), nw.cuda(),
+                                           packed=packed, **kw)
+        u = P.read_streams(want, np.ones(streams) if read is None else f64(read))
+        assert_close(xs, want.reshape(rows, -1), 5e-6)
+        assert_close(h, u * f64(nw), 5e-3)
+        assert_close(sumsq.sum(1), (u ** 2).sum(1), 2e-5)
+    with pytest.raises(ops.KernelError):
+        ops.gemm_skinny_streams(x.cuda(), wg, xs, streams + 1, mix.cuda(), out_w.cuda(), None, nw.cuda(), packed=packed)
+
+
 def attention_part(m, dtype, page, d=64, eps=1e-5, seed=11):
     from llama_cu_amd.parts import PartSpec
     from llama_cu_amd.models.lapunex import ATTENTION_NAMES
@@ -571,6 +598,38 @@ def test_many_requests_decoding_together():
         assert_close(together[k], apart, SAME["bfloat16"], f"token {k}")
     plain = plain_logits(cfg, w, prompts[3] + tails[3])[-4:]
     assert_close(torch.stack([t[3] for t in together]), plain, REL["bfloat16"], "against the plain model")
+
+
+def test_few_rows_end_in_the_streams_within_their_products(monkeypatch):
+    """Single tokens and a short portion of a model whose feed-forwards are dense: every sublayer but those in front of experts ends
+    in the next norm, and the last one in the final norm."""
+    from llama_cu_amd.kernels import ops
+    cfg = config(96, 256, [
+        light(lightning([0.9, 0.99], 64, 64), dense(256)),
+        both(left(4, 2, 64, 64, 0.12, 64, 5000.0, yarn(4.0, 64, 8.0, 0.5)), right(2, 64, 64, 9.0), 0.7, 0.9, dense(512)),
+        light(lightning([0.95, 0.6], 64, 64))], eps=1e-6, streams=3, loop=(0, 2, 2))
+    w = random_weights(cfg, 22)
+    r = runner_for(make_folder(cfg, w), "bfloat16")
+    r.use_graphs = False
+    toks = tokens_of(96, 40, 60)
+    want = plain_logits(cfg, w, toks)
+    calls, real = [], ops.gemm_skinny_streams
+
+    def counted(*a, **kw):
+        calls.append(kw.get("row_sumsq") is not None)
+        return real(*a, **kw)
+
+    monkeypatch.setattr(ops, "gemm_skinny_streams", counted)
+    got = []
+    for at in range(0, 30, 6):
+        calls.clear()
+        got.append(r.step([0], [toks[at:at + 6]], [list(range(6))]).clone())
+        assert len(calls) == 9 and not any(calls)            # (a portion: the lightning layers' norm is made by their own kernel)
+    for t in toks[30:]:
+        calls.clear()
+        got.append(r.step([0], [[t]], [[0]]).clone())
+        assert len(calls) == 9 and sum(calls) == 3
+    assert_close(torch.cat(got), want, REL["bfloat16"])
 
 
 def test_logits_do_not_depend_on_the_cut_or_the_batch_in_32_bit():
