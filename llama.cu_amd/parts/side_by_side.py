@@ -23,11 +23,11 @@ class SideBySide(Part):
         self.mixers = [make_part("mixer", m) for m in mixers]
         self.scales = [float(x) for x in scales]
         self.graph_safe = all(m.graph_safe for m in self.mixers)
-        # under which name each mixer with a need finds a state of its own in the one LayerCache (SeveralNeeds)
         self.joint = all(m.splits_output for m in self.mixers)
         if self.joint:
             for m in self.mixers:
                 m.own_output = False
+        # under which name each mixer with a need finds a state of its own in the one LayerCache (SeveralNeeds)
         self._state_of, kept = {}, 0
         for i, m in enumerate(self.mixers):
             if m.cache_need() is not None:
